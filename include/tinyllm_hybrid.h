@@ -21,6 +21,8 @@
  *                      before it), one gate number per head (gated 2), and differential attention (diff_maps): every head has two
  *                      query / key maps [map 1 | map 2] over the same values, each an attention of its own; the read-outs combine
  *                      as a1 - lambda a2, are divided by their RMS over vdim and multiplied by 1 - diff_init.
+ *                      Also: scores capped by softcap tanh(s / softcap), a distance bias taken off the scores (bias_slope_dev[h] times
+ *                      the distance between query and key), and a query temperature 1 + q_temp_coef ln(floor((p + 1) / q_temp_every) + 1).
  *   TL_MIX_DELTA       gated delta rule: a [key_dim, value_dim] float32 state per head that decays, is corrected
  *                      towards the new value along the new key and is read with the query; q/k/v pass a short
  *                      causal depthwise convolution + SiLU first.  The state and the convolution's last inputs
@@ -35,22 +37,29 @@
  *                      read-out is unit-RMS per head, times a [heads*vdim] weight, gated by a sigmoid.
  *                      rec_kind TL_REC_FIXED: one constant decay per head (decay_dev), b = 1, no normaliser (retention); q and k
  *                      may carry rotary positions on their first rot_dims dimensions and k (not q) is scaled by dim^-1/2; the
- *                      read-out is unit-RMS per head without a weight (out_norm_dev NULL) and gated by SiLU.
+ *                      read-out is unit-RMS per head without a weight (out_norm_dev NULL) and gated by SiLU.  Options: SiLU on q, k and v
+ *                      (rec_silu), no scale on k (rec_plain_k), the read-out of all heads normed together with a [heads*vdim] weight
+ *                      (rec_joint_norm), a sigmoid gate (rec_sigmoid_gate) -- lightning attention has all four.
  *                      State (and m) live in the state slot of the sequence.
- *   TL_MIX_LATENT      latent attention: queries through a normed low-rank latent; keys and values are per-head
+ *   TL_MIX_LATENT      latent attention: queries through a normed low-rank latent (q_rank 0: directly); keys and values are per-head
  *                      projections (W_uk, W_uv) of ONE normed latent c [kv_rank] per token, plus one rotated key part
  *                      [rot_dim] shared by all heads; only (c | rotated part) is cached, one row per token.  The engine
  *                      runs it in absorbed form: q_h' = W_uk,h^T q_h, scores (q_h' . c + q_rot . k_rot) * scale, output
  *                      W_uv,h (sum_j p_j c_j) -- one K/V head of width kv_rank + rot_dim whose values are its leading
  *                      kv_rank columns.  Rotation frequencies may be rescaled (YaRN: rot_factor > 0).  kv_from >= 0: the
- *                      layer has no latent projection of its own and reads the pages of that earlier layer.
+ *                      layer has no latent projection of its own and reads the pages of that earlier layer.  Options: a sliding
+ *                      window (window), learned sinks (sink + sink_dev), one gate per head (gated 2).
+ *
+ * A layer may hold TWO mixers side by side (beside): both read the same normed input, their results are summed with the factors
+ * mix_scale.  Their projections share one input product and their output projections one output product.
  *
  * Block forms: parallel_block 1 is x += m (mixer(h) + ff(h)) with one norm; 0 is the sequential pre-norm block
  * x += ls1 * mixer(norm1 x); x += ls2 * ff(norm2 x) with optional per-channel scales ls1 / ls2; 2 is the block with the norm on
  * the branch's OUTPUT, x += m norm1(mixer(x)); x += m norm2(ff(x)), whose sublayers read the stream itself; 3 has a norm on both sides
  * of every sublayer, x += m ls1 post1(mixer(norm1 x)); x += m ls2 post2(ff(norm2 x)).  A layer may end with a per-layer token input
  * (side_*): e = the layer's columns of a second embedding table, y = W_proj (gelu_tanh(W_gate x) * e), x += y / rms(y) * side_norm.
- * The embedding output may pass an RMS norm (embed_norm_dev).  Norms: RMS or
+ * The embedding output may pass an RMS norm (embed_norm_dev); a second table indexed by a hash of the token and the one before it may
+ * be added to it first (pair_embed_dev).  Norms: RMS or
  * Dynamic Tanh (tanh(alpha x) w + b).  Feed-forward kinds: W_down act(W_up h), W_down (act(W_gate h) * W_up h), or a
  * mixture of experts (softmax or sigmoid router with a selection-only correction, groups of neighbouring experts, identity
  * experts, a shared expert with or without a scalar gate; experts W_down act(W_up h) or, with moe_gated, W_down (act(W_gate h) *
@@ -87,7 +96,7 @@ enum { TL_MIX_ATTENTION = 0, TL_MIX_DELTA = 1, TL_MIX_LINREC = 2, TL_MIX_LATENT 
 enum { TL_REC_CHANNEL = 0, TL_REC_EXPGATE = 1, TL_REC_FIXED = 2 };
 enum { TL_NORM_RMS = 0, TL_NORM_DYT = 1 };
 enum { TL_FF_PLAIN = 0, TL_FF_GATED = 1, TL_FF_MOE = 2 };
-enum { TL_ROUTER_SOFTMAX = 0, TL_ROUTER_SIGMOID = 1 };
+enum { TL_ROUTER_SOFTMAX = 0, TL_ROUTER_SIGMOID = 1, TL_ROUTER_CHOSEN_SOFTMAX = 2 };
 enum { TL_BLOCK_SEQUENTIAL = 0, TL_BLOCK_PARALLEL = 1, TL_BLOCK_POSTNORM = 2, TL_BLOCK_SANDWICH = 3 };
 enum { TL_VMIX_NONE = 0, TL_VMIX_FIRST = 1, TL_VMIX_BLEND = 2 };
 enum { TL_ACT_GELU_ERF = 0, TL_ACT_GELU_TANH = 1, TL_ACT_SILU = 2, TL_ACT_RELU2 = 3 };
@@ -100,7 +109,9 @@ enum { TL_HY_F32 = 0, TL_HY_BF16 = 2 }; /* the values of tl_dtype in tinyllm_hip
  *   delta:     q (kv_heads*dim) | k (kv_heads*dim) | v (heads*vdim) | gate (heads*vdim) | a (heads) | b (heads) | up (ff)
  *   linrec:    q (heads*dim) | k (heads*dim) | v (heads*vdim) | gate (heads*vdim) | expgate: i (heads) | f (heads)
  *                                                                                    | channel: a1 (a_rank) | fixed: nothing
- *   latent:    dq (q_rank) | dkv (kv_rank + rot_dim, unless kv_from >= 0) | gate (heads*vdim, if gated)
+ *   latent:    dq (q_rank; q_rank 0: q itself, heads*(dim + rot_dim), per head [dim | rot_dim]) | dkv (kv_rank + rot_dim, unless kv_from >= 0)
+ *              | gate (heads*vdim if gated 1, heads if gated 2)
+ *   beside:    the rows of the layer's own mixer, then those of the second mixer; w_out likewise by columns (heads*vdim of each)
  * w_out: [width, heads*vdim + ff]: the mixer's output projection beside the feed-forward's down projection, so
  *   one product yields mixer(h) + ff(h).
  * Sequential block (parallel_block 0): w_in / w_out hold the mixer's rows / columns only; the feed-forward reads
@@ -115,7 +126,7 @@ typedef struct tl_hybrid_layer {
     int kind;
     int heads, kv_heads, dim, vdim;
     int ff;                 /* 0: no feed-forward */
-    int ff_act;             /* 0 exact (erf) GELU, 1 tanh GELU, 2 SiLU */
+    int ff_act;             /* 0 exact (erf) GELU, 1 tanh GELU, 2 SiLU, 3 squared ReLU */
     const void *w_in_dev, *w_out_dev;
     const float *norm_dev;  /* [width] pre-norm weight */
     float norm_offset;      /* weight is applied as (norm_offset + w): 1 for weights stored around zero */
@@ -172,7 +183,7 @@ typedef struct tl_hybrid_layer {
                                before they are cached */
     float v_mix_lambda;
     /* mixture of experts, further options */
-    int moe_router;         /* TL_ROUTER_*: scores softmax(z) or sigmoid(z) */
+    int moe_router;         /* TL_ROUTER_*: scores softmax(z) or sigmoid(z); 2: the top logits z, weights = softmax over the chosen ones */
     int moe_gated;          /* experts (and the shared one) are W_down (act(W_gate h) * W_up h) */
     int moe_scale_input;    /* the router's weight multiplies the expert's input: expert(w h) */
     int moe_shared_sg;      /* the shared expert is scaled by sigmoid of a scalar projection (its row follows the router's) */
@@ -192,6 +203,16 @@ typedef struct tl_hybrid_layer {
     const void *side_proj_dev;  /* [width, side_dim] engine dtype */
     const float *side_norm_dev; /* [width], plain weight */
     int side_col0;              /* first of the layer's side_dim columns in the side embedding table */
+    /* attention, further options (3): score = cap(q.k * scale) - slope[h] * (i - j) */
+    float softcap;              /* > 0: s <- softcap tanh(s / softcap) */
+    const float *bias_slope_dev; /* [heads] distance bias; NULL: none */
+    float q_temp_coef, q_temp_every; /* coef != 0: q *= 1 + coef ln(floor((p + 1) / every) + 1) */
+    /* constant-decay recurrence, further options */
+    int rec_silu, rec_plain_k, rec_joint_norm, rec_sigmoid_gate;
+    const float *router_bias_dev; /* [experts + identity] added to the router's logits; NULL: none */
+    /* a second mixer on the same input: its kind, sizes, options and vectors (matrices of the layer itself are not read from it) */
+    const struct tl_hybrid_layer *beside;
+    float mix_scale;            /* factor on this mixer's result (0 is read as 1) */
 } tl_hybrid_layer;
 
 typedef struct tl_hybrid_config {
@@ -216,6 +237,10 @@ typedef struct tl_hybrid_config {
     const float *embed_norm_dev; /* [width]: x = rms_norm(embed[token] * embed_scale) * (final_norm_offset + w); NULL: none */
     const void *side_embed_dev;  /* [vocab, side_cols] engine dtype: the table of the per-layer token inputs */
     int side_cols, side_dim;     /* columns of a table row; columns one layer reads */
+    const void *pair_embed_dev;  /* [pair_buckets + 1, width] engine dtype: x += row (previous token * pair_mul_prev + token * pair_mul_cur) mod
+                                    pair_buckets, row pair_buckets for a sequence's first token; NULL: none */
+    int64_t pair_buckets, pair_mul_prev, pair_mul_cur;
+    float logit_softcap;         /* > 0: logits <- logit_softcap tanh(logits / logit_softcap), after logit_scale */
 } tl_hybrid_config;
 
 typedef struct tl_hybrid_stats {

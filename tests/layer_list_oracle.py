@@ -868,3 +868,223 @@ def muduvik_config(layers, width=64, vocab=101, eps=1e-5, loop=None, side=8):
     if side:
         cfg["token_side"] = {"dim": side}
     return cfg
+
+
+# ---- Karorax: x = embed[token] + bigram row; sequential pre-norm blocks (RMS norms with weights around zero, layer scales).  Mixers: latent
+# ---- attention with direct queries, a sliding window, learned sinks and one gate per head; two mixers side by side on one input (capped
+# ---- attention with a distance bias and a query temperature beside a constant-decay recurrence).  Same conventions as above. ----------------
+
+def bigram_rows(tokens, mul_prev, mul_cur, buckets):
+    """Row of the pair table for every token of a sequence: (previous * mul_prev + token * mul_cur) mod buckets; `buckets` for the first one."""
+    rows = [buckets]
+    for a, b in zip(tokens[:-1], tokens[1:]):
+        rows.append((int(a) * int(mul_prev) + int(b) * int(mul_cur)) % int(buckets))
+    return rows
+
+
+def window_sink_attention(q, k, v, scale, window=None, sinks=None):
+    """q, k [L, H, D], v [L, H, V]: query i sees keys j with 0 <= i - j < window; the denominator also holds exp(sinks[h])."""
+    L, H, _ = q.shape
+    out = np.zeros((L, H, v.shape[2]))
+    for h in range(H):
+        for i in range(L):
+            lo = max(0, i - window + 1) if window else 0
+            s = (k[lo:i + 1, h] @ q[i, h]) * scale
+            top = s.max() if sinks is None else max(s.max(), sinks[h])
+            e = np.exp(s - top)
+            out[i, h] = (e / (e.sum() + (0.0 if sinks is None else math.exp(sinks[h] - top)))) @ v[lo:i + 1, h]
+    return out
+
+
+def distance_slopes(heads):
+    return np.array([2.0 ** (-8.0 * (h + 1) / heads) for h in range(heads)])
+
+
+def query_temperature(pos, coef, every):
+    """1 + coef * ln(floor((p + 1) / every) + 1) per position."""
+    return np.array([1.0 + coef * math.log(math.floor((p + 1) / every) + 1) for p in pos])
+
+
+def capped_bias_attention(q, k, v, scale, softcap=None, slopes=None):
+    """q [L, H, D], k [L, G, D], v [L, G, V]; causal.  s = cap tanh(q.k scale / cap), minus slopes[h] * (i - j), then an ordinary softmax."""
+    L, H, _ = q.shape
+    G = k.shape[1]
+    out = np.zeros((L, H, v.shape[2]))
+    for h in range(H):
+        g = h // (H // G)
+        for i in range(L):
+            s = (k[:i + 1, g] @ q[i, h]) * scale
+            if softcap:
+                s = softcap * np.tanh(s / softcap)
+            if slopes is not None:
+                s = s - slopes[h] * (i - np.arange(i + 1))
+            e = np.exp(s - s.max())
+            out[i, h] = (e / e.sum()) @ v[:i + 1, g]
+    return out
+
+
+def karorax_capped_attention(W, m, mc, h, pos):
+    L, H, G, D, V = h.shape[0], mc["heads"], mc["kv_heads"], mc["dim"], mc["vdim"]
+    q, k, v = (h @ W[m + "q"].T).reshape(L, H, D), (h @ W[m + "k"].T).reshape(L, G, D), (h @ W[m + "v"].T).reshape(L, G, V)
+    if mc.get("q_temp"):
+        q = q * query_temperature(pos, mc["q_temp"]["coef"], mc["q_temp"]["every"])[:, None, None]
+    return capped_bias_attention(q, k, v, mc["scale"], mc.get("softcap"), distance_slopes(H)).reshape(L, H * V) @ W[m + "o"].T
+
+
+def lightning_attention(W, m, mc, h, eps):
+    """silu on q, k and v; the constant-decay recurrence without any other scale; all heads normed together, sigmoid gate."""
+    L, H, D, V = h.shape[0], mc["heads"], mc["dim"], mc["vdim"]
+    q, k, v = silu(h @ W[m + "q"].T).reshape(L, H, D), silu(h @ W[m + "k"].T).reshape(L, H, D), silu(h @ W[m + "v"].T).reshape(L, H, V)
+    o = retention_states(q, k, v, np.asarray(mc["decay"], dtype=np.float64)).reshape(L, H * V)
+    return (rms_norm(o, W[m + "norm"], eps) * sigmoid(h @ W[m + "g"].T)) @ W[m + "o"].T
+
+
+def karorax_latent(W, m, mc, h, pos, eps, shared=None):
+    """Returns (result, (latent, rotated key part)).  ``shared``: the pair another layer computed (the layer has no down-projection of its own)."""
+    L, H, D, R, V, C = h.shape[0], mc["heads"], mc["dim"], mc["rot_dim"], mc["vdim"], mc["kv_rank"]
+    f = scaled_frequencies((mc.get("rot") or {}).get("dims", 0), (mc.get("rot") or {}).get("base", 1.0))[0] if R else []
+    q = (h @ W[m + "q"].T).reshape(L, H, D + R)
+    if shared is None:
+        down = h @ W[m + "dkv"].T
+        shared = (rms_norm(down[:, :C], W[m + "dkv.norm"], eps), rotate_pairs_by(down[:, None, C:], pos, f)[:, 0])
+    c, kr = shared
+    kp, v = (c @ W[m + "uk"].T).reshape(L, H, D), (c @ W[m + "uv"].T).reshape(L, H, V)
+    full_q = np.concatenate([q[..., :D], rotate_pairs_by(q[..., D:], pos, f)], -1)
+    full_k = np.concatenate([kp, np.repeat(kr[:, None], H, 1)], -1)
+    o = window_sink_attention(full_q, full_k, v, mc["scale"], (mc.get("mask") or {}).get("size"), W[m + "sink"])
+    o = o * sigmoid(h @ W[m + "g"].T)[:, :, None]
+    return o.reshape(L, H * V) @ W[m + "o"].T, shared
+
+
+def chosen_softmax_route(z, top):
+    """The `top` largest logits (ties: the lower index); weights = softmax over the chosen logits only.  {expert: weight}."""
+    chosen = sorted(range(len(z)), key=lambda j: (-z[j], j))[:top]
+    e = {j: math.exp(z[j] - z[chosen[0]]) for j in chosen}
+    return {j: e[j] / sum(e.values()) for j in chosen}
+
+
+def karorax_feed_forward(mlp, W, f, h):
+    if mlp["kind"] == "dense":
+        return relu2(h @ W[f + "up"].T) @ W[f + "down"].T
+    out = np.zeros_like(h)
+    z = h @ W[f + "router"].T + W[f + "router.b"]
+    for t in range(h.shape[0]):
+        for j, w in chosen_softmax_route(z[t], mlp["router"]["top"]).items():
+            out[t] += w * gated_expert(W, f + f"e{j}.", h[t])
+    if mlp.get("shared"):
+        out = out + gated_expert(W, f + "shared.", h)
+    return out
+
+
+def karorax_forward(config, W, tokens, streams=None):
+    """Logits [L, vocab] of a whole sequence; ``streams`` (a list) receives the residual stream after every layer."""
+    W = {k: np.asarray(v, dtype=np.float64) for k, v in W.items()}
+    eps = config["norm"]["eps"]
+    tokens = [int(t) for t in tokens]
+    pos = np.arange(len(tokens), dtype=np.float64)
+    x = W["embed"][np.asarray(tokens)]
+    big = (config.get("embedding") or {}).get("bigram")
+    if big:
+        x = x + W["bigram"][np.asarray(bigram_rows(tokens, big["mul_prev"], big["mul_cur"], big["buckets"]))]
+    latents = {}
+    for i, spec in enumerate(config["layers"]):
+        p, m, mc = f"l{i}.", f"l{i}.mix.", spec["mixer"]
+        h = rms_norm(x, W[p + "norm1"], eps, 1.0)
+        if spec["type"] == "latent_attention":
+            y, latents[i] = karorax_latent(W, m, mc, h, pos, eps, latents[mc["kv_from"]] if mc.get("kv_from") is not None else None)
+        elif spec["type"] == "parallel":
+            y = mc["left_scale"] * karorax_capped_attention(W, m + "left.", mc["left"], h, pos) + \
+                mc["right_scale"] * lightning_attention(W, m + "right.", mc["right"], h, eps)
+        else:
+            raise ValueError(spec["type"])
+        x = x + y * W[p + "ls1"]
+        if spec.get("mlp"):
+            x = x + karorax_feed_forward(spec["mlp"], W, p + "mlp.", rms_norm(x, W[p + "norm2"], eps, 1.0)) * W[p + "ls2"]
+        if streams is not None:
+            streams.append(x.copy())
+    logits = rms_norm(x, W["final.norm"], eps, 1.0) @ W["head"].T
+    cap = config.get("logit_softcap")
+    return cap * np.tanh(logits / cap) if cap else logits
+
+
+def make_karorax_weights(config, seed=0):
+    """Random bf16-representable weights by tensor name (float32 arrays) for a Karorax config dict."""
+    import torch
+
+    gen = torch.Generator().manual_seed(seed)
+    Wd, out = config["width"], {}
+
+    def mat(rows, cols, scale=None):
+        s = scale if scale is not None else cols ** -0.5
+        return (torch.randn(rows, cols, generator=gen) * s).to(torch.bfloat16).float().numpy()
+
+    def vec(n, scale=0.1, shift=0.0):
+        return (torch.randn(n, generator=gen) * scale + shift).to(torch.bfloat16).float().numpy()
+
+    out["embed"], out["head"], out["final.norm"] = mat(config["vocab"], Wd, 1.0), mat(config["vocab"], Wd), vec(Wd)
+    big = (config.get("embedding") or {}).get("bigram")
+    if big:
+        out["bigram"] = mat(big["buckets"] + 1, Wd, 0.7)
+    for i, spec in enumerate(config["layers"]):
+        p, m, mc = f"l{i}.", f"l{i}.mix.", spec["mixer"]
+        out[p + "norm1"], out[p + "ls1"] = vec(Wd), vec(Wd, 0.2, 0.6)
+        if spec["type"] == "latent_attention":
+            H, D, R, V, C = mc["heads"], mc["dim"], mc["rot_dim"], mc["vdim"], mc["kv_rank"]
+            out[m + "q"], out[m + "uk"], out[m + "uv"] = mat(H * (D + R), Wd), mat(H * D, C), mat(H * V, C)
+            out[m + "sink"], out[m + "g"], out[m + "o"] = vec(H, 1.0, 0.5), mat(H, Wd, 2.0 * Wd ** -0.5), mat(Wd, H * V)
+            if mc.get("kv_from") is None:
+                out[m + "dkv"], out[m + "dkv.norm"] = mat(C + R, Wd), vec(C, 0.1, 1.0)
+        else:
+            L, R = mc["left"], mc["right"]
+            for name, n in (("left.q", L["heads"] * L["dim"]), ("left.k", L["kv_heads"] * L["dim"]), ("left.v", L["kv_heads"] * L["vdim"]),
+                            ("right.q", R["heads"] * R["dim"]), ("right.k", R["heads"] * R["dim"]), ("right.v", R["heads"] * R["vdim"]),
+                            ("right.g", R["heads"] * R["vdim"])):
+                out[m + name] = mat(n, Wd)
+            out[m + "left.o"], out[m + "right.o"] = mat(Wd, L["heads"] * L["vdim"]), mat(Wd, R["heads"] * R["vdim"])
+            out[m + "right.norm"] = vec(R["heads"] * R["vdim"], 0.2, 1.0)
+        mlp = spec.get("mlp")
+        if mlp:
+            f = p + "mlp."
+            out[p + "norm2"], out[p + "ls2"] = vec(Wd), vec(Wd, 0.2, 0.6)
+            if mlp["kind"] == "dense":
+                out[f + "up"], out[f + "down"] = mat(mlp["ff"], Wd), mat(Wd, mlp["ff"])
+            else:
+                E = mlp["router"]["experts"]
+                out[f + "router"], out[f + "router.b"] = mat(E, Wd, 2.0 * Wd ** -0.5), vec(E, 0.5)
+                names = [(f"e{e}.", mlp["expert"]["ff"]) for e in range(E)] + ([("shared.", mlp["shared"]["ff"])] if mlp.get("shared") else [])
+                for name, n in names:
+                    out[f + name + "gate"], out[f + name + "up"], out[f + name + "down"] = mat(n, Wd), mat(n, Wd), mat(Wd, n)
+    return out
+
+
+def karorax_moe(experts=6, top=2, ff=24, shared=40):
+    mlp = {"kind": "moe", "expert": {"ff": ff}, "router": {"experts": experts, "top": top}}
+    if shared:
+        mlp["shared"] = {"ff": shared}
+    return mlp
+
+
+def karorax_latent_layer(heads=4, dim=16, vdim=24, rot_dim=8, kv_rank=40, base=5000.0, scale=0.2, window=20, kv_from=None, mlp="default"):
+    mixer = {"heads": heads, "dim": dim, "vdim": vdim, "rot_dim": rot_dim, "kv_rank": kv_rank, "rot": {"base": base, "dims": rot_dim}, "scale": scale}
+    if window:
+        mixer["mask"] = {"size": window}
+    if kv_from is not None:
+        mixer["kv_from"] = kv_from
+    return {"type": "latent_attention", "mixer": mixer, "mlp": karorax_moe() if mlp == "default" else mlp}
+
+
+def karorax_parallel_layer(heads=4, kv_heads=2, dim=16, vdim=24, scale=0.3, softcap=4.0, coef=0.25, every=16, right_heads=3, right_dim=12, right_vdim=16,
+                           decay=None, left_scale=0.9, right_scale=1.2, mlp="default"):
+    decay = list(decay) if decay is not None else [math.exp(-(2.0 ** -(1 + 2 * h))) for h in range(right_heads)]
+    mixer = {"left": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "scale": scale, "softcap": softcap, "q_temp": {"coef": coef, "every": every}},
+             "left_scale": left_scale, "right": {"heads": right_heads, "dim": right_dim, "vdim": right_vdim, "decay": decay}, "right_scale": right_scale}
+    return {"type": "parallel", "mixer": mixer, "mlp": {"kind": "dense", "ff": 72} if mlp == "default" else mlp}
+
+
+def karorax_config(layers, width=64, vocab=101, eps=1e-5, bigram=(53, 5, 3), logit_softcap=6.0):
+    cfg = {"architecture": "Karorax", "layers": layers, "norm": {"eps": eps}, "vocab": vocab, "width": width}
+    if bigram:
+        cfg["embedding"] = {"bigram": {"buckets": bigram[0], "mul_prev": bigram[1], "mul_cur": bigram[2]}}
+    if logit_softcap:
+        cfg["logit_softcap"] = logit_softcap
+    return cfg

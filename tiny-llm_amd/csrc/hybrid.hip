@@ -41,18 +41,22 @@ int qmm3_num_cus() {  // gemm8.hip sizes its persistent grid by the CU count
 }
 namespace hy {
 
-struct Run {
-    int layer = 0;
-    int pass = -1;            // loop pass this run belongs to, -1 outside the loop
-    bool enters_pass = false; // the loop-entry projection + pass offset come right before this run
+struct MixState {             // what one mixer of a layer run keeps per sequence
     void *kpool = nullptr, *vpool = nullptr;      // attention: [pages, G, page, dim] / [pages, G, page, vdim] of the engine dtype
     float *state = nullptr, *conv_state = nullptr; // delta: [slots, H, vdim, dim] / [slots, taps-1, C]
                                                    // linrec: [slots, H, vdim (+1), dim] / the gates' running maximum [slots, H]
     // latent: kpool = [pages, page, kv_rank + rot_dim] (vpool unused); with kv_from the pages of an earlier run (not owned)
 };
+struct Run {
+    int layer = 0;
+    int pass = -1;            // loop pass this run belongs to, -1 outside the loop
+    bool enters_pass = false; // the loop-entry projection + pass offset come right before this run
+    MixState mix[2];          // the layer's mixer, and the one beside it (if there is one)
+};
 
 struct Meta {  // device int32 arrays of one step
     int32_t *tokens, *row_seq, *row_pos, *seq_row0, *seq_slot, *want_rows, *want_slot;
+    int32_t *seq_prev;  // the token each sequence was fed last before the step (written on the device)
 };
 
 }  // namespace hy
@@ -61,9 +65,10 @@ struct Meta {  // device int32 arrays of one step
 struct tl_hybrid {
     tl_hybrid_config cfg{};
     std::vector<tl_hybrid_layer> layers;
+    std::vector<tl_hybrid_layer> beside;  // per layer: its second mixer (kind < 0: none)
     std::vector<tl::hy::Run> runs;
-    std::vector<float *> inv_freq;  // per layer (attention with rotary positions), device
-    std::vector<float> rot_mult;    // per layer: factor on cos and sin (rescaled frequencies)
+    std::vector<float *> inv_freq;  // per mixer (2 layer + 0 / 1; those with rotary positions), device
+    std::vector<float> rot_mult;    // per mixer: factor on cos and sin (rescaled frequencies)
     float *f32a = nullptr, *gates = nullptr, *idw = nullptr;  // [R, max_c] scratch (conv output, latent queries, channel decays); [R, H, 3]; [R]
     void *da = nullptr, *db = nullptr;                         // D-typed scratch rows: latents / low-rank inputs / attention read-out; plain queries
     hipStream_t stream = nullptr;
@@ -83,6 +88,7 @@ struct tl_hybrid {
     int32_t *meta_dev = nullptr, *meta_host = nullptr;  // step metadata (host side pinned)
     int32_t *dmeta_dev = nullptr;                        // decode-loop metadata (its own copy: captured graphs point into it)
     int32_t *ctx_dev = nullptr, *pending_dev = nullptr, *argmax_dev = nullptr;
+    int32_t *last_tok_dev = nullptr;                     // [slots] the token each sequence was fed last
     tl::hy::Meta meta{}, dmeta{};
     int last_rows = 0;
     // trace of the residual stream
@@ -107,7 +113,8 @@ static int mixer_cols(const tl_hybrid_layer &L) {  // rows of w_in that belong t
     if (L.kind == TL_MIX_ATTENTION) return attn_maps(L) * (L.heads + L.kv_heads) * L.dim + L.kv_heads * L.vdim + gate_cols(L);
     if (L.kind == TL_MIX_LINREC)
         return 2 * L.heads * L.dim + 2 * L.heads * L.vdim + (L.rec_kind == TL_REC_EXPGATE ? 2 * L.heads : (L.rec_kind == TL_REC_CHANNEL ? L.a_rank : 0));
-    if (L.kind == TL_MIX_LATENT) return L.q_rank + (L.kv_from < 0 ? L.kv_rank + L.rot_dim : 0) + (L.gated ? L.heads * L.vdim : 0);
+    if (L.kind == TL_MIX_LATENT)
+        return (L.q_rank ? L.q_rank : L.heads * (L.dim + L.rot_dim)) + (L.kv_from < 0 ? L.kv_rank + L.rot_dim : 0) + gate_cols(L);
     return 2 * L.kv_heads * L.dim + 2 * L.heads * L.vdim + 2 * L.heads;
 }
 static int ff_in_cols(const tl_hybrid_layer &L) {  // rows of the feed-forward's input matrix
@@ -116,6 +123,14 @@ static int ff_in_cols(const tl_hybrid_layer &L) {  // rows of the feed-forward's
     if (L.ff_kind == TL_FF_MOE && L.moe_gated) return (2 * L.ff + L.experts + L.identity + (L.moe_shared_sg ? 1 : 0) + 7) / 8 * 8;
     if (L.ff_kind == TL_FF_MOE) return (L.shared_ff + L.experts * L.expert_ff + L.experts + L.identity + 1 + 7) / 8 * 8;
     return L.ff;
+}
+// a layer's mixer and, if it has one, the mixer beside it: rows of w_in, columns of w_out
+static int layer_mixer_cols(const tl_hybrid *e, int layer) {
+    return mixer_cols(e->layers[layer]) + (e->beside[layer].kind >= 0 ? mixer_cols(e->beside[layer]) : 0);
+}
+static int layer_read_cols(const tl_hybrid *e, int layer) {
+    const tl_hybrid_layer &L = e->layers[layer], &B = e->beside[layer];
+    return L.heads * L.vdim + (B.kind >= 0 ? B.heads * B.vdim : 0);
 }
 static int conv_channels(const tl_hybrid_layer &L) { return 2 * L.kv_heads * L.dim + L.heads * L.vdim; }
 // floats of one sequence's recurrent state, and of what travels beside it (delta: the convolution's last inputs; expgate: the running maximum)
@@ -147,9 +162,10 @@ static Meta carve(int32_t *base, int R, int S) {
     m.want_slot = base + 4 * R;
     m.seq_row0 = base + 5 * R;
     m.seq_slot = base + 5 * R + S + 1;
+    m.seq_prev = base + 5 * R + 2 * S + 1;
     return m;
 }
-static size_t meta_ints(int R, int S) { return (size_t)5 * R + 2 * S + 2; }
+static size_t meta_ints(int R, int S) { return (size_t)5 * R + 3 * S + 2; }
 
 // a Dynamic Tanh norm that may leave with the product completing a residual sum (epilogue 4 of the row and 64-wide tile kernels)
 struct NormTail {
@@ -218,7 +234,7 @@ static int linear_t(const void *A, int lda, const void *W, float *out, int ldc, 
     return TL_OK;
 }
 
-static int launch_delta(const tl_hybrid *e, const tl_hybrid_layer &L, const Run &run, const Meta &m, int n_seqs, int ldp) {
+static int launch_delta(const tl_hybrid *e, const tl_hybrid_layer &L, const MixState &run, const Meta &m, int n_seqs, const float *proj, int ldp) {
     // LPC lanes per state column with RPT key rows each: key_dim <= LPC * RPT.  The token loop is a dependency chain whose cost per wave hardly
     // depends on RPT, so the fewest lanes per column that still give every SIMD a wave: 64 while the step's columns are at most the SIMDs, then 32, then
     // a DPP row of 16 (also for narrow keys)
@@ -232,7 +248,7 @@ static int launch_delta(const tl_hybrid *e, const tl_hybrid_layer &L, const Run 
     const int C = conv_channels(L);
     const int a0 = 2 * L.kv_heads * L.dim + 2 * L.heads * L.vdim, b0 = a0 + L.heads;
 #define HY_DELTA(RPT, LPC)                                                                                                                  \
-    hipLaunchKernelGGL((delta_kernel<RPT, LPC>), grid, block, 0, e->stream, e->f32a, C, e->proj, ldp, a0, b0, L.a_log_dev, L.dt_bias_dev, \
+    hipLaunchKernelGGL((delta_kernel<RPT, LPC>), grid, block, 0, e->stream, e->f32a, C, proj, ldp, a0, b0, L.a_log_dev, L.dt_bias_dev, \
                        L.unit_eps, m.seq_row0, m.seq_slot, run.state, e->obuf, L.heads, L.kv_heads, L.dim, L.vdim)
 #define HY_DELTA_R(LPC)                          \
     switch (rpt) {                               \
@@ -287,6 +303,11 @@ struct AttnExtra {
     int vshare = 1;          // K/V heads in a row that read one value head
     int gate_per_head = 0;   // the gate holds one number per head
     float *out32 = nullptr;  // float32 read-out [rows, heads, vdim] instead of D rows
+    float softcap = 0.f;     // > 0: s <- softcap tanh(s / softcap)
+    const float *slopes = nullptr;  // [heads] distance bias: s -= slope (i - j)
+    const float *sinks = nullptr;   // [heads] learned sinks (with L.sink)
+    float out_scale = 1.f;   // factor on the read-out
+    bool any() const { return window > 0 || vshare != 1 || gate_per_head || out32 || softcap > 0.f || slopes || sinks || out_scale != 1.f; }
 };
 
 // a windowed layer's split of the keys: a decode step sees at most `window` keys, whatever the context
@@ -316,18 +337,19 @@ static int launch_attn_tile(tl_hybrid *e, const tl_hybrid_layer &L, const void *
     // chunks whose rows fit one 16-row MFMA tile (decode steps): the four waves share the keys of a tile instead of the rows
     const bool wsplit = sh.max_len * HGB <= 16;
     const size_t lds = std::max(lds_tiles, (size_t)(128 + 4 * 64 * 4 * VT) * 4);
-    const bool ext = x.window > 0 || x.vshare != 1 || x.gate_per_head || x.out32;  // (plain causal attention keeps a kernel of its own)
+    const bool ext = x.any();  // (plain causal attention keeps a kernel of its own)
     auto kern = ext ? (wsplit ? attn_tile_kernel<D, DK4, VT, true, true> : attn_tile_kernel<D, DK4, VT, false, true>)
                     : (wsplit ? attn_tile_kernel<D, DK4, VT, true, false> : attn_tile_kernel<D, DK4, VT, false, false>);
     (void)hipFuncSetAttribute(reinterpret_cast<const void *>(kern), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
     dim3 grid((sh.max_len + TQ - 1) / TQ, L.kv_heads * n_hblk, sh.n_seqs * sh.n_splits);
     hipLaunchKernelGGL(kern, grid, dim3(256), lds, e->stream, e->qbuf, (const S *)kpool, (const S *)vpool, m.seq_row0, m.seq_slot, m.row_pos,
                        e->table_dev, c.max_pages_per_seq, c.page_size, L.heads, L.kv_heads, L.dim, L.vdim, L.scale, L.sink, HGB, n_hblk, sh.keys_per_split,
-                       sh.n_splits, gate, ldg, (S *)out, ldo, e->part_acc, e->part_ml, page_shift, vec_ok, v_row, x.window, x.vshare, x.gate_per_head, x.out32);
+                       sh.n_splits, gate, ldg, (S *)out, ldo, e->part_acc, e->part_ml, page_shift, vec_ok, v_row, x.window, x.vshare, x.gate_per_head, x.out32,
+                       x.softcap, x.slopes, x.sinks, x.out_scale);
     TL_CHECK_LAUNCH("hybrid attention tile");
     if (sh.n_splits > 1) {
         hipLaunchKernelGGL((attn_merge_kernel<D>), dim3(sh.rows, L.heads), dim3(64), 0, e->stream, e->part_acc, e->part_ml, sh.n_splits, L.heads, L.vdim, gate,
-                           ldg, (S *)out, ldo, x.gate_per_head, x.out32);
+                           ldg, (S *)out, ldo, x.gate_per_head, x.out32, x.out_scale);
         TL_CHECK_LAUNCH("hybrid attention merge");
     }
     return TL_OK;
@@ -346,13 +368,14 @@ static int attention_core(tl_hybrid *e, const tl_hybrid_layer &L, const void *kp
     // value template for every width beyond 8 tiles
     const bool whole_chunks = L.dim % 8 == 0 && L.vdim % 8 == 0 && v_row % 8 == 0;
     const bool beyond_mid = dk4 > 32 || vt_n > 8;
-    const bool ext = x.window > 0 || x.vshare != 1 || x.gate_per_head || x.out32;
+    const bool ext = x.any();
     // (the 64-wide templates are built for plain causal attention only: with a window, shared values or float32 read-outs the 16-tile one gave
     // wrong rows in decode steps, so those options stay on the templates up to 128 x 128 and take the row kernel beyond)
     if (e->attn_rows_only || dk4 > 64 || vt_n > 16 || (beyond_mid && (!whole_chunks || ext))) {
         hipLaunchKernelGGL((attn_rows_kernel<D>), dim3(sh.rows, L.heads), dim3(64), (L.dim + 64) * sizeof(float), e->stream, e->qbuf, (const S *)kpool,
                            (const S *)vpool, m.row_seq, m.row_pos, m.seq_slot, e->table_dev, c.max_pages_per_seq, c.page_size, L.heads, L.kv_heads, L.dim,
-                           L.vdim, L.scale, L.sink, gate, ldg, (S *)out, ldo, v_row, x.window, x.vshare, x.gate_per_head, x.out32);
+                           L.vdim, L.scale, L.sink, gate, ldg, (S *)out, ldo, v_row, x.window, x.vshare, x.gate_per_head, x.out32, x.softcap, x.slopes,
+                           x.sinks, x.out_scale);
         TL_CHECK_LAUNCH("hybrid attention");
         return TL_OK;
     }
@@ -387,7 +410,7 @@ static int launch_attn_talk_tile(tl_hybrid *e, const tl_hybrid_layer &L, const v
     TL_CHECK_LAUNCH("hybrid attention tile (mixed heads)");
     if (sh.n_splits > 1) {
         hipLaunchKernelGGL((attn_merge_kernel<D>), dim3(sh.rows, L.heads), dim3(64), 0, e->stream, e->part_acc, e->part_ml, sh.n_splits, L.heads, L.vdim, gate,
-                           ldg, (S *)out, ldo, 0, (float *)nullptr);
+                           ldg, (S *)out, ldo, 0, (float *)nullptr, 1.f);
         TL_CHECK_LAUNCH("hybrid attention merge");
     }
     return TL_OK;
@@ -433,7 +456,7 @@ static int attention_talk(tl_hybrid *e, const tl_hybrid_layer &L, const void *kp
     return TL_OK;
 }
 
-static int launch_linrec(const tl_hybrid *e, const tl_hybrid_layer &L, const Run &run, const Meta &m, int n_seqs, int ldp) {
+static int launch_linrec(const tl_hybrid *e, const tl_hybrid_layer &L, const MixState &run, const Meta &m, int n_seqs, const float *proj, int ldp) {
     const bool chan = L.rec_kind == TL_REC_CHANNEL;
     const int ones = L.rec_kind == TL_REC_EXPGATE ? 1 : 0, VE = L.vdim + ones;
     // lanes per state column: a wave while the step's columns are few (decode), a DPP row of 16 otherwise (or for narrow keys)
@@ -446,9 +469,13 @@ static int launch_linrec(const tl_hybrid *e, const tl_hybrid_layer &L, const Run
     TL_REQUIRE(rpt <= 16, "hybrid linrec: key width above 1024 is not supported");
     dim3 grid(L.heads, n_seqs, (VE + 256 / lpc - 1) / (256 / lpc)), block(256);
     const int q0 = 0, k0 = L.heads * L.dim, v0 = 2 * L.heads * L.dim;
+    // constant decays: with a rotation q and k come prepared (fixed_decay_prep_kernel), without one the kernel applies SiLU and the scale itself
+    const bool fixed = L.rec_kind == TL_REC_FIXED;
+    const int silu = fixed && L.rec_silu ? (L.rot_dims > 0 ? 2 : 3) : 0;
+    const float k_mul = fixed && L.rot_dims <= 0 && !L.rec_plain_k ? 1.f / sqrtf((float)L.dim) : 1.f;
 #define HY_LR(RPT, LPC, CHAN)                                                                                                                      \
-    hipLaunchKernelGGL((linrec_kernel<RPT, LPC, CHAN>), grid, block, 0, e->stream, e->proj, ldp, q0, k0, v0, e->gates, e->f32a, m.seq_row0, m.seq_slot, \
-                       run.state, e->obuf, L.heads, L.dim, L.vdim, ones)
+    hipLaunchKernelGGL((linrec_kernel<RPT, LPC, CHAN>), grid, block, 0, e->stream, proj, ldp, q0, k0, v0, e->gates, e->f32a, m.seq_row0, m.seq_slot, \
+                       run.state, e->obuf, L.heads, L.dim, L.vdim, ones, fixed ? L.decay_dev : (const float *)nullptr, silu, k_mul)
 #define HY_LR_R(LPC, CHAN)                    \
     switch (rpt) {                            \
         case 1: HY_LR(1, LPC, CHAN); break;   \
@@ -481,12 +508,16 @@ static int norm_t(tl_hybrid *e, int kind, const float *w, const float *b, float 
     return TL_OK;
 }
 
-// the token mixer of one layer run: proj [rows, ldp] (every projection of the normed input) -> cat[:, 0 .. heads * vdim) as D rows of ldcat
+// one token mixer of a layer run (part 0: the layer's own, 1: the one beside it): proj [rows, ldp] (its projections of the normed input) ->
+// cat[:, 0 .. heads * vdim) as D rows of ldcat, times out_scale
 template <typename D>
-static int mixer_t(tl_hybrid *e, size_t ri, const Meta &m, const StepShape &sh, int ldp, int ldcat) {
+static int mixer_part_t(tl_hybrid *e, size_t ri, int part, float *proj, typename D::storage *cat, float out_scale, const Meta &m, const StepShape &sh, int ldp,
+                        int ldcat) {
     using S = typename D::storage;
-    const Run &run = e->runs[ri];
-    const tl_hybrid_layer &L = e->layers[run.layer];
+    const MixState &run = e->runs[ri].mix[part];
+    const int layer = e->runs[ri].layer;
+    const tl_hybrid_layer &L = part ? e->beside[layer] : e->layers[layer];
+    const float *inv_freq = e->inv_freq[2 * layer + part];
     const tl_hybrid_config &c = e->cfg;
     hipStream_t st = e->stream;
     const int rows = sh.rows, n_seqs = sh.n_seqs, H = L.heads, HV = L.heads * L.vdim;
@@ -495,55 +526,68 @@ static int mixer_t(tl_hybrid *e, size_t ri, const Meta &m, const StepShape &sh, 
         if (L.diff_maps || L.qk_head_norm || L.window > 0 || L.gated == 2) {
             // q / k normed per head ahead of the rotation, maps side by side, a window on the keys, one gate per head
             const int M = attn_maps(L);
-            hipLaunchKernelGGL((attn_prep_head_kernel<D>), dim3(rows, M * (H + G) + G), dim3(64), 0, st, e->proj, ldp, m.row_seq, m.row_pos, m.seq_slot, e->table_dev,
-                               c.max_pages_per_seq, c.page_size, e->inv_freq[run.layer], L.rot_dims, L.rot_half, L.qk_head_norm, L.q_norm_dev, L.k_norm_dev, c.norm_eps,
-                               H, G, M, L.dim, L.vdim, e->qbuf, (S *)run.kpool, (S *)run.vpool, L.w_in_bias_dev);
+            hipLaunchKernelGGL((attn_prep_head_kernel<D>), dim3(rows, M * (H + G) + G), dim3(64), 0, st, proj, ldp, m.row_seq, m.row_pos, m.seq_slot, e->table_dev,
+                               c.max_pages_per_seq, c.page_size, inv_freq, L.rot_dims, L.rot_half, L.qk_head_norm, L.q_norm_dev, L.k_norm_dev, c.norm_eps,
+                               H, G, M, L.dim, L.vdim, e->qbuf, (S *)run.kpool, (S *)run.vpool, L.w_in_bias_dev,
+                               L.q_temp_coef, L.q_temp_every);
             TL_CHECK_LAUNCH("hybrid attention prep (per-head norm)");
-            const float *gate = L.gated ? e->proj + (size_t)M * (H + G) * L.dim + (size_t)G * L.vdim : nullptr;
+            const float *gate = L.gated ? proj + (size_t)M * (H + G) * L.dim + (size_t)G * L.vdim : nullptr;
             AttnExtra x;
-            x.window = L.window, x.vshare = M, x.gate_per_head = L.gated == 2;
-            if (!L.diff_maps) return attention_core<D>(e, L, run.kpool, run.vpool, L.vdim, m, sh, gate, ldp, e->cat, ldcat, x);
+            x.window = L.window, x.vshare = M, x.gate_per_head = L.gated == 2, x.out_scale = out_scale;
+            x.softcap = L.softcap, x.slopes = L.bias_slope_dev;
+            if (!L.diff_maps) return attention_core<D>(e, L, run.kpool, run.vpool, L.vdim, m, sh, gate, ldp, cat, ldcat, x);
             tl_hybrid_layer A = L;  // every map is a head of its own over M * G K/V heads; the read-outs stay float32 for the combination
             A.heads = M * H, A.kv_heads = M * G;
             x.out32 = e->obuf;
             HY_TRY(attention_core<D>(e, A, run.kpool, run.vpool, L.vdim, m, sh, nullptr, 0, nullptr, 0, x));
             hipLaunchKernelGGL((diff_combine_kernel<D>), dim3(rows, H), dim3(64), 0, st, e->obuf, L.diff_lambda, L.diff_init, c.norm_eps, gate, ldp, x.gate_per_head, H, G,
-                               L.vdim, (S *)e->cat, ldcat);
+                               L.vdim, cat, ldcat);
             TL_CHECK_LAUNCH("hybrid differential combination");
             return TL_OK;
         }
         if (L.qk_norm || L.rot_half || L.v_mix != TL_VMIX_NONE)  // (options of the row-wise preparation; create checked that it covers the layer)
-            hipLaunchKernelGGL((attn_prep_row_kernel<D>), dim3(rows), dim3(rows < 64 ? 1024 : 256), 0, st, e->proj, ldp, m.row_seq, m.row_pos, m.seq_slot, e->table_dev,
-                               c.max_pages_per_seq, c.page_size, e->inv_freq[run.layer], L.rot_dims, L.rot_half, L.qk_norm, L.q_norm_dev, L.k_norm_dev,
-                               c.norm_eps, H, G, L.dim, L.vdim, L.v_mix, L.v_mix_lambda, e->vref, e->qbuf, (S *)run.kpool, (S *)run.vpool);
+            hipLaunchKernelGGL((attn_prep_row_kernel<D>), dim3(rows), dim3(rows < 64 ? 1024 : 256), 0, st, proj, ldp, m.row_seq, m.row_pos, m.seq_slot, e->table_dev,
+                               c.max_pages_per_seq, c.page_size, inv_freq, L.rot_dims, L.rot_half, L.qk_norm, L.q_norm_dev, L.k_norm_dev,
+                               c.norm_eps, H, G, L.dim, L.vdim, L.v_mix, L.v_mix_lambda, e->vref, e->qbuf, (S *)run.kpool, (S *)run.vpool,
+                               L.q_temp_coef, L.q_temp_every);
         else
-            hipLaunchKernelGGL((attn_prep_kernel<D>), dim3(rows, H + 2 * G), dim3(64), 0, st, e->proj, ldp, m.row_seq, m.row_pos, m.seq_slot,
-                               e->table_dev, c.max_pages_per_seq, c.page_size, e->inv_freq[run.layer], L.rot_dims, L.qk_unit_rms, c.norm_eps, H, G, L.dim,
-                               L.vdim, e->qbuf, (S *)run.kpool, (S *)run.vpool);
+            hipLaunchKernelGGL((attn_prep_kernel<D>), dim3(rows, H + 2 * G), dim3(64), 0, st, proj, ldp, m.row_seq, m.row_pos, m.seq_slot,
+                               e->table_dev, c.max_pages_per_seq, c.page_size, inv_freq, L.rot_dims, L.qk_unit_rms, c.norm_eps, H, G, L.dim,
+                               L.vdim, e->qbuf, (S *)run.kpool, (S *)run.vpool, L.q_temp_coef, L.q_temp_every);
         TL_CHECK_LAUNCH("hybrid attention prep");
-        const float *gate = L.gated ? e->proj + (size_t)(H + G) * L.dim + (size_t)G * L.vdim : nullptr;
-        if (L.talk_dev || L.sink_dev || L.chunk > 0) return attention_talk<D>(e, L, run.kpool, run.vpool, m, sh, gate, ldp, e->cat, ldcat);
-        return attention_core<D>(e, L, run.kpool, run.vpool, L.vdim, m, sh, gate, ldp, e->cat, ldcat);
+        const float *gate = L.gated ? proj + (size_t)(H + G) * L.dim + (size_t)G * L.vdim : nullptr;
+        if (L.talk_dev || L.sink_dev || L.chunk > 0) return attention_talk<D>(e, L, run.kpool, run.vpool, m, sh, gate, ldp, cat, ldcat);
+        AttnExtra x;
+        x.softcap = L.softcap, x.slopes = L.bias_slope_dev, x.out_scale = out_scale;
+        return attention_core<D>(e, L, run.kpool, run.vpool, L.vdim, m, sh, gate, ldp, cat, ldcat, x);
     }
     if (L.kind == TL_MIX_LATENT) {
-        // proj: dq (q_rank) | [dkv (kv_rank + rot_dim)] | gate (H * vdim)
-        const int own = L.kv_from < 0, kv0 = L.q_rank, g0 = L.q_rank + (own ? L.kv_rank + L.rot_dim : 0), DT = L.kv_rank + L.rot_dim, DQ = L.dim + L.rot_dim;
-        hipLaunchKernelGGL((rms_cols_kernel<D>), dim3(rows), dim3(rows < 64 ? 512 : 128), 0, st, e->proj, ldp, L.q_rank, L.dq_norm_dev, c.norm_eps, (S *)e->da, L.q_rank);
-        TL_CHECK_LAUNCH("hybrid latent query norm");
-        HY_TRY(linear_t<D>(e->da, L.q_rank, L.uq_dev, e->f32a, H * DQ, rows, H * DQ, L.q_rank, 0, 1.f, nullptr, 0, st));
-        hipLaunchKernelGGL((latent_prep_kernel<D>), dim3(rows, H + 1), dim3(64), 0, st, e->f32a, H, L.dim, L.rot_dim, L.kv_rank, e->proj, ldp, kv0,
+        // proj: dq (q_rank) or q itself (H (dim + rot_dim)) | [dkv (kv_rank + rot_dim)] | gate (H * vdim, or H)
+        const int own = L.kv_from < 0, DT = L.kv_rank + L.rot_dim, DQ = L.dim + L.rot_dim, kv0 = L.q_rank ? L.q_rank : H * DQ, g0 = kv0 + (own ? DT : 0);
+        const float *q = proj;
+        int ldq = ldp;
+        if (L.q_rank) {
+            hipLaunchKernelGGL((rms_cols_kernel<D>), dim3(rows), dim3(rows < 64 ? 512 : 128), 0, st, proj, ldp, L.q_rank, L.dq_norm_dev, c.norm_eps, (S *)e->da, L.q_rank);
+            TL_CHECK_LAUNCH("hybrid latent query norm");
+            HY_TRY(linear_t<D>(e->da, L.q_rank, L.uq_dev, e->f32a, H * DQ, rows, H * DQ, L.q_rank, 0, 1.f, nullptr, 0, st));
+            q = e->f32a, ldq = H * DQ;
+        }
+        hipLaunchKernelGGL((latent_prep_kernel<D>), dim3(rows, H + 1), dim3(64), 0, st, q, ldq, H, L.dim, L.rot_dim, L.kv_rank, proj, ldp, kv0,
                            L.dkv_norm_dev, c.norm_eps, own, m.row_seq, m.row_pos, m.seq_slot, e->table_dev, c.max_pages_per_seq, c.page_size,
-                           e->inv_freq[run.layer], L.rot_dims, e->rot_mult[run.layer], (S *)e->db, e->qbuf, (S *)run.kpool);
+                           inv_freq, L.rot_dims, e->rot_mult[2 * layer + part], (S *)e->db, e->qbuf, (S *)run.kpool);
         TL_CHECK_LAUNCH("hybrid latent prep");
         // the keys' per-head projection moves onto the query: q_h' = W_uk,h^T q_h  -> qbuf[t, h, 0 .. kv_rank)
         HY_TRY(linear_t<D>(e->db, H * L.dim, L.uk_t_dev, e->qbuf, H * DT, rows, L.kv_rank, L.dim, 0, 1.f, nullptr, 0, st, H, L.dim, (long)L.kv_rank * L.dim, DT));
         tl_hybrid_layer A = L;  // one K/V head: keys [c | rotated part], values = the keys' leading kv_rank columns
-        A.kv_heads = 1, A.dim = DT, A.vdim = L.kv_rank, A.sink = 0;
-        HY_TRY(attention_core<D>(e, A, run.kpool, run.kpool, DT, m, sh, nullptr, 0, e->da, H * L.kv_rank));
+        A.kv_heads = 1, A.dim = DT, A.vdim = L.kv_rank;
+        AttnExtra x;
+        x.window = L.window, x.sinks = L.sink ? L.sink_dev : nullptr;
+        HY_TRY(attention_core<D>(e, A, run.kpool, run.kpool, DT, m, sh, nullptr, 0, e->da, H * L.kv_rank, x));
         // ... and the values' onto the read-out: o_h = W_uv,h (sum_j p_j c_j)
         HY_TRY(linear_t<D>(e->da, H * L.kv_rank, L.uv_dev, e->obuf, HV, rows, L.vdim, L.kv_rank, 0, 1.f, nullptr, 0, st, H, L.kv_rank, (long)L.vdim * L.kv_rank, L.vdim));
         const size_t n = (size_t)rows * HV;
-        hipLaunchKernelGGL((gate_mul_kernel<D>), dim3((unsigned)((n + 255) / 256)), dim3(256), 0, st, e->obuf, HV, e->proj + g0, ldp, HV, L.gated ? 0 : 2, (S *)e->cat, ldcat, rows);
+        hipLaunchKernelGGL((gate_mul_kernel<D>), dim3((unsigned)((n + 255) / 256)), dim3(256), 0, st, e->obuf, HV, proj + g0, ldp, HV, L.gated ? 0 : 2,
+                           L.gated == 2 ? L.vdim : 1, out_scale, cat, ldcat, rows);
         TL_CHECK_LAUNCH("hybrid latent gate");
         return TL_OK;
     }
@@ -551,52 +595,72 @@ static int mixer_t(tl_hybrid *e, size_t ri, const Meta &m, const StepShape &sh, 
         // proj: q (H dim) | k (H dim) | v (H vdim) | gate (H vdim) | i (H) | f (H)   or   ... | a1 (a_rank)
         const int g0 = 2 * H * L.dim + HV, x0 = g0 + HV;
         const bool chan = L.rec_kind == TL_REC_CHANNEL;
-        if (L.rec_kind == TL_REC_FIXED) {  // rotation of q and k, k * dim^-1/2, the constant decays as this step's gates
-            hipLaunchKernelGGL(fixed_decay_prep_kernel, dim3(rows, H), dim3(64), 0, st, e->proj, ldp, 0, H * L.dim, m.row_pos, e->inv_freq[run.layer], L.rot_dims,
-                               L.rot_half, 1.f / sqrtf((float)L.dim), L.decay_dev, e->gates, H, L.dim);
-            TL_CHECK_LAUNCH("hybrid constant decay prep");
-            HY_TRY(launch_linrec(e, L, run, m, n_seqs, ldp));
-            hipLaunchKernelGGL((linrec_out_kernel<D>), dim3(rows, H), dim3(64), 0, st, e->obuf, L.vdim, 0, e->gates, 1.f, L.out_norm_dev, 0, c.norm_eps, e->proj + g0, ldp,
-                               1, H, L.vdim, (S *)e->cat, ldcat);
+        if (L.rec_kind == TL_REC_FIXED) {
+            if (L.rot_dims > 0) {  // rotation of q and k (behind their SiLU), k * dim^-1/2
+                hipLaunchKernelGGL(fixed_decay_prep_kernel, dim3(rows, H), dim3(64), 0, st, proj, ldp, 0, H * L.dim, m.row_pos, inv_freq, L.rot_dims, L.rot_half,
+                                   L.rec_plain_k ? 1.f : 1.f / sqrtf((float)L.dim), L.rec_silu, H, L.dim);
+                TL_CHECK_LAUNCH("hybrid constant decay prep");
+            }
+            HY_TRY(launch_linrec(e, L, run, m, n_seqs, proj, ldp));
+            const int gate_kind = L.rec_sigmoid_gate ? 0 : 1;
+            if (L.rec_joint_norm)
+                hipLaunchKernelGGL((linrec_out_joint_kernel<D>), dim3(rows), dim3(rows < 64 ? 1024 : 256), 0, st, e->obuf, L.out_norm_dev, c.norm_eps, proj + g0, ldp,
+                                   gate_kind, HV, cat, ldcat, out_scale);
+            else
+                hipLaunchKernelGGL((linrec_out_kernel<D>), dim3(rows, H), dim3(64), 0, st, e->obuf, L.vdim, 0, e->gates, 1.f, L.out_norm_dev, 0, c.norm_eps, proj + g0,
+                                   ldp, gate_kind, H, L.vdim, cat, ldcat, out_scale);
             TL_CHECK_LAUNCH("hybrid linrec out");
             return TL_OK;
         }
         if (chan) {
             const size_t na = (size_t)rows * L.a_rank, nd = (size_t)rows * H * L.dim;
-            hipLaunchKernelGGL((cast_cols_kernel<D>), dim3((unsigned)((na + 255) / 256)), dim3(256), 0, st, e->proj, ldp, x0, L.a_rank, (S *)e->da, L.a_rank, rows);
+            hipLaunchKernelGGL((cast_cols_kernel<D>), dim3((unsigned)((na + 255) / 256)), dim3(256), 0, st, proj, ldp, x0, L.a_rank, (S *)e->da, L.a_rank, rows);
             TL_CHECK_LAUNCH("hybrid decay input");
             HY_TRY(linear_t<D>(e->da, L.a_rank, L.a2_dev, e->f32a, H * L.dim, rows, H * L.dim, L.a_rank, 0, 1.f, nullptr, 0, st));
             hipLaunchKernelGGL(channel_decay_kernel, dim3((unsigned)((nd + 255) / 256)), dim3(256), 0, st, e->f32a, L.a2_bias_dev, H * L.dim, 1.f / L.tau, rows);
             TL_CHECK_LAUNCH("hybrid channel decay");
         } else {
-            hipLaunchKernelGGL(expgate_scan_kernel, dim3(n_seqs, H), dim3(64), 0, st, e->proj, ldp, x0, x0 + H, L.i_bias_dev, L.f_bias_dev, L.gate_cap,
+            hipLaunchKernelGGL(expgate_scan_kernel, dim3(n_seqs, H), dim3(64), 0, st, proj, ldp, x0, x0 + H, L.i_bias_dev, L.f_bias_dev, L.gate_cap,
                                m.seq_row0, m.seq_slot, run.conv_state, e->gates, H);
             TL_CHECK_LAUNCH("hybrid gate scan");
         }
-        HY_TRY(launch_linrec(e, L, run, m, n_seqs, ldp));
+        HY_TRY(launch_linrec(e, L, run, m, n_seqs, proj, ldp));
         hipLaunchKernelGGL((linrec_out_kernel<D>), dim3(rows, H), dim3(64), 0, st, e->obuf, L.vdim + (chan ? 0 : 1), chan ? 0 : 1, e->gates,
-                           1.f / sqrtf((float)L.dim), L.out_norm_dev, chan ? 0 : L.vdim, c.norm_eps, e->proj + g0, ldp, chan ? 1 : 0, H, L.vdim, (S *)e->cat,
-                           ldcat);
+                           1.f / sqrtf((float)L.dim), L.out_norm_dev, chan ? 0 : L.vdim, c.norm_eps, proj + g0, ldp, chan ? 1 : 0, H, L.vdim, cat,
+                           ldcat, out_scale);
         TL_CHECK_LAUNCH("hybrid linrec out");
         return TL_OK;
     }
     const int C = conv_channels(L);
     const size_t n = (size_t)rows * C;
-    hipLaunchKernelGGL(conv_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, st, e->proj, ldp, L.conv_dev, L.conv_taps, C, m.row_seq,
+    hipLaunchKernelGGL(conv_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, st, proj, ldp, L.conv_dev, L.conv_taps, C, m.row_seq,
                        m.seq_row0, m.seq_slot, run.conv_state, e->f32a, rows);
     TL_CHECK_LAUNCH("hybrid conv");
     if (L.conv_taps > 1) {
-        hipLaunchKernelGGL(conv_state_kernel, dim3((unsigned)(((size_t)n_seqs * C + 255) / 256)), dim3(256), 0, st, e->proj, ldp, L.conv_taps, C,
+        hipLaunchKernelGGL(conv_state_kernel, dim3((unsigned)(((size_t)n_seqs * C + 255) / 256)), dim3(256), 0, st, proj, ldp, L.conv_taps, C,
                            m.seq_row0, m.seq_slot, run.conv_state, n_seqs);
         TL_CHECK_LAUNCH("hybrid conv state");
     }
-    HY_TRY(launch_delta(e, L, run, m, n_seqs, ldp));
-    const float *gate = e->proj + (size_t)C;
+    HY_TRY(launch_delta(e, L, run, m, n_seqs, proj, ldp));
+    const float *gate = proj + (size_t)C;
     hipLaunchKernelGGL((delta_out_kernel<D>), dim3(rows, L.heads), dim3(64), 0, st, e->obuf, L.out_norm_dev, c.norm_eps, gate, ldp, L.heads,
-                       L.vdim, (S *)e->cat, ldcat);
+                       L.vdim, cat, ldcat, out_scale);
     TL_CHECK_LAUNCH("hybrid delta out");
     return TL_OK;
 }
+
+// every mixer of a layer run: the layer's own, then the one beside it on the projections behind (their read-outs lie side by side in cat, each
+// times its factor, so one product with the output matrices side by side sums their results)
+template <typename D>
+static int mixer_t(tl_hybrid *e, size_t ri, const Meta &m, const StepShape &sh, int ldp, int ldcat) {
+    using S = typename D::storage;
+    const int layer = e->runs[ri].layer;
+    const tl_hybrid_layer &L = e->layers[layer], &B = e->beside[layer];
+    if (B.kind < 0) return mixer_part_t<D>(e, ri, 0, e->proj, (S *)e->cat, 1.f, m, sh, ldp, ldcat);
+    HY_TRY(mixer_part_t<D>(e, ri, 0, e->proj, (S *)e->cat, L.mix_scale, m, sh, ldp, ldcat));
+    return mixer_part_t<D>(e, ri, 1, e->proj + mixer_cols(L), (S *)e->cat + L.heads * L.vdim, B.mix_scale, m, sh, ldp, ldcat);
+}
+
 
 // the feed-forward's activation: proj columns up0 .. -> cat columns col0 .. col0 + L.ff
 template <typename D>
@@ -608,14 +672,14 @@ static int ff_act_t(tl_hybrid *e, const tl_hybrid_layer &L, int rows, int ldp, i
         if (L.moe_gated) {  // gates | ups | router | [scalar shared gate] | padding
             const int ET = L.experts + L.identity, r0 = up0 + 2 * L.ff;
             hipLaunchKernelGGL((moe_gated_act_kernel<D>), grid, dim3(256), 0, st, e->proj, ldp, r0, L.moe_shared_sg ? r0 + ET : -1, up0, up0 + L.ff, L.experts,
-                               L.identity, L.top, L.groups, L.keep, L.expert_ff, L.shared_ff, L.correction_dev, (S *)e->cat, ldcat, col0, e->idw, L.moe_router,
+                               L.identity, L.top, L.groups, L.keep, L.expert_ff, L.shared_ff, L.correction_dev, L.router_bias_dev, (S *)e->cat, ldcat, col0, e->idw, L.moe_router,
                                L.moe_scale_input, L.ff_act);
             TL_CHECK_LAUNCH("hybrid moe route (gated experts)");
             return TL_OK;
         }
         const int ET = L.experts + L.identity, r0 = up0 + L.ff;  // shared up | expert ups | router | shared gate | padding
         hipLaunchKernelGGL((moe_route_act_kernel<D>), grid, dim3(256), 0, st, e->proj, ldp, r0, r0 + ET, up0, up0 + L.shared_ff,
-                           L.experts, L.identity, L.top, L.groups, L.keep, L.expert_ff, L.shared_ff, L.correction_dev, (S *)e->cat, ldcat, col0, e->idw, L.moe_router);
+                           L.experts, L.identity, L.top, L.groups, L.keep, L.expert_ff, L.shared_ff, L.correction_dev, L.router_bias_dev, (S *)e->cat, ldcat, col0, e->idw, L.moe_router);
         TL_CHECK_LAUNCH("hybrid moe route");
         return TL_OK;
     }
@@ -630,6 +694,35 @@ static int ff_act_t(tl_hybrid *e, const tl_hybrid_layer &L, int rows, int ldp, i
     return TL_OK;
 }
 
+// a feed-forward of its own matrices on the D rows e->h: out (+)= (epi, alpha, col as in linear_t) its result.  Where the result is added (epi 1 / 3) the
+// identity experts' part is added too; a caller that takes the bare result (epi 0) adds it itself.
+template <typename D>
+static int ff_t(tl_hybrid *e, const tl_hybrid_layer &L, int rows, float *out, int epi, float alpha, const float *col, NormTail *tail) {
+    using S = typename D::storage;
+    const int W = e->cfg.width, nin2 = ff_in_cols(L);
+    hipStream_t st = e->stream;
+    // a step of a few rows takes few experts: the router's rows first, then only the experts some row takes are streamed
+    const bool few = rows <= 8 && L.ff_kind == TL_FF_MOE && L.moe_gated && L.experts <= 64 && L.top < L.experts && L.expert_ff % 8 == 0 && L.shared_ff % 8 == 0 && e->moe_mask;
+    SegSkip in_skip, out_skip;
+    if (few) {
+        HY_TRY(linear_t<D>(e->h, W, (const S *)L.w_in2_dev + (size_t)2 * L.ff * W, e->proj + 2 * L.ff, nin2, rows, nin2 - 2 * L.ff, W, 0, 1.f, nullptr, 0, st));
+        hipLaunchKernelGGL(moe_taken_mask_kernel, dim3(1), dim3(256), 0, st, e->proj, nin2, 2 * L.ff, rows, L.experts, L.identity, L.top, L.groups, L.keep,
+                           L.correction_dev, L.router_bias_dev, L.moe_router, e->moe_mask);
+        TL_CHECK_LAUNCH("hybrid moe taken experts");
+        in_skip.mask = out_skip.mask = e->moe_mask;
+        in_skip.lead = out_skip.lead = L.shared_ff, in_skip.len = out_skip.len = L.expert_ff;
+        in_skip.period = L.ff, in_skip.limit = 2 * L.ff, out_skip.on_k = 1;
+    }
+    HY_TRY(linear_t<D>(e->h, W, L.w_in2_dev, e->proj, nin2, rows, few ? 2 * L.ff : nin2, W, 0, 1.f, nullptr, 0, st, 1, 0, 0, 0, nullptr, few ? &in_skip : nullptr));
+    HY_TRY(ff_act_t<D>(e, L, rows, nin2, 0, L.ff, 0));
+    if (epi != 0 && L.ff_kind == TL_FF_MOE && L.identity > 0) {  // (before the experts' product: that one completes the sum and may carry the next norm, which overwrites h)
+        const size_t n = (size_t)rows * W;
+        hipLaunchKernelGGL((identity_axpy_kernel<D>), dim3((unsigned)((n + 255) / 256)), dim3(256), 0, st, out, (const S *)e->h, e->idw, col, alpha, W, rows);
+        TL_CHECK_LAUNCH("hybrid identity experts");
+    }
+    return linear_t<D>(e->cat, L.ff, L.w_out2_dev, out, W, rows, W, L.ff, epi, alpha, col, 0, st, 1, 0, 0, 0, tail, few ? &out_skip : nullptr);
+}
+
 // every layer run over the packed rows described by m
 template <typename D>
 static int forward_t(tl_hybrid *e, const Meta &m, const StepShape &sh) {
@@ -638,8 +731,13 @@ static int forward_t(tl_hybrid *e, const Meta &m, const StepShape &sh) {
     const tl_hybrid_config &c = e->cfg;
     hipStream_t st = e->stream;
     const int W = c.width;
+    PairEmbed pe;
+    if (c.pair_embed_dev) {
+        pe.table = c.pair_embed_dev, pe.buckets = c.pair_buckets, pe.mul_prev = c.pair_mul_prev, pe.mul_cur = c.pair_mul_cur;
+        pe.row_seq = m.row_seq, pe.row_pos = m.row_pos, pe.seq_row0 = m.seq_row0, pe.seq_prev = m.seq_prev;
+    }
     hipLaunchKernelGGL((embed_kernel<D>), dim3(rows), dim3(256), 0, st, m.tokens, (const S *)c.embed_dev, e->x0, e->x, W, c.vocab,
-                       c.embed_scale != 0.f ? c.embed_scale : 1.f, c.embed_norm_dev, c.final_norm_offset, c.norm_eps);
+                       c.embed_scale != 0.f ? c.embed_scale : 1.f, c.embed_norm_dev, c.final_norm_offset, c.norm_eps, pe);
     TL_CHECK_LAUNCH("hybrid embed");
     bool h_ready = false;  // e->h already holds this run's first norm (it left with the product that completed the previous residual sum)
     // the Dynamic Tanh norm that follows a residual sum: element-wise, so it can ride the completing product's epilogue
@@ -666,7 +764,7 @@ static int forward_t(tl_hybrid *e, const Meta &m, const StepShape &sh) {
             TL_CHECK_LAUNCH("hybrid pack2");
             HY_TRY(linear_t<D>(e->cat2, 2 * W, c.loop_in_dev, e->x, W, rows, W, 2 * W, 2, 1.f, c.loop_step_dev + (size_t)run.pass * W, 0, st));
         }
-        const int nmix = mixer_cols(L), HV = L.heads * L.vdim;
+        const int nmix = layer_mixer_cols(e, run.layer), HV = layer_read_cols(e, run.layer);
         if (c.parallel_block == TL_BLOCK_POSTNORM) {
             // x += m norm1(W_o mixer(x));  x += m norm2(ff(x)): the sublayers read the stream itself, the norm sits on what they return
             const size_t n = (size_t)rows * W;
@@ -681,26 +779,7 @@ static int forward_t(tl_hybrid *e, const Meta &m, const StepShape &sh) {
                                c.residual_mult, (S *)e->h, W);
             TL_CHECK_LAUNCH("hybrid norm on the mixer's output");
             if (L.ff > 0) {
-                const int nin2 = ff_in_cols(L);
-                // a step of a few rows takes few experts: the router's rows first, then only the experts some row takes are streamed
-                const bool few = rows <= 8 && L.ff_kind == TL_FF_MOE && L.moe_gated && L.experts <= 64 && L.top < L.experts && L.expert_ff % 8 == 0 && L.shared_ff % 8 == 0 && e->moe_mask;
-                if (few) {
-                    HY_TRY(linear_t<D>(e->h, W, (const S *)L.w_in2_dev + (size_t)2 * L.ff * W, e->proj + 2 * L.ff, nin2, rows, nin2 - 2 * L.ff, W, 0, 1.f, nullptr, 0, st));
-                    hipLaunchKernelGGL(moe_taken_mask_kernel, dim3(1), dim3(256), 0, st, e->proj, nin2, 2 * L.ff, rows, L.experts, L.identity, L.top, L.groups, L.keep,
-                                       L.correction_dev, L.moe_router, e->moe_mask);
-                    TL_CHECK_LAUNCH("hybrid moe taken experts");
-                    SegSkip in_skip, out_skip;
-                    in_skip.mask = out_skip.mask = e->moe_mask;
-                    in_skip.lead = out_skip.lead = L.shared_ff, in_skip.len = out_skip.len = L.expert_ff;
-                    in_skip.period = L.ff, in_skip.limit = 2 * L.ff, out_skip.on_k = 1;
-                    HY_TRY(linear_t<D>(e->h, W, L.w_in2_dev, e->proj, nin2, rows, 2 * L.ff, W, 0, 1.f, nullptr, 0, st, 1, 0, 0, 0, nullptr, &in_skip));
-                    HY_TRY(ff_act_t<D>(e, L, rows, nin2, 0, L.ff, 0));
-                    HY_TRY(linear_t<D>(e->cat, L.ff, L.w_out2_dev, e->y, W, rows, W, L.ff, 0, 1.f, nullptr, 0, st, 1, 0, 0, 0, nullptr, &out_skip));
-                } else {
-                    HY_TRY(linear_t<D>(e->h, W, L.w_in2_dev, e->proj, nin2, rows, nin2, W, 0, 1.f, nullptr, 0, st));
-                    HY_TRY(ff_act_t<D>(e, L, rows, nin2, 0, L.ff, 0));
-                    HY_TRY(linear_t<D>(e->cat, L.ff, L.w_out2_dev, e->y, W, rows, W, L.ff, 0, 1.f, nullptr, 0, st));
-                }
+                HY_TRY(ff_t<D>(e, L, rows, e->y, 0, 1.f, nullptr, nullptr));
                 if (L.ff_kind == TL_FF_MOE && L.identity > 0) {  // identity experts return their input: weight * h joins the branch ahead of its norm
                     hipLaunchKernelGGL((identity_axpy_kernel<D>), dim3((unsigned)((n + 255) / 256)), dim3(256), 0, st, e->y, (const S *)e->h, e->idw,
                                        (const float *)nullptr, 1.f, W, rows);
@@ -737,10 +816,7 @@ static int forward_t(tl_hybrid *e, const Meta &m, const StepShape &sh) {
                 h_ready = L.ff <= 0 && !side && next == 2;
             }
             if (L.ff > 0) {
-                const int nin2 = ff_in_cols(L);
-                HY_TRY(linear_t<D>(e->h, W, L.w_in2_dev, e->proj, nin2, rows, nin2, W, 0, 1.f, nullptr, 0, st));
-                HY_TRY(ff_act_t<D>(e, L, rows, nin2, 0, L.ff, 0));
-                HY_TRY(linear_t<D>(e->cat, L.ff, L.w_out2_dev, e->y, W, rows, W, L.ff, 0, 1.f, nullptr, 0, st));
+                HY_TRY(ff_t<D>(e, L, rows, e->y, 0, 1.f, nullptr, nullptr));
                 const int next = side ? 1 : (Nx ? 2 : 0);
                 hipLaunchKernelGGL((sandwich_add_kernel<D>), dim3(rows), dim3(threads), 0, st, e->x, e->y, L.post_norm2_dev, L.norm_offset, c.norm_eps, c.residual_mult,
                                    L.ls2_dev, next, Nx ? Nx->norm_dev : nullptr, Nx ? Nx->norm_offset : 0.f, (S *)e->h, W);
@@ -776,16 +852,7 @@ static int forward_t(tl_hybrid *e, const Meta &m, const StepShape &sh) {
             HY_TRY(linear_t<D>(e->cat, HV, L.w_out_dev, e->x, W, rows, W, HV, L.ls1_dev ? 3 : 1, c.residual_mult, L.ls1_dev, 0, st, 1, 0, 0, 0, after_mixer));
             if (L.ff > 0) {
                 if (!second.done) HY_TRY(norm_t<D>(e, L.norm_kind, L.norm2_dev, L.norm2_bias_dev, L.norm2_alpha, L.norm_offset, e->h, nullptr, rows));
-                const int nin2 = ff_in_cols(L);
-                HY_TRY(linear_t<D>(e->h, W, L.w_in2_dev, e->proj, nin2, rows, nin2, W, 0, 1.f, nullptr, 0, st));
-                HY_TRY(ff_act_t<D>(e, L, rows, nin2, 0, L.ff, 0));
-                if (L.ff_kind == TL_FF_MOE && L.identity > 0) {  // (before the experts' product: that one completes the sum and may carry the next norm, which overwrites h)
-                    const size_t n = (size_t)rows * W;
-                    hipLaunchKernelGGL((identity_axpy_kernel<D>), dim3((unsigned)((n + 255) / 256)), dim3(256), 0, st, e->x, (const S *)e->h, e->idw, L.ls2_dev,
-                                       c.residual_mult, W, rows);
-                    TL_CHECK_LAUNCH("hybrid identity experts");
-                }
-                HY_TRY(linear_t<D>(e->cat, L.ff, L.w_out2_dev, e->x, W, rows, W, L.ff, L.ls2_dev ? 3 : 1, c.residual_mult, L.ls2_dev, 0, st, 1, 0, 0, 0, &next_first));
+                HY_TRY(ff_t<D>(e, L, rows, e->x, L.ls2_dev ? 3 : 1, c.residual_mult, L.ls2_dev, &next_first));
             }
             h_ready = next_first.done;
         }
@@ -802,9 +869,10 @@ static int head_t(tl_hybrid *e, const Meta &m, int n_want, bool set_pending) {
     if (n_want <= 0) return TL_OK;
     HY_TRY(norm_t<D>(e, c.final_norm_kind, c.final_norm_dev, c.final_norm_bias_dev, c.final_norm_alpha, c.final_norm_offset, e->hsel, m.want_rows, n_want));
     HY_TRY(linear_t<D>(e->hsel, c.width, c.head_dev, e->logits, c.vocab, n_want, c.vocab, c.width, 0, 1.f, nullptr, 0, e->stream));
-    if (c.logit_scale != 0.f && c.logit_scale != 1.f) {
+    if ((c.logit_scale != 0.f && c.logit_scale != 1.f) || c.logit_softcap > 0.f) {
         const size_t n = (size_t)n_want * c.vocab;
-        hipLaunchKernelGGL(scale_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, e->stream, e->logits, c.logit_scale, n);
+        hipLaunchKernelGGL(logit_scale_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, e->stream, e->logits, c.logit_scale != 0.f ? c.logit_scale : 1.f,
+                           c.logit_softcap, n);
         TL_CHECK_LAUNCH("hybrid logit scale");
     }
     hipLaunchKernelGGL(argmax_kernel, dim3(n_want), dim3(1024), 0, e->stream, e->logits, c.vocab, e->argmax_dev, set_pending ? m.want_slot : (const int32_t *)nullptr,
@@ -856,6 +924,65 @@ static int reserve_all(tl_hybrid *e, int n_seqs, const int *slots, const int *ex
     return TL_OK;
 }
 
+// what a mixer's description must hold (layer i's own or the one beside it); vmix_width: the values width of the value-mixing layers so far (0: none)
+static int check_mixer(const tl_hybrid_layer *layers, int i, const tl_hybrid_layer &L, int &vmix_width) {
+    TL_REQUIRE(L.kind == TL_MIX_ATTENTION || L.kind == TL_MIX_DELTA || L.kind == TL_MIX_LINREC || L.kind == TL_MIX_LATENT, "hybrid_create: unknown mixer kind");
+    TL_REQUIRE(L.heads > 0 && L.kv_heads > 0 && L.heads % L.kv_heads == 0, "hybrid_create: heads must be a positive multiple of kv_heads");
+    TL_REQUIRE(L.dim > 0 && L.dim <= 1024 && L.vdim > 0 && L.vdim <= 512, "hybrid_create: head widths: dim 1..1024, vdim 1..512");
+    if (L.kind == TL_MIX_ATTENTION) {
+        TL_REQUIRE(L.rot_dims >= 0 && L.rot_dims % 2 == 0 && L.rot_dims <= L.dim, "hybrid_create: rot_dims must be even and at most dim");
+        TL_REQUIRE(!L.qk_norm || (L.q_norm_dev && L.k_norm_dev), "hybrid_create: a norm over the whole q / k projection needs its weights");
+        TL_REQUIRE(!(L.qk_unit_rms && (L.qk_norm || L.rot_half || L.v_mix != TL_VMIX_NONE)),
+                   "hybrid_create: unit-RMS heads after the rotation do not combine with the whole-projection norm, half-split rotation pairs or value mixing");
+        TL_REQUIRE(L.chunk >= 0 && L.v_mix >= TL_VMIX_NONE && L.v_mix <= TL_VMIX_BLEND, "hybrid_create: chunk >= 0, v_mix 0..2");
+        TL_REQUIRE(L.gated >= 0 && L.gated <= 2 && L.window >= 0, "hybrid_create: gated 0..2, window >= 0");
+        if (L.diff_maps || L.qk_head_norm || L.window > 0 || L.gated == 2) {
+            TL_REQUIRE(!L.qk_unit_rms && !L.qk_norm && L.v_mix == TL_VMIX_NONE && !L.talk_dev && !L.sink_dev && L.chunk == 0,
+                       "hybrid_create: per-head norms, maps, a window and per-head gates do not combine with unit-RMS heads, the whole-projection norm, value mixing, "
+                       "mixed scores, learned sinks or a chunked mask");
+            TL_REQUIRE(!L.qk_head_norm || (L.q_norm_dev && L.k_norm_dev), "hybrid_create: a norm per head needs its weights");
+            TL_REQUIRE(!L.diff_maps || !L.sink, "hybrid_create: differential attention takes no sink");
+        }
+        TL_REQUIRE(L.softcap >= 0.f && (L.q_temp_coef == 0.f || L.q_temp_every > 0.f), "hybrid_create: softcap >= 0; a query temperature needs q_temp_every > 0");
+        TL_REQUIRE((L.softcap == 0.f && !L.bias_slope_dev) || (!L.talk_dev && !L.sink_dev && L.chunk == 0 && !L.diff_maps),
+                   "hybrid_create: capped scores and a distance bias do not combine with mixed scores, learned sinks, a chunked mask or maps");
+        if (L.v_mix != TL_VMIX_NONE) {
+            if (vmix_width == 0) {
+                TL_REQUIRE(L.v_mix == TL_VMIX_FIRST, "hybrid_create: the first value-mixing layer keeps its values (v_mix 1), later ones blend (v_mix 2)");
+                vmix_width = L.kv_heads * L.vdim;
+            } else
+                TL_REQUIRE(L.v_mix == TL_VMIX_BLEND && L.kv_heads * L.vdim == vmix_width, "hybrid_create: value-mixing layers share one values width");
+        }
+    } else if (L.kind == TL_MIX_LINREC) {
+        TL_REQUIRE(L.kv_heads == L.heads && (L.out_norm_dev || L.rec_kind == TL_REC_FIXED), "hybrid_create: a linear recurrence has one key head per head and an output norm weight");
+        TL_REQUIRE(!L.rec_joint_norm || (L.rec_kind == TL_REC_FIXED && L.out_norm_dev), "hybrid_create: a norm over all heads belongs to a constant decay and needs its weight");
+        if (L.rec_kind == TL_REC_FIXED)
+            TL_REQUIRE(L.decay_dev && L.rot_dims >= 0 && L.rot_dims % 2 == 0 && L.rot_dims <= L.dim, "hybrid_create: a constant decay needs its values; rot_dims even and at most dim");
+        else if (L.rec_kind == TL_REC_CHANNEL)
+            TL_REQUIRE(L.a_rank >= 1 && L.a2_dev && L.a2_bias_dev && L.tau > 0.f, "hybrid_create: channel decay needs its projection pair, bias and tau > 0");
+        else
+            TL_REQUIRE(L.rec_kind == TL_REC_EXPGATE && L.i_bias_dev && L.f_bias_dev && L.gate_cap > 0.f, "hybrid_create: exponential gates need biases and a cap > 0");
+    } else if (L.kind == TL_MIX_LATENT) {
+        TL_REQUIRE(L.q_rank >= 0 && L.kv_rank >= 1 && L.rot_dim >= 0 && (L.q_rank == 0 || (L.dq_norm_dev && L.uq_dev)) && L.uk_t_dev && L.uv_dev,
+                   "hybrid_create: latent attention needs its ranks and per-head projections");
+        TL_REQUIRE(L.rot_dims >= 0 && L.rot_dims % 2 == 0 && L.rot_dims <= L.rot_dim, "hybrid_create: rot_dims must be even and at most rot_dim");
+        TL_REQUIRE(L.window >= 0 && L.gated >= 0 && L.gated <= 2 && (!L.sink_dev || L.sink), "hybrid_create: latent attention: window >= 0, gated 0..2, sinks with sink set");
+        TL_REQUIRE(L.kv_rank + L.rot_dim <= 1024 && L.kv_rank <= 512, "hybrid_create: latent widths: kv_rank + rot_dim <= 1024, kv_rank <= 512");
+        if (L.kv_from >= 0) {
+            TL_REQUIRE(L.kv_from < i, "hybrid_create: kv_from must name an earlier layer");
+            const tl_hybrid_layer &J = layers[L.kv_from];
+            TL_REQUIRE(J.kind == TL_MIX_LATENT && J.kv_from < 0 && J.kv_rank == L.kv_rank && J.rot_dim == L.rot_dim,
+                       "hybrid_create: kv_from must name a latent-attention layer with its own latent of the same widths");
+        } else {
+            TL_REQUIRE(L.dkv_norm_dev, "hybrid_create: a latent of its own needs its norm weight");
+        }
+    } else {
+        TL_REQUIRE(L.conv_taps >= 1 && L.conv_taps <= 64 && L.conv_dev && L.a_log_dev && L.dt_bias_dev && L.out_norm_dev,
+                   "hybrid_create: a delta layer needs conv taps and weights, a_log, dt_bias and its output norm");
+    }
+    return TL_OK;
+}
+
 }  // namespace hy
 }  // namespace tl
 
@@ -876,6 +1003,8 @@ extern "C" int tl_hybrid_create(const tl_hybrid_config *cfg, const tl_hybrid_lay
     TL_REQUIRE(c.final_norm_kind == TL_NORM_RMS || (c.final_norm_kind == TL_NORM_DYT && c.final_norm_bias_dev), "hybrid_create: final norm kind");
     TL_REQUIRE(c.page_size > 0 && c.num_pages > 0 && c.max_slots > 0 && c.max_pages_per_seq > 0 && c.max_rows > 0, "hybrid_create: pool sizes must be positive");
     TL_REQUIRE(c.embed_dev && c.final_norm_dev && c.head_dev, "hybrid_create: embed, final norm and head are required");
+    TL_REQUIRE(!c.pair_embed_dev || c.pair_buckets >= 1, "hybrid_create: a token-pair table needs at least one bucket");
+    TL_REQUIRE(c.logit_softcap >= 0.f, "hybrid_create: logit_softcap must not be negative");
     const bool looped = c.loop_times > 1 || (c.loop_times == 1 && c.loop_stop > c.loop_start);
     if (looped) {
         TL_REQUIRE(c.loop_start >= 0 && c.loop_stop > c.loop_start && c.loop_stop <= c.num_layers, "hybrid_create: loop range outside the layer list");
@@ -884,18 +1013,33 @@ extern "C" int tl_hybrid_create(const tl_hybrid_config *cfg, const tl_hybrid_lay
     auto e = std::make_unique<tl_hybrid>();
     e->cfg = c;
     e->layers.assign(layers, layers + c.num_layers);
+    e->beside.assign(c.num_layers, tl_hybrid_layer{});
+    for (int i = 0; i < c.num_layers; ++i) {
+        if (layers[i].beside) e->beside[i] = *layers[i].beside;
+        else e->beside[i].kind = -1;
+        e->layers[i].beside = e->beside[i].beside = nullptr;  // (the caller's structs are not kept)
+    }
     if (stream) e->stream = (hipStream_t)stream;
     else {
         HY_HIP(hipDeviceSynchronize());
         HY_HIP(hipStreamCreateWithFlags(&e->stream, hipStreamNonBlocking));
         e->owns_stream = true;
     }
+    const tl_hybrid_layer *p_layers = e->layers.data();
     int max_in = 0, max_cat = 0, max_q = 0, max_c = 0, max_hv = 0, max_gh = 1, max_da = 1, max_db = 1, vmix_width = 0;
+    bool any_moe = false;
     for (int i = 0; i < c.num_layers; ++i) {
         const tl_hybrid_layer &L = e->layers[i];
-        TL_REQUIRE(L.kind == TL_MIX_ATTENTION || L.kind == TL_MIX_DELTA || L.kind == TL_MIX_LINREC || L.kind == TL_MIX_LATENT, "hybrid_create: unknown mixer kind");
-        TL_REQUIRE(L.heads > 0 && L.kv_heads > 0 && L.heads % L.kv_heads == 0, "hybrid_create: heads must be a positive multiple of kv_heads");
-        TL_REQUIRE(L.dim > 0 && L.dim <= 1024 && L.vdim > 0 && L.vdim <= 512, "hybrid_create: head widths: dim 1..1024, vdim 1..512");
+        HY_TRY(check_mixer(p_layers, i, L, vmix_width));
+        const tl_hybrid_layer &B = e->beside[i];
+        if (B.kind >= 0) {
+            HY_TRY(check_mixer(p_layers, i, B, vmix_width));
+            TL_REQUIRE(L.v_mix == TL_VMIX_NONE && B.v_mix == TL_VMIX_NONE && !L.w_in_bias_dev && !B.w_in_bias_dev && (B.kind != TL_MIX_LATENT || B.kv_from < 0),
+                       "hybrid_create: side-by-side mixers take no value mixing, no projection biases and no cache of another layer");
+            for (const tl_hybrid_layer *X : {&L, &B})
+                TL_REQUIRE(X->kind != TL_MIX_ATTENTION || (!X->talk_dev && !X->sink_dev && X->chunk == 0 && !X->diff_maps),
+                           "hybrid_create: side-by-side mixers: the attention's read-out takes a factor only without mixed scores, learned sinks, chunks and maps");
+        }
         TL_REQUIRE(L.w_in_dev && L.w_out_dev && L.norm_dev && L.ff >= 0, "hybrid_create: layer matrices and norm are required");
         TL_REQUIRE(L.norm_kind == TL_NORM_RMS || (L.norm_kind == TL_NORM_DYT && L.norm_bias_dev), "hybrid_create: norm kind (Dynamic Tanh needs its bias)");
         if (c.parallel_block == TL_BLOCK_POSTNORM)
@@ -922,73 +1066,33 @@ extern "C" int tl_hybrid_create(const tl_hybrid_config *cfg, const tl_hybrid_lay
                 TL_REQUIRE(L.top >= 1 && L.top <= L.keep * (ET / L.groups), "hybrid_create: top exceeds the experts of the kept groups");
                 TL_REQUIRE(L.expert_ff >= 0 && L.shared_ff >= 0 && L.ff == L.shared_ff + L.experts * L.expert_ff,
                            "hybrid_create: mixture of experts: ff = shared_ff + experts * expert_ff");
-                TL_REQUIRE(L.correction_dev || L.moe_router == TL_ROUTER_SIGMOID, "hybrid_create: a softmax router needs its correction vector");
-                TL_REQUIRE(L.moe_router == TL_ROUTER_SOFTMAX || L.moe_router == TL_ROUTER_SIGMOID, "hybrid_create: unknown router kind");
+                TL_REQUIRE(L.correction_dev || L.moe_router != TL_ROUTER_SOFTMAX, "hybrid_create: a softmax router needs its correction vector");
+                TL_REQUIRE(L.moe_router >= TL_ROUTER_SOFTMAX && L.moe_router <= TL_ROUTER_CHOSEN_SOFTMAX, "hybrid_create: unknown router kind");
+                TL_REQUIRE(L.moe_router != TL_ROUTER_CHOSEN_SOFTMAX || !L.correction_dev, "hybrid_create: weights from the chosen logits take no correction");
                 TL_REQUIRE(L.moe_gated || (!L.moe_scale_input && !L.moe_shared_sg), "hybrid_create: a weight on the expert's input needs gated experts");
             }
         }
-        if (L.kind == TL_MIX_ATTENTION) {
-            TL_REQUIRE(L.rot_dims >= 0 && L.rot_dims % 2 == 0 && L.rot_dims <= L.dim, "hybrid_create: rot_dims must be even and at most dim");
-            TL_REQUIRE(!L.qk_norm || (L.q_norm_dev && L.k_norm_dev), "hybrid_create: a norm over the whole q / k projection needs its weights");
-            TL_REQUIRE(!(L.qk_unit_rms && (L.qk_norm || L.rot_half || L.v_mix != TL_VMIX_NONE)),
-                       "hybrid_create: unit-RMS heads after the rotation do not combine with the whole-projection norm, half-split rotation pairs or value mixing");
-            TL_REQUIRE(L.chunk >= 0 && L.v_mix >= TL_VMIX_NONE && L.v_mix <= TL_VMIX_BLEND, "hybrid_create: chunk >= 0, v_mix 0..2");
-            TL_REQUIRE(L.gated >= 0 && L.gated <= 2 && L.window >= 0, "hybrid_create: gated 0..2, window >= 0");
-            if (L.diff_maps || L.qk_head_norm || L.window > 0 || L.gated == 2) {
-                TL_REQUIRE(!L.qk_unit_rms && !L.qk_norm && L.v_mix == TL_VMIX_NONE && !L.talk_dev && !L.sink_dev && L.chunk == 0,
-                           "hybrid_create: per-head norms, maps, a window and per-head gates do not combine with unit-RMS heads, the whole-projection norm, value mixing, "
-                           "mixed scores, learned sinks or a chunked mask");
-                TL_REQUIRE(!L.qk_head_norm || (L.q_norm_dev && L.k_norm_dev), "hybrid_create: a norm per head needs its weights");
-                TL_REQUIRE(!L.diff_maps || !L.sink, "hybrid_create: differential attention takes no sink");
-            }
-            if (L.v_mix != TL_VMIX_NONE) {
-                if (vmix_width == 0) {
-                    TL_REQUIRE(L.v_mix == TL_VMIX_FIRST, "hybrid_create: the first value-mixing layer keeps its values (v_mix 1), later ones blend (v_mix 2)");
-                    vmix_width = L.kv_heads * L.vdim;
-                } else
-                    TL_REQUIRE(L.v_mix == TL_VMIX_BLEND && L.kv_heads * L.vdim == vmix_width, "hybrid_create: value-mixing layers share one values width");
-            }
-        } else if (L.kind == TL_MIX_LINREC) {
-            TL_REQUIRE(L.kv_heads == L.heads && (L.out_norm_dev || L.rec_kind == TL_REC_FIXED), "hybrid_create: a linear recurrence has one key head per head and an output norm weight");
-            if (L.rec_kind == TL_REC_FIXED)
-                TL_REQUIRE(L.decay_dev && L.rot_dims >= 0 && L.rot_dims % 2 == 0 && L.rot_dims <= L.dim, "hybrid_create: a constant decay needs its values; rot_dims even and at most dim");
-            else if (L.rec_kind == TL_REC_CHANNEL)
-                TL_REQUIRE(L.a_rank >= 1 && L.a2_dev && L.a2_bias_dev && L.tau > 0.f, "hybrid_create: channel decay needs its projection pair, bias and tau > 0");
-            else
-                TL_REQUIRE(L.rec_kind == TL_REC_EXPGATE && L.i_bias_dev && L.f_bias_dev && L.gate_cap > 0.f, "hybrid_create: exponential gates need biases and a cap > 0");
-        } else if (L.kind == TL_MIX_LATENT) {
-            TL_REQUIRE(L.q_rank >= 1 && L.kv_rank >= 1 && L.rot_dim >= 0 && L.dq_norm_dev && L.uq_dev && L.uk_t_dev && L.uv_dev,
-                       "hybrid_create: latent attention needs its ranks and per-head projections");
-            TL_REQUIRE(L.rot_dims >= 0 && L.rot_dims % 2 == 0 && L.rot_dims <= L.rot_dim, "hybrid_create: rot_dims must be even and at most rot_dim");
-            TL_REQUIRE(L.kv_rank + L.rot_dim <= 1024 && L.kv_rank <= 512, "hybrid_create: latent widths: kv_rank + rot_dim <= 1024, kv_rank <= 512");
-            if (L.kv_from >= 0) {
-                TL_REQUIRE(L.kv_from < i, "hybrid_create: kv_from must name an earlier layer");
-                const tl_hybrid_layer &J = e->layers[L.kv_from];
-                TL_REQUIRE(J.kind == TL_MIX_LATENT && J.kv_from < 0 && J.kv_rank == L.kv_rank && J.rot_dim == L.rot_dim,
-                           "hybrid_create: kv_from must name a latent-attention layer with its own latent of the same widths");
-            } else {
-                TL_REQUIRE(L.dkv_norm_dev, "hybrid_create: a latent of its own needs its norm weight");
-            }
-        } else {
-            TL_REQUIRE(L.conv_taps >= 1 && L.conv_taps <= 64 && L.conv_dev && L.a_log_dev && L.dt_bias_dev && L.out_norm_dev,
-                       "hybrid_create: a delta layer needs conv taps and weights, a_log, dt_bias and its output norm");
-        }
         const bool par = c.parallel_block == TL_BLOCK_PARALLEL;
-        max_in = std::max(max_in, par ? mixer_cols(L) + L.ff : std::max(mixer_cols(L), ff_in_cols(L)));
-        max_cat = std::max(max_cat, par ? L.heads * L.vdim + L.ff : std::max(L.heads * L.vdim, L.ff));
-        max_hv = std::max(max_hv, attn_maps(L) * L.heads * (L.vdim + 1));
-        max_gh = std::max(max_gh, L.heads);
+        max_in = std::max(max_in, par ? layer_mixer_cols(e.get(), i) + L.ff : std::max(layer_mixer_cols(e.get(), i), ff_in_cols(L)));
+        max_cat = std::max(max_cat, par ? layer_read_cols(e.get(), i) + L.ff : std::max(layer_read_cols(e.get(), i), L.ff));
         if (L.side_gate_dev) max_in = std::max(max_in, c.side_dim), max_cat = std::max(max_cat, c.side_dim);
-        if (L.kind == TL_MIX_ATTENTION) max_q = std::max(max_q, attn_maps(L) * L.heads * L.dim);
-        else if (L.kind == TL_MIX_LATENT) {
-            max_q = std::max(max_q, L.heads * (L.kv_rank + L.rot_dim));
-            max_c = std::max(max_c, L.heads * (L.dim + L.rot_dim));
-            max_da = std::max(max_da, std::max(L.q_rank, L.heads * L.kv_rank));
-            max_db = std::max(max_db, L.heads * L.dim);
-        } else if (L.kind == TL_MIX_LINREC) {
-            max_c = std::max(max_c, L.heads * L.dim);
-            max_da = std::max(max_da, L.a_rank);
-        } else max_c = std::max(max_c, conv_channels(L));
+        any_moe |= L.ff > 0 && L.ff_kind == TL_FF_MOE;
+        for (const tl_hybrid_layer *X : {&L, &B}) {
+            const tl_hybrid_layer &M = *X;
+            if (M.kind < 0) continue;
+            max_hv = std::max(max_hv, attn_maps(M) * M.heads * (M.vdim + 1));
+            max_gh = std::max(max_gh, M.heads);
+            if (M.kind == TL_MIX_ATTENTION) max_q = std::max(max_q, attn_maps(M) * M.heads * M.dim);
+            else if (M.kind == TL_MIX_LATENT) {
+                max_q = std::max(max_q, M.heads * (M.kv_rank + M.rot_dim));
+                max_c = std::max(max_c, M.heads * (M.dim + M.rot_dim));
+                max_da = std::max(max_da, std::max(M.q_rank, M.heads * M.kv_rank));
+                max_db = std::max(max_db, M.heads * M.dim);
+            } else if (M.kind == TL_MIX_LINREC) {
+                max_c = std::max(max_c, M.heads * M.dim);
+                max_da = std::max(max_da, M.a_rank);
+            } else max_c = std::max(max_c, conv_channels(M));
+        }
     }
     // layer runs
     for (int i = 0; i < c.num_layers;) {
@@ -1010,10 +1114,10 @@ extern "C" int tl_hybrid_create(const tl_hybrid_config *cfg, const tl_hybrid_lay
     }
     tl_hybrid *p = e.get();
     const size_t es = esize(c.dtype);
-    e->inv_freq.assign(c.num_layers, nullptr);
-    e->rot_mult.assign(c.num_layers, 1.f);
-    for (int i = 0; i < c.num_layers; ++i) {
-        const tl_hybrid_layer &L = e->layers[i];
+    e->inv_freq.assign(2 * c.num_layers, nullptr);
+    e->rot_mult.assign(2 * c.num_layers, 1.f);
+    for (int i = 0; i < 2 * c.num_layers; ++i) {
+        const tl_hybrid_layer &L = i % 2 ? e->beside[i / 2] : e->layers[i / 2];
         if (L.kind != TL_MIX_ATTENTION && L.kind != TL_MIX_LATENT && !(L.kind == TL_MIX_LINREC && L.rec_kind == TL_REC_FIXED)) continue;
         const int half = std::max(1, L.rot_dims / 2);
         std::vector<float> f(half, 0.f);
@@ -1047,14 +1151,16 @@ extern "C" int tl_hybrid_create(const tl_hybrid_config *cfg, const tl_hybrid_lay
         HY_TRY(dev_alloc(p, &e->inv_freq[i], half));
         HY_HIP(hipMemcpy(e->inv_freq[i], f.data(), half * 4, hipMemcpyHostToDevice));
     }
-    for (size_t ri = 0; ri < e->runs.size(); ++ri) {
-        Run &r = e->runs[ri];
-        const tl_hybrid_layer &L = e->layers[r.layer];
+    for (size_t rm = 0; rm < 2 * e->runs.size(); ++rm) {
+        const size_t ri = rm / 2;
+        MixState &r = e->runs[ri].mix[rm % 2];
+        const tl_hybrid_layer &L = rm % 2 ? e->beside[e->runs[ri].layer] : e->layers[e->runs[ri].layer];
+        if (L.kind < 0) continue;
         if (L.kind == TL_MIX_LATENT) {
             if (L.kv_from >= 0) {  // the pages of the latest earlier run of that layer (the same loop pass, or the last pass before)
                 for (size_t rj = ri; rj-- > 0;)
                     if (e->runs[rj].layer == L.kv_from) {
-                        r.kpool = e->runs[rj].kpool;
+                        r.kpool = e->runs[rj].mix[0].kpool;
                         break;
                     }
                 TL_REQUIRE(r.kpool, "hybrid_create: kv_from names a layer that has not run before this one");
@@ -1086,11 +1192,8 @@ extern "C" int tl_hybrid_create(const tl_hybrid_config *cfg, const tl_hybrid_lay
     e->ld_cat = (max_cat + 7) / 8 * 8;
     HY_TRY(dev_alloc(p, &e->x, (size_t)R * W));
     HY_TRY(dev_alloc(p, &e->x0, (size_t)R * W));
-    if (c.parallel_block == TL_BLOCK_POSTNORM) {
-        HY_TRY(dev_alloc(p, &e->y, (size_t)R * W));
-        HY_TRY(dev_alloc(p, &e->moe_mask, 1, true));
-    } else if (c.parallel_block == TL_BLOCK_SANDWICH)
-        HY_TRY(dev_alloc(p, &e->y, (size_t)R * W));
+    if (c.parallel_block == TL_BLOCK_POSTNORM || c.parallel_block == TL_BLOCK_SANDWICH) HY_TRY(dev_alloc(p, &e->y, (size_t)R * W));
+    if (any_moe) HY_TRY(dev_alloc(p, &e->moe_mask, 1, true));
     if (vmix_width > 0) HY_TRY(dev_alloc(p, &e->vref, (size_t)R * vmix_width));
     HY_TRY(dev_alloc(p, &e->proj, (size_t)R * e->ld_proj));
     HY_TRY(dev_alloc(p, &e->qbuf, (size_t)R * std::max(1, max_q)));
@@ -1102,9 +1205,11 @@ extern "C" int tl_hybrid_create(const tl_hybrid_config *cfg, const tl_hybrid_lay
     HY_TRY(dev_alloc(p, &e->obuf, (size_t)R * std::max(1, max_hv)));
     HY_TRY(dev_alloc(p, &e->logits, (size_t)R * c.vocab));
     int max_h = 1, max_v = 1;
-    for (const tl_hybrid_layer &L : e->layers)
+    for (int i = 0; i < 2 * c.num_layers; ++i) {
+        const tl_hybrid_layer &L = i % 2 ? e->beside[i / 2] : e->layers[i / 2];
         if (L.kind == TL_MIX_ATTENTION) max_h = std::max(max_h, attn_maps(L) * L.heads), max_v = std::max(max_v, L.vdim);
         else if (L.kind == TL_MIX_LATENT) max_h = std::max(max_h, L.heads), max_v = std::max(max_v, L.kv_rank);
+    }
     HY_TRY(dev_alloc(p, &e->part_acc, (size_t)c.max_slots * max_h * 64 * max_v));
     HY_TRY(dev_alloc(p, &e->part_ml, (size_t)c.max_slots * max_h * 64 * 2));
     if (const char *v = getenv("TL_HYBRID_ATTN_ROWS")) e->attn_rows_only = v[0] != '\0' && v[0] != '0';
@@ -1122,6 +1227,7 @@ extern "C" int tl_hybrid_create(const tl_hybrid_config *cfg, const tl_hybrid_lay
     HY_TRY(dev_alloc(p, &e->table_dev, (size_t)c.max_slots * c.max_pages_per_seq));
     HY_TRY(dev_alloc(p, &e->ctx_dev, (size_t)c.max_slots, true));
     HY_TRY(dev_alloc(p, &e->pending_dev, (size_t)c.max_slots, true));
+    HY_TRY(dev_alloc(p, &e->last_tok_dev, (size_t)c.max_slots, true));
     HY_TRY(dev_alloc(p, &e->argmax_dev, (size_t)R, true));
     e->stats.layer_runs = (int)e->runs.size();
     HY_HIP(hipDeviceSynchronize());
@@ -1151,8 +1257,9 @@ extern "C" int tl_hybrid_begin(tl_hybrid *e, int slot) {
     TL_REQUIRE(slot >= 0 && slot < e->cfg.max_slots, "hybrid_begin: slot out of range");
     TL_REQUIRE(!e->pool->live(slot), "hybrid_begin: slot is live");
     e->pool->begin(slot);
-    for (Run &r : e->runs) {  // the slot's recurrent state starts at zero (fill kernels: a caller may have a capture open on this stream)
-        const tl_hybrid_layer &L = e->layers[r.layer];
+    for (size_t rm = 0; rm < 2 * e->runs.size(); ++rm) {  // the slot's recurrent state starts at zero (fill kernels: a caller may have a capture open on this stream)
+        MixState &r = e->runs[rm / 2].mix[rm % 2];
+        const tl_hybrid_layer &L = rm % 2 ? e->beside[e->runs[rm / 2].layer] : e->layers[e->runs[rm / 2].layer];
         if (L.kind != TL_MIX_DELTA && L.kind != TL_MIX_LINREC) continue;
         const size_t sn = state_floats(L), cn = aux_floats(L);
         hipLaunchKernelGGL(fill_kernel, dim3((unsigned)std::min<size_t>(1024, (sn + 255) / 256)), dim3(256), 0, e->stream, r.state + slot * sn, sn, 0.f);
@@ -1175,13 +1282,15 @@ extern "C" int tl_hybrid_move(tl_hybrid *e, int src, int dst) {
     TL_REQUIRE(e, "hybrid: null engine");
     TL_REQUIRE(src >= 0 && src < e->cfg.max_slots && dst >= 0 && dst < e->cfg.max_slots && src != dst, "hybrid_move: slot out of range");
     TL_REQUIRE(e->pool->live(src) && !e->pool->live(dst), "hybrid_move: src must hold a sequence and dst must be free");
-    for (Run &r : e->runs) {  // recurrent state and convolution inputs travel with the sequence; K/V pages stay where they are
-        const tl_hybrid_layer &L = e->layers[r.layer];
+    for (size_t rm = 0; rm < 2 * e->runs.size(); ++rm) {  // recurrent state and convolution inputs travel with the sequence; K/V pages stay where they are
+        MixState &r = e->runs[rm / 2].mix[rm % 2];
+        const tl_hybrid_layer &L = rm % 2 ? e->beside[e->runs[rm / 2].layer] : e->layers[e->runs[rm / 2].layer];
         if (L.kind != TL_MIX_DELTA && L.kind != TL_MIX_LINREC) continue;
         const size_t sn = state_floats(L), cn = aux_floats(L);
         HY_HIP(hipMemcpyAsync(r.state + dst * sn, r.state + src * sn, sn * 4, hipMemcpyDeviceToDevice, e->stream));
         HY_HIP(hipMemcpyAsync(r.conv_state + dst * cn, r.conv_state + src * cn, cn * 4, hipMemcpyDeviceToDevice, e->stream));
     }
+    HY_HIP(hipMemcpyAsync(e->last_tok_dev + dst, e->last_tok_dev + src, 4, hipMemcpyDeviceToDevice, e->stream));
     int32_t tok = 0;
     HY_HIP(hipMemcpyAsync(&tok, e->pending_dev + src, 4, hipMemcpyDeviceToHost, e->stream));
     HY_HIP(hipStreamSynchronize(e->stream));
@@ -1241,6 +1350,11 @@ extern "C" int tl_hybrid_step(tl_hybrid *e, int n_seqs, const int *slots, const 
         ctx_bound = std::max(ctx_bound, e->pool->context(slots[i]) + lens[i]);
     }
     plan_splits(sh, ctx_bound);
+    if (c.pair_embed_dev) {
+        hipLaunchKernelGGL(seq_prev_kernel, dim3((n_seqs + 63) / 64), dim3(64), 0, e->stream, e->meta.tokens, e->meta.seq_row0, e->meta.seq_slot, n_seqs, e->meta.seq_prev,
+                           e->last_tok_dev);
+        TL_CHECK_LAUNCH("hybrid previous tokens");
+    }
     HY_TRY(forward(e, e->meta, sh));
     HY_TRY(head(e, e->meta, n_want, true));
     for (int i = 0; i < n_seqs; ++i) e->pool->advance(slots[i], lens[i]);
@@ -1300,12 +1414,12 @@ extern "C" int tl_hybrid_decode(tl_hybrid *e, int n_seqs, const int *slots, int 
     HY_HIP(hipStreamSynchronize(e->stream));
     auto one_step = [&]() -> int {
         hipLaunchKernelGGL(decode_meta_kernel, dim3((n_seqs + 63) / 64), dim3(64), 0, e->stream, e->dmeta.seq_slot, n_seqs, e->pending_dev, e->ctx_dev,
-                           e->dmeta.tokens, e->dmeta.row_pos, 0);
+                           e->dmeta.tokens, e->dmeta.row_pos, e->dmeta.seq_prev, e->last_tok_dev, 0);
         TL_CHECK_LAUNCH("hybrid decode meta");
         HY_TRY(forward(e, e->dmeta, sh));
         HY_TRY(head(e, e->dmeta, n_seqs, true));
         hipLaunchKernelGGL(decode_meta_kernel, dim3((n_seqs + 63) / 64), dim3(64), 0, e->stream, e->dmeta.seq_slot, n_seqs, e->pending_dev, e->ctx_dev,
-                           e->dmeta.tokens, e->dmeta.row_pos, 1);
+                           e->dmeta.tokens, e->dmeta.row_pos, e->dmeta.seq_prev, e->last_tok_dev, 1);
         TL_CHECK_LAUNCH("hybrid decode advance");
         return TL_OK;
     };

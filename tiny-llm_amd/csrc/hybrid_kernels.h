@@ -34,16 +34,43 @@ __device__ __forceinline__ float act_f(float z, int kind) {
         const float u = 0.79788456080286535588f * (z + 0.044715f * z * z * z);
         return z / (1.f + expf(-2.f * u));
     }
+    if (kind == 3) {
+        const float r = fmaxf(z, 0.f);
+        return r * r;
+    }
     return silu_f(z);
 }
+// a query's temperature at position pos: 1 + coef ln(floor((pos + 1) / every) + 1); coef 0: 1
+__device__ __forceinline__ float q_temperature(int pos, float coef, float every) {
+    return coef == 0.f ? 1.f : 1.f + coef * logf((float)floor((double)(pos + 1) / (double)every) + 1.f);
+}
 
-// ---- embedding gather: x0 = x = embed[token] * scale; with nw the row then passes an RMS norm, * (noffset + nw) ------
+// A second embedding table indexed by a hash of a token and the one before it (table NULL: none).  seq_prev: the last token each sequence of the step
+// was fed before this step; a sequence's first token takes the row behind the buckets.
+struct PairEmbed {
+    const void *table = nullptr;
+    long long buckets = 1, mul_prev = 0, mul_cur = 0;
+    const int32_t *row_seq = nullptr, *row_pos = nullptr, *seq_row0 = nullptr, *seq_prev = nullptr;
+};
+
+// ---- embedding gather: x0 = x = embed[token] * scale (+ the pair's row); with nw the row then passes an RMS norm, * (noffset + nw) ------
 template <typename D>
 __global__ void embed_kernel(const int32_t *tokens, const typename D::storage *embed, float *x0, float *x, int width, int vocab, float scale,
-                             const float *nw, float noffset, float eps) {
+                             const float *nw, float noffset, float eps, PairEmbed pe) {
     __shared__ float red[16];
     const int t = blockIdx.x;
     int tok = tokens[t];
+    const typename D::storage *pair = nullptr;
+    if (pe.table) {
+        const int s = pe.row_seq[t];
+        long long row = pe.buckets;
+        if (pe.row_pos[t] > 0) {
+            const int prev = t > pe.seq_row0[s] ? tokens[t - 1] : pe.seq_prev[s];
+            row = ((long long)prev * pe.mul_prev + (long long)tok * pe.mul_cur) % pe.buckets;
+            row = row < 0 ? row + pe.buckets : row;
+        }
+        pair = reinterpret_cast<const typename D::storage *>(pe.table) + (size_t)row * width;
+    }
     tok = tok < 0 ? 0 : (tok >= vocab ? vocab - 1 : tok);
     float inv = 1.f, keep[16];  // (the row's first 16 elements a thread stay in registers between the two passes)
     if (nw) {
@@ -51,11 +78,11 @@ __global__ void embed_kernel(const int32_t *tokens, const typename D::storage *e
 #pragma unroll
         for (int i = 0; i < 16; ++i) {
             const int c = threadIdx.x + i * blockDim.x;
-            keep[i] = c < width ? ld<D>(embed, (size_t)tok * width + c) * scale : 0.f;
+            keep[i] = c < width ? ld<D>(embed, (size_t)tok * width + c) * scale + (pair ? ld<D>(pair, c) : 0.f) : 0.f;
             ss += keep[i] * keep[i];
         }
         for (int c = threadIdx.x + 16 * blockDim.x; c < width; c += blockDim.x) {
-            const float v = ld<D>(embed, (size_t)tok * width + c) * scale;
+            const float v = ld<D>(embed, (size_t)tok * width + c) * scale + (pair ? ld<D>(pair, c) : 0.f);
             ss += v * v;
         }
         ss = block_sum(ss, red);
@@ -71,7 +98,7 @@ __global__ void embed_kernel(const int32_t *tokens, const typename D::storage *e
         }
     }
     for (int c = threadIdx.x + (nw ? 16 * blockDim.x : 0); c < width; c += blockDim.x) {
-        float v = ld<D>(embed, (size_t)tok * width + c) * scale;
+        float v = ld<D>(embed, (size_t)tok * width + c) * scale + (pair ? ld<D>(pair, c) : 0.f);
         if (nw) v = v * inv * (noffset + nw[c]);
         x0[(size_t)t * width + c] = v;
         x[(size_t)t * width + c] = v;
@@ -316,7 +343,8 @@ template <typename D>
 __global__ __launch_bounds__(64) void attn_prep_kernel(const float *proj, int ldp, const int32_t *row_seq, const int32_t *row_pos,
                                                        const int32_t *seq_slot, const int32_t *block_table, int max_pages, int page_size,
                                                        const float *inv_freq, int rot_dims, int unit_rms, float eps, int H, int G, int dim,
-                                                       int vdim, float *qbuf, typename D::storage *kpool, typename D::storage *vpool) {
+                                                       int vdim, float *qbuf, typename D::storage *kpool, typename D::storage *vpool, float temp_coef,
+                                                       float temp_every) {
     const int t = blockIdx.x, hh = blockIdx.y, lane = threadIdx.x;
     const int pos = row_pos[t], slot = seq_slot[row_seq[t]];
     const int page = block_table[(size_t)slot * max_pages + pos / page_size], in_page = pos % page_size;
@@ -357,7 +385,7 @@ __global__ __launch_bounds__(64) void attn_prep_kernel(const float *proj, int ld
         }
     }
     ss = wave_sum(ss);
-    const float inv = unit_rms ? 1.f / sqrtf(ss / (float)dim + eps) : 1.f;
+    const float inv = (unit_rms ? 1.f / sqrtf(ss / (float)dim + eps) : 1.f) * (is_q ? q_temperature(pos, temp_coef, temp_every) : 1.f);
 #pragma unroll
     for (int it = 0; it < 8; ++it) {
         const int p = lane + it * 64;
@@ -382,7 +410,8 @@ __global__ __launch_bounds__(64) void attn_rows_kernel(const float *qbuf, const 
                                                        const int32_t *row_seq, const int32_t *row_pos, const int32_t *seq_slot,
                                                        const int32_t *block_table, int max_pages, int page_size, int H, int G, int dim, int vdim,
                                                        float scale, int sink, const float *gate, int ldg, typename D::storage *out, int ldo, int v_row,
-                                                       int window, int vshare, int gate_per_head, float *out32) {
+                                                       int window, int vshare, int gate_per_head, float *out32, float softcap, const float *slopes,
+                                                       const float *sinks, float out_scale) {
     extern __shared__ float smem[];
     float *qs = smem;        // [dim]
     float *ps = smem + dim;  // [64]
@@ -393,7 +422,8 @@ __global__ __launch_bounds__(64) void attn_rows_kernel(const float *qbuf, const 
     const int32_t *bt = block_table + (size_t)slot * max_pages;
     for (int c = lane; c < dim; c += 64) qs[c] = qbuf[((size_t)t * H + h) * dim + c];
     __syncthreads();
-    float m = sink ? 0.f : -INFINITY, l = sink ? 1.f : 0.f;
+    float m = sink ? (sinks ? sinks[h] : 0.f) : -INFINITY, l = sink ? 1.f : 0.f;
+    const float slope = slopes ? slopes[h] : 0.f;
     float acc[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};  // vdim <= 512
     for (int kb = k_lo; kb <= pos; kb += 64) {
         const int j = kb + lane;
@@ -403,6 +433,8 @@ __global__ __launch_bounds__(64) void attn_rows_kernel(const float *qbuf, const 
             float d = 0.f;
             for (int c = 0; c < dim; ++c) d += qs[c] * D::to_float(kr[c]);
             s = d * scale;
+            if (softcap > 0.f) s = softcap * tanhf(s / softcap);
+            s -= slope * (float)(pos - j);
         }
         const float m_new = fmaxf(m, wave_max(s));
         const float p = (j <= pos) ? expf(s - m_new) : 0.f;
@@ -426,7 +458,7 @@ __global__ __launch_bounds__(64) void attn_rows_kernel(const float *qbuf, const 
             }
         }
     }
-    const float invl = l > 0.f ? 1.f / l : 0.f;
+    const float invl = l > 0.f ? out_scale / l : 0.f;
 #pragma unroll
     for (int i = 0; i < 8; ++i) {
         const int c = lane + i * 64;
@@ -449,16 +481,27 @@ __global__ __launch_bounds__(64) void attn_rows_kernel(const float *qbuf, const 
 //                                 step r is key 4 g + r of the 16-key sub-tile (a sum does not care in which order its terms are paired)
 // Per query row (= per lane column) a running maximum and sum; the sink is their start value (0, 1).  The key range may be split over
 // gridDim.z (decode steps over long contexts): then unnormalised partial sums + (max, sum) go to part_* and attn_merge_kernel finishes.
+// EXT, in order: the score's cap (s <- softcap tanh(s / softcap)), a distance bias per head (s -= slopes[h] (i - j)), learned sinks (the start value of
+// the running maximum), a factor on the read-out.
+// tanh of a capped score: with bfloat16 pages through one hardware exponential (absolute error ~1e-7; the score comes from 8-bit mantissas)
+template <bool FAST>
+__device__ __forceinline__ float tanh_t(float x) {
+    if constexpr (FAST) return 1.f - 2.f / (1.f + __expf(2.f * x));
+    else return tanhf(x);
+}
 template <typename D, int DK4, int VT, bool WSPLIT, bool EXT>
 __global__ __launch_bounds__(256) void attn_tile_kernel(const float *qbuf, const typename D::storage *kpool, const typename D::storage *vpool,
                                                         const int32_t *seq_row0, const int32_t *seq_slot, const int32_t *row_pos,
                                                         const int32_t *block_table, int max_pages, int page_size, int H, int G, int dim, int vdim,
                                                         float scale, int sink, int HGB, int n_hblk, int keys_per_split, int n_splits, const float *gate,
                                                         int ldg, typename D::storage *out, int ldo, float *part_acc, float *part_ml, int page_shift,
-                                                        int vec_ok, int v_row, int window_, int vshare_, int gate_per_head_, float *out32_) {
+                                                        int vec_ok, int v_row, int window_, int vshare_, int gate_per_head_, float *out32_,
+                                                        float softcap_, const float *slopes_, const float *sinks_, float out_scale_) {
     using S = typename D::storage;
     extern __shared__ float smem[];
-    // EXT false: plain causal attention into D rows, the four options folded away at compile time
+    // EXT false: plain causal attention into D rows, the options folded away at compile time
+    const float softcap = EXT ? softcap_ : 0.f, out_scale = EXT ? out_scale_ : 1.f;
+    const float *const slopes = EXT ? slopes_ : nullptr, *const sinks = EXT ? sinks_ : nullptr;
     const int window = EXT ? window_ : 0, vshare = EXT ? vshare_ : 1, gate_per_head = EXT ? gate_per_head_ : 0;
     float *const out32 = EXT ? out32_ : nullptr;
     // window > 0: a query sees key j <= its position only if position - j < window; the walk starts at the first key the tile's first row sees,
@@ -491,7 +534,8 @@ __global__ __launch_bounds__(256) void attn_tile_kernel(const float *qbuf, const
     const bool row_ok = t0 + tl < len && hb < HG;
     const int trow = r0 + t0 + tl, head = kvh * HG + hb, qpos = pos0 + t0 + tl;
     const bool owns_sink = sink && split == 0 && (!WSPLIT || wave == 0);
-    float m_run = owns_sink ? 0.f : -INFINITY, l_run = owns_sink ? 1.f : 0.f;
+    const float slope = (slopes && row_ok) ? slopes[head] : 0.f, inv_cap = softcap > 0.f ? 1.f / softcap : 0.f;
+    float m_run = owns_sink ? (sinks && row_ok ? sinks[head] : 0.f) : -INFINITY, l_run = owns_sink ? 1.f : 0.f;
     f32x4 o[VT];
 #pragma unroll
     for (int v = 0; v < VT; ++v) o[v] = f32x4{0.f, 0.f, 0.f, 0.f};
@@ -607,6 +651,8 @@ __global__ __launch_bounds__(256) void attn_tile_kernel(const float *qbuf, const
 #pragma unroll
                 for (int r = 0; r < 4; ++r) {
                     const int j = kb + 16 * n + 4 * g4 + r;
+                    if (softcap > 0.f) a4[r] = softcap * tanh_t<KB16>(a4[r] * inv_cap);
+                    if (slopes) a4[r] -= slope * (float)(qpos - j);
                     a4[r] = (row_ok && j <= qpos && j < k_end && (window <= 0 || qpos - j < window)) ? a4[r] : -INFINITY;
                     m_tile = fmaxf(m_tile, a4[r]);
                 }
@@ -679,7 +725,7 @@ __global__ __launch_bounds__(256) void attn_tile_kernel(const float *qbuf, const
     }
     if (!row_ok) return;
     if (n_splits == 1) {
-        const float invl = l_run > 0.f ? 1.f / l_run : 0.f;
+        const float invl = l_run > 0.f ? out_scale / l_run : 0.f;
 #pragma unroll
         for (int v = 0; v < VT; ++v)
 #pragma unroll
@@ -712,7 +758,7 @@ __global__ __launch_bounds__(256) void attn_tile_kernel(const float *qbuf, const
 // sum and the weights exp(m_s - M); then the lanes turn to the value columns and walk the splits with those weights.
 template <typename D>
 __global__ __launch_bounds__(64) void attn_merge_kernel(const float *part_acc, const float *part_ml, int n_splits, int H, int vdim, const float *gate,
-                                                        int ldg, typename D::storage *out, int ldo, int gate_per_head, float *out32) {
+                                                        int ldg, typename D::storage *out, int ldo, int gate_per_head, float *out32, float out_scale) {
     __shared__ float ws[64];
     const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
     const size_t p0 = ((size_t)t * H + h) * n_splits;
@@ -723,7 +769,7 @@ __global__ __launch_bounds__(64) void attn_merge_kernel(const float *part_acc, c
     const float L = wave_sum(l * w);
     ws[lane] = w;
     __syncthreads();
-    const float invl = L > 0.f ? 1.f / L : 0.f;
+    const float invl = L > 0.f ? out_scale / L : 0.f;
     for (int c = lane; c < vdim; c += 64) {
         float acc = 0.f;
 #pragma unroll 8
@@ -745,7 +791,8 @@ template <typename D>
 __global__ __launch_bounds__(64) void attn_prep_head_kernel(const float *proj, int ldp, const int32_t *row_seq, const int32_t *row_pos, const int32_t *seq_slot,
                                                             const int32_t *block_table, int max_pages, int page_size, const float *inv_freq, int rot_dims,
                                                             int rot_half, int head_norm, const float *qw, const float *kw, float eps, int H, int G, int M, int dim,
-                                                            int vdim, float *qbuf, typename D::storage *kpool, typename D::storage *vpool, const float *bias) {
+                                                            int vdim, float *qbuf, typename D::storage *kpool, typename D::storage *vpool, const float *bias,
+                                                            float temp_coef, float temp_every) {
     const int t = blockIdx.x, hh = blockIdx.y, lane = threadIdx.x;
     const int pos = row_pos[t], slot = seq_slot[row_seq[t]];
     const int page = block_table[(size_t)slot * max_pages + pos / page_size], in_page = pos % page_size;
@@ -779,6 +826,7 @@ __global__ __launch_bounds__(64) void attn_prep_head_kernel(const float *proj, i
         qdst = qbuf + ((size_t)t * HM + ((size_t)(h / HG) * M + mp) * HG + h % HG) * dim;
     } else
         kdst = kpool + (((size_t)page * GM + (hh - HM)) * page_size + in_page) * dim;
+    const float temp = is_q ? q_temperature(pos, temp_coef, temp_every) : 1.f;
     const int half = rot_dims / 2, units = dim - half;  // `half` rotation pairs, then the dimensions that pass
     for (int u = lane; u < units; u += 64) {
         int c0, c1 = -1;
@@ -793,8 +841,8 @@ __global__ __launch_bounds__(64) void attn_prep_head_kernel(const float *proj, i
             a = na, b2 = nb;
         }
         if (is_q) {
-            qdst[c0] = a;
-            if (c1 >= 0) qdst[c1] = b2;
+            qdst[c0] = a * temp;
+            if (c1 >= 0) qdst[c1] = b2 * temp;
         } else {
             kdst[c0] = D::from_float(a);
             if (c1 >= 0) kdst[c1] = D::from_float(b2);
@@ -839,7 +887,7 @@ __global__ __launch_bounds__(1024) void attn_prep_row_kernel(const float *proj, 
                                                             const int32_t *block_table, int max_pages, int page_size, const float *inv_freq, int rot_dims,
                                                             int rot_half, int qk_norm, const float *qw, const float *kw, float eps, int H, int G, int dim, int vdim,
                                                             int v_mix, float lambda, float *vref, float *qbuf, typename D::storage *kpool,
-                                                            typename D::storage *vpool) {
+                                                            typename D::storage *vpool, float temp_coef, float temp_every) {
     __shared__ float red[16];
     const int t = blockIdx.x, tid = threadIdx.x;
     const int pos = row_pos[t], slot = seq_slot[row_seq[t]];
@@ -856,6 +904,7 @@ __global__ __launch_bounds__(1024) void attn_prep_row_kernel(const float *proj, 
         inv_q = 1.f / sqrtf(sq / (float)nq + eps);
         inv_k = 1.f / sqrtf(sk / (float)nk + eps);
     }
+    const float temp = q_temperature(pos, temp_coef, temp_every);
     const int half = rot_dims / 2, units = dim - half;  // per head: `half` rotation pairs, then the dimensions that pass
     for (int e = tid; e < (H + G) * units; e += blockDim.x) {
         const int hh = e / units, u = e % units;
@@ -876,8 +925,8 @@ __global__ __launch_bounds__(1024) void attn_prep_row_kernel(const float *proj, 
         }
         if (is_q) {
             float *dst = qbuf + (size_t)t * nq + (size_t)hh * dim;
-            dst[c0] = a;
-            if (c1 >= 0) dst[c1] = b2;
+            dst[c0] = a * temp;
+            if (c1 >= 0) dst[c1] = b2 * temp;
         } else {
             typename D::storage *dst = kpool + (((size_t)page * G + (hh - H)) * page_size + in_page) * dim;
             dst[c0] = D::from_float(a);
@@ -1397,9 +1446,12 @@ __global__ void cast_rows_kernel(const float *x, typename D::storage *out, size_
     const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
     if (i < n) out[i] = D::from_float(x[i]);
 }
-__global__ void scale_kernel(float *x, float a, size_t n) {
+// logits: x <- x * a, then (cap > 0) cap tanh(x / cap)
+__global__ void logit_scale_kernel(float *x, float a, float cap, size_t n) {
     const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
-    if (i < n) x[i] *= a;
+    if (i >= n) return;
+    const float v = x[i] * a;
+    x[i] = cap > 0.f ? cap * tanhf(v / cap) : v;
 }
 
 // ---- feed-forward activation: cat[t, col0 + c] = act(proj[t, up0 + c]) ---------------------------------------------------
@@ -1603,13 +1655,13 @@ __global__ __launch_bounds__(256) void delta_kernel(const float *qkv, int C, con
 // ---- read-out of the delta rule: per (row, head) o / rms(o) * w * silu(gate) -> cat columns h*vdim .. ----------------------
 template <typename D>
 __global__ __launch_bounds__(64) void delta_out_kernel(const float *obuf, const float *w, float eps, const float *gate, int ldg, int H, int vdim,
-                                                       typename D::storage *out, int ldo) {
+                                                       typename D::storage *out, int ldo, float out_scale) {
     const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
     const float *o = obuf + ((size_t)t * H + h) * vdim;
     float ss = 0.f;
     for (int c = lane; c < vdim; c += 64) ss += o[c] * o[c];
     ss = wave_sum(ss);
-    const float inv = 1.f / sqrtf(ss / (float)vdim + eps);
+    const float inv = out_scale / sqrtf(ss / (float)vdim + eps);
     for (int c = lane; c < vdim; c += 64)
         out[(size_t)t * ldo + (size_t)h * vdim + c] = D::from_float(o[c] * inv * w[c] * silu_f(gate[(size_t)t * ldg + (size_t)h * vdim + c]));
 }
@@ -1635,13 +1687,13 @@ __global__ void rms_cols_kernel(const float *in, int ldi, int n, const float *w,
     for (int c = threadIdx.x; c < n; c += blockDim.x) out[(size_t)t * ldo + c] = D::from_float(src[c] * inv * w[c]);
 }
 
-// ---- latent attention, step 1.  Queries q [rows, H, dim + rot] (float32): the plain part -> qn (D, the input of the per-head key
+// ---- latent attention, step 1.  Queries q [rows of ldq; H, dim + rot] (float32): the plain part -> qn (D, the input of the per-head key
 // absorption), the rotated part -> qbuf[t, h, rank ..] after its rotation.  With own_kv (the layer has its own latent projection, columns
 // kv0 .. of proj: rank latent columns, then rot columns of one rotated key part shared by all heads): the latent is RMS-normed with
 // its weight and appended to the sequence's page row [c (rank) | rotated key part (rot)] -- the whole K/V cache of the layer.
 // Rotation: pair (2i, 2i+1) by pos * freq[i], cos and sin times mult.  grid (rows, H + 1), one wave each.
 template <typename D>
-__global__ __launch_bounds__(64) void latent_prep_kernel(const float *q, int H, int dim, int rot, int rank, const float *proj, int ldp, int kv0,
+__global__ __launch_bounds__(64) void latent_prep_kernel(const float *q, int ldq, int H, int dim, int rot, int rank, const float *proj, int ldp, int kv0,
                                                          const float *c_norm, float eps, int own_kv, const int32_t *row_seq, const int32_t *row_pos,
                                                          const int32_t *seq_slot, const int32_t *block_table, int max_pages, int page_size,
                                                          const float *freq, int rot_dims, float mult, typename D::storage *qn, float *qbuf,
@@ -1660,7 +1712,7 @@ __global__ __launch_bounds__(64) void latent_prep_kernel(const float *q, int H, 
         }
     };
     if (hh < H) {
-        const float *src = q + ((size_t)t * H + hh) * (dim + rot);
+        const float *src = q + (size_t)t * ldq + (size_t)hh * (dim + rot);
         for (int c = lane; c < dim; c += 64) qn[((size_t)t * H + hh) * dim + c] = D::from_float(src[c]);
         float *dst = qbuf + ((size_t)t * H + hh) * (rank + rot) + rank;
         for (int p = lane; 2 * p < rot; p += 64) {
@@ -1689,14 +1741,16 @@ __global__ __launch_bounds__(64) void latent_prep_kernel(const float *q, int H, 
     }
 }
 
-// ---- out[t, c] = in[t, c] * gate(g[t, c]) as D rows.  kind 0: sigmoid, 1: SiLU, 2: no gate (g is not read) ----------------------------
+// ---- out[t, c] = in[t, c] * gate(g[t, c / per]) * scale as D rows.  kind 0: sigmoid, 1: SiLU, 2: no gate (g is not read).  per: columns of one gate
+// number (1, or a head's width) ----------------------------
 template <typename D>
-__global__ void gate_mul_kernel(const float *in, int ldi, const float *g, int ldg, int n, int kind, typename D::storage *out, int ldo, int rows) {
+__global__ void gate_mul_kernel(const float *in, int ldi, const float *g, int ldg, int n, int kind, int per, float scale, typename D::storage *out, int ldo,
+                                int rows) {
     const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
     if (i >= (size_t)rows * n) return;
     const int t = (int)(i / n), c = (int)(i % n);
-    const float z = kind == 2 ? 0.f : g[(size_t)t * ldg + c];
-    out[(size_t)t * ldo + c] = D::from_float(in[(size_t)t * ldi + c] * (kind == 2 ? 1.f : (kind == 0 ? sigmoid_f(z) : silu_f(z))));
+    const float z = kind == 2 ? 0.f : g[(size_t)t * ldg + c / per];
+    out[(size_t)t * ldo + c] = D::from_float(in[(size_t)t * ldi + c] * scale * (kind == 2 ? 1.f : (kind == 0 ? sigmoid_f(z) : silu_f(z))));
 }
 
 // ---- gated feed-forward activation: cat[t, col0 + c] = act(proj[t, g0 + c]) * proj[t, u0 + c] ------------------------------------
@@ -1773,10 +1827,11 @@ __global__ void cast_cols_kernel(const float *in, int ldi, int c0, int n, typena
 // ones != 0 appends one column whose value is 1 for every token: it carries the normaliser n_t = a n + b k, read out as n_t . q_t.
 // grid (heads, sequences, blocks of 256 / LPC columns), 256 threads; LPC lanes share a column, RPT key rows each in registers (as delta_kernel).
 // q | k | v at columns q0 | k0 | v0 of proj (head-major).  State [slot, head, column, key_dim].  obuf [rows, H, VE], VE = vdim + ones.
+// fixed (CHAN false): a_t = fixed[h] for every token and b_t = 1 (gates is not read).  silu: bit 0 puts q and k through SiLU, bit 1 v.  k_mul: factor on k.
 template <int RPT, int LPC, bool CHAN>
 __global__ __launch_bounds__(256) void linrec_kernel(const float *proj, int ldp, int q0, int k0, int v0, const float *gates, const float *decay,
                                                      const int32_t *seq_row0, const int32_t *seq_slot, float *state, float *obuf, int H, int dim,
-                                                     int vdim, int ones) {
+                                                     int vdim, int ones, const float *fixed, int silu, float k_mul) {
     constexpr int DP = LPC * RPT, CPB = 256 / LPC;
     constexpr int TB = 4096 / DP < 32 ? 4096 / DP : 32;
     __shared__ __attribute__((aligned(16))) float qs[TB * DP], ks[TB * DP], as[CHAN ? TB * DP : TB];
@@ -1810,8 +1865,8 @@ __global__ __launch_bounds__(256) void linrec_kernel(const float *proj, int ldp,
             rv[it] = (tt < nt && c < VE) ? (c < vdim ? proj[(size_t)(r0 + t0 + tt) * ldp + v0 + (size_t)h * vdim + c] : 1.f) : 0.f;
         }
         if (tid < nt) {
-            if constexpr (!CHAN) rg = gates[((size_t)(r0 + t0 + tid) * H + h) * 3];
-            rb = CHAN ? 1.f : gates[((size_t)(r0 + t0 + tid) * H + h) * 3 + 1];
+            if constexpr (!CHAN) rg = fixed ? fixed[h] : gates[((size_t)(r0 + t0 + tid) * H + h) * 3];
+            rb = (CHAN || fixed) ? 1.f : gates[((size_t)(r0 + t0 + tid) * H + h) * 3 + 1];
         }
     };
     if (n > 0) fetch(0);
@@ -1820,13 +1875,13 @@ __global__ __launch_bounds__(256) void linrec_kernel(const float *proj, int ldp,
         __syncthreads();  // the previous tile's recurrence is done with the LDS
 #pragma unroll
         for (int it = 0; it < NIT; ++it) {
-            qs[tid + 256 * it] = rq[it];
-            ks[tid + 256 * it] = rk[it];
+            qs[tid + 256 * it] = (silu & 1) ? silu_f(rq[it]) : rq[it];  // (silu(0) = 0: padding stays zero)
+            ks[tid + 256 * it] = ((silu & 1) ? silu_f(rk[it]) : rk[it]) * k_mul;
             if constexpr (CHAN) as[tid + 256 * it] = ra[it];
         }
 #pragma unroll
         for (int it = 0; it < NV; ++it)
-            if (tid + 256 * it < TB * CPB) vs[tid + 256 * it] = rv[it];
+            if (tid + 256 * it < TB * CPB) vs[tid + 256 * it] = (silu & 2) ? silu_f(rv[it]) : rv[it];
         if (tid < TB) {
             if constexpr (!CHAN) as[tid] = rg;
             bs[tid] = rb;
@@ -1892,10 +1947,10 @@ __global__ __launch_bounds__(256) void linrec_kernel(const float *proj, int ldp,
 }
 
 // Constant decay per head (retention), ahead of the recurrence: q and k of every (row, head) turn in place (float32 columns q0 / k0 of proj) on their
-// first rot_dims dimensions by pos * inv_freq[i] -- pairs (i, i + rot_dims/2) with rot_half, (2i, 2i+1) without -- then k is multiplied by k_scale;
-// gates[t, h] = (decay[h], 1, -).  One wave per (row, head).
+// first rot_dims dimensions by pos * inv_freq[i] -- pairs (i, i + rot_dims/2) with rot_half, (2i, 2i+1) without -- after SiLU with `silu`, then k is
+// multiplied by k_scale.  One wave per (row, head).
 __global__ __launch_bounds__(64) void fixed_decay_prep_kernel(float *proj, int ldp, int q0, int k0, const int32_t *row_pos, const float *inv_freq, int rot_dims,
-                                                              int rot_half, float k_scale, const float *decay, float *gates, int H, int dim) {
+                                                              int rot_half, float k_scale, int silu, int H, int dim) {
     const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
     const int pos = row_pos[t], half = rot_dims / 2;
     float *q = proj + (size_t)t * ldp + q0 + (size_t)h * dim, *k = proj + (size_t)t * ldp + k0 + (size_t)h * dim;
@@ -1904,15 +1959,14 @@ __global__ __launch_bounds__(64) void fixed_decay_prep_kernel(float *proj, int l
             const int c0 = rot_half ? u : 2 * u, c1 = rot_half ? u + half : 2 * u + 1;
             float sn, cs;
             sincosf((float)pos * inv_freq[u], &sn, &cs);
-            const float qa = q[c0], qb = q[c1], ka = k[c0], kb = k[c1];
+            float qa = q[c0], qb = q[c1], ka = k[c0], kb = k[c1];
+            if (silu) qa = silu_f(qa), qb = silu_f(qb), ka = silu_f(ka), kb = silu_f(kb);
             q[c0] = qa * cs - qb * sn, q[c1] = qb * cs + qa * sn;
             k[c0] = (ka * cs - kb * sn) * k_scale, k[c1] = (kb * cs + ka * sn) * k_scale;
-        } else
-            k[u + half] *= k_scale;
-    }
-    if (lane == 0) {
-        float *g = gates + ((size_t)t * H + h) * 3;
-        g[0] = decay[h], g[1] = 1.f, g[2] = 0.f;
+        } else {
+            k[u + half] = (silu ? silu_f(k[u + half]) : k[u + half]) * k_scale;
+            if (silu) q[u + half] = silu_f(q[u + half]);
+        }
     }
 }
 
@@ -1921,7 +1975,7 @@ __global__ __launch_bounds__(64) void fixed_decay_prep_kernel(float *proj, int l
 template <typename D>
 __global__ __launch_bounds__(64) void linrec_out_kernel(const float *obuf, int VE, int ones, const float *gates, float qscale, const float *w,
                                                         int w_stride, float eps, const float *gate, int ldg, int gate_kind, int H, int vdim,
-                                                        typename D::storage *out, int ldo) {
+                                                        typename D::storage *out, int ldo, float out_scale) {
     const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
     const float *o = obuf + ((size_t)t * H + h) * VE;
     float mul = qscale;
@@ -1932,10 +1986,27 @@ __global__ __launch_bounds__(64) void linrec_out_kernel(const float *obuf, int V
         ss += v * v;
     }
     ss = wave_sum(ss);
-    const float inv = mul / sqrtf(ss / (float)vdim + eps);
+    const float inv = out_scale * mul / sqrtf(ss / (float)vdim + eps);
     for (int c = lane; c < vdim; c += 64) {
         const float z = gate[(size_t)t * ldg + (size_t)h * vdim + c];
         out[(size_t)t * ldo + (size_t)h * vdim + c] = D::from_float(o[c] * inv * (w ? w[(size_t)h * w_stride + c] : 1.f) * (gate_kind == 0 ? sigmoid_f(z) : silu_f(z)));
+    }
+}
+
+// the same with one norm over all heads, a workgroup per row: o / sqrt(mean over n = H * vdim columns + eps) * w[c] * gate(g) * out_scale
+template <typename D>
+__global__ void linrec_out_joint_kernel(const float *obuf, const float *w, float eps, const float *gate, int ldg, int gate_kind, int n,
+                                        typename D::storage *out, int ldo, float out_scale) {
+    __shared__ float red[16];
+    const int t = blockIdx.x;
+    const float *o = obuf + (size_t)t * n;
+    float ss = 0.f;
+    for (int c = threadIdx.x; c < n; c += blockDim.x) ss += o[c] * o[c];
+    ss = block_sum(ss, red);
+    const float inv = out_scale / sqrtf(ss / (float)n + eps);
+    for (int c = threadIdx.x; c < n; c += blockDim.x) {
+        const float z = gate[(size_t)t * ldg + c];
+        out[(size_t)t * ldo + c] = D::from_float(o[c] * inv * (w ? w[c] : 1.f) * (gate_kind == 0 ? sigmoid_f(z) : silu_f(z)));
     }
 }
 
@@ -1947,15 +2018,16 @@ __global__ __launch_bounds__(64) void linrec_out_kernel(const float *obuf, int V
 // cat row: [ sigmoid(sg) * relu(up)^2  (ffs) | w_e * relu(up_e)^2 (ffe each; 0 for experts not taken) ].
 // the router of one row, by every thread of a 256-thread workgroup: scores s = softmax(z) or sigmoid(z) (router 0 / 1); choice = s + correction
 // (NULL: 0); groups, kept groups, the `top` largest choices (ties: the lower index).  Leaves sw[e] = s_e for the experts taken, 0 for the others.
-__device__ __forceinline__ void moe_route_row(const float *row, int r0, int ET, int top, int groups, int keep, const float *correction, int router, float *sw,
-                                              float *sc, float *gm) {
+// bias (NULL: none) is added to the logits.  router 2: s = z, and the weights are the softmax over the chosen experts' logits only.
+__device__ __forceinline__ void moe_route_row(const float *row, int r0, int ET, int top, int groups, int keep, const float *correction, const float *bias, int router,
+                                              float *sw, float *sc, float *gm) {
     const int tid = threadIdx.x;
     if (tid < 64) {  // one wave scores (ET <= 256: four experts a lane at most)
         float z[4], mx = -INFINITY;
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
             const int e = tid + 64 * i;
-            z[i] = e < ET ? row[r0 + e] : -INFINITY;
+            z[i] = e < ET ? row[r0 + e] + (bias ? bias[e] : 0.f) : -INFINITY;
             mx = fmaxf(mx, z[i]);
         }
         float sum = 1.f;
@@ -1968,7 +2040,7 @@ __device__ __forceinline__ void moe_route_row(const float *row, int r0, int ET, 
                 sum += z[i];
             }
             sum = wave_sum(sum);
-        } else {
+        } else if (router == 1) {
 #pragma unroll
             for (int i = 0; i < 4; ++i) z[i] = (tid + 64 * i) < ET ? sigmoid_f(z[i]) : 0.f;
         }
@@ -1999,27 +2071,39 @@ __device__ __forceinline__ void moe_route_row(const float *row, int r0, int ET, 
     }
     __syncthreads();
     float wgt = 0.f;
+    bool taken = false;
     if (tid < ET) {
         const float c = sc[tid];
         int rank = 0;
         for (int o = 0; o < ET; ++o) rank += (sc[o] > c) || (sc[o] == c && o < tid);
-        wgt = (rank < top && !(c == -INFINITY)) ? sw[tid] : 0.f;
+        taken = rank < top && !(c == -INFINITY);
+        wgt = taken ? sw[tid] : 0.f;
     }
     __syncthreads();
+    if (router == 2) {  // softmax over the taken: the others leave the sum as -inf
+        if (tid < ET) sc[tid] = taken ? wgt : -INFINITY;
+        __syncthreads();
+        if (taken) {
+            float mx = -INFINITY, sum = 0.f;
+            for (int o = 0; o < ET; ++o) mx = fmaxf(mx, sc[o]);
+            for (int o = 0; o < ET; ++o) sum += expf(sc[o] - mx);
+            wgt = expf(wgt - mx) / sum;
+        }
+    }
     if (tid < ET) sw[tid] = wgt;
     __syncthreads();
 }
 
 template <typename D>
 __global__ __launch_bounds__(256) void moe_route_act_kernel(const float *proj, int ldp, int r0, int sg0, int su0, int eu0, int experts, int identity, int top,
-                                                            int groups, int keep, int ffe, int ffs, const float *correction,
+                                                            int groups, int keep, int ffe, int ffs, const float *correction, const float *bias,
                                                             typename D::storage *out, int ldo, int col0, float *idw, int router) {
     __shared__ float sw[256], sc[256];
     __shared__ float gm[256];
     // blockIdx.y: a share of the row's columns (every share routes the row again: a few dozen comparisons against thousands of columns)
     const int t = blockIdx.x, tid = threadIdx.x, ET = experts + identity;
     const float *row = proj + (size_t)t * ldp;
-    moe_route_row(row, r0, ET, top, groups, keep, correction, router, sw, sc, gm);
+    moe_route_row(row, r0, ET, top, groups, keep, correction, bias, router, sw, sc, gm);
     if (tid == 0 && blockIdx.y == 0) {
         float a = 0.f;
         for (int e = experts; e < ET; ++e) a += sw[e];
@@ -2036,14 +2120,14 @@ __global__ __launch_bounds__(256) void moe_route_act_kernel(const float *proj, i
 // which experts the rows of a small step take: bit e of *mask is set when some row's router takes expert e (the products around the activation then leave the
 // others out, see SegSkip).  One workgroup; experts <= 64.
 __global__ __launch_bounds__(256) void moe_taken_mask_kernel(const float *proj, int ldp, int r0, int rows, int experts, int identity, int top, int groups, int keep,
-                                                             const float *correction, int router, unsigned long long *mask) {
+                                                             const float *correction, const float *bias, int router, unsigned long long *mask) {
     __shared__ float sw[256], sc[256];
     __shared__ float gm[256];
     __shared__ unsigned long long taken;
     if (threadIdx.x == 0) taken = 0ull;
     __syncthreads();
     for (int t = 0; t < rows; ++t) {
-        moe_route_row(proj + (size_t)t * ldp, r0, experts + identity, top, groups, keep, correction, router, sw, sc, gm);
+        moe_route_row(proj + (size_t)t * ldp, r0, experts + identity, top, groups, keep, correction, bias, router, sw, sc, gm);
         if ((int)threadIdx.x < experts && sw[threadIdx.x] != 0.f) atomicOr(&taken, 1ull << threadIdx.x);
         __syncthreads();
     }
@@ -2055,13 +2139,13 @@ __global__ __launch_bounds__(256) void moe_taken_mask_kernel(const float *proj, 
 // cat row: [ shared (ffs) | expert columns (ffe each; 0 for experts not taken) ].
 template <typename D>
 __global__ __launch_bounds__(256) void moe_gated_act_kernel(const float *proj, int ldp, int r0, int sg0, int g0, int u0, int experts, int identity, int top,
-                                                            int groups, int keep, int ffe, int ffs, const float *correction, typename D::storage *out,
-                                                            int ldo, int col0, float *idw, int router, int scale_input, int act) {
+                                                            int groups, int keep, int ffe, int ffs, const float *correction, const float *bias,
+                                                            typename D::storage *out, int ldo, int col0, float *idw, int router, int scale_input, int act) {
     __shared__ float sw[256], sc[256];
     __shared__ float gm[256];
     const int t = blockIdx.x, tid = threadIdx.x, ET = experts + identity;
     const float *row = proj + (size_t)t * ldp;
-    moe_route_row(row, r0, ET, top, groups, keep, correction, router, sw, sc, gm);
+    moe_route_row(row, r0, ET, top, groups, keep, correction, bias, router, sw, sc, gm);
     if (tid == 0 && blockIdx.y == 0) {
         float a = 0.f;
         for (int e = experts; e < ET; ++e) a += sw[e];
@@ -2132,8 +2216,9 @@ __global__ __launch_bounds__(1024) void argmax_kernel(const float *logits, int v
     }
 }
 // decode bookkeeping on the device: the step's rows are one token per listed slot; tokens come from `pending`, positions from `ctx`
+// seq_prev: the token each sequence was fed last (last_tok, by slot), which this step's token replaces
 __global__ void decode_meta_kernel(const int32_t *slots, int n, const int32_t *pending, int32_t *ctx, int32_t *tokens, int32_t *row_pos,
-                                   int advance) {
+                                   int32_t *seq_prev, int32_t *last_tok, int advance) {
     const int i = blockIdx.x * blockDim.x + threadIdx.x;
     if (i >= n) return;
     const int s = slots[i];
@@ -2141,7 +2226,17 @@ __global__ void decode_meta_kernel(const int32_t *slots, int n, const int32_t *p
     else {
         tokens[i] = pending[s];
         row_pos[i] = ctx[s];
+        seq_prev[i] = last_tok[s];
+        last_tok[s] = pending[s];
     }
+}
+// the same bookkeeping of a packed step: per sequence the token fed before the step, replaced by the step's last one
+__global__ void seq_prev_kernel(const int32_t *tokens, const int32_t *seq_row0, const int32_t *seq_slot, int n, int32_t *seq_prev, int32_t *last_tok) {
+    const int i = blockIdx.x * blockDim.x + threadIdx.x;
+    if (i >= n) return;
+    const int s = seq_slot[i];
+    seq_prev[i] = last_tok[s];
+    last_tok[s] = tokens[seq_row0[i + 1] - 1];
 }
 
 }  // namespace hy

@@ -26,7 +26,7 @@ MIX_ATTENTION, MIX_DELTA, MIX_LINREC, MIX_LATENT = 0, 1, 2, 3
 REC_CHANNEL, REC_EXPGATE, REC_FIXED = 0, 1, 2
 NORM_RMS, NORM_DYT = 0, 1
 FF_PLAIN, FF_GATED, FF_MOE = 0, 1, 2
-ROUTER_SOFTMAX, ROUTER_SIGMOID = 0, 1
+ROUTER_SOFTMAX, ROUTER_SIGMOID, ROUTER_CHOSEN_SOFTMAX = 0, 1, 2
 BLOCK_SEQUENTIAL, BLOCK_PARALLEL, BLOCK_POSTNORM, BLOCK_SANDWICH = 0, 1, 2, 3
 VMIX_NONE, VMIX_FIRST, VMIX_BLEND = 0, 1, 2
 HY_F32, HY_BF16 = 0, 2
@@ -53,7 +53,10 @@ class TlHybridLayer(ctypes.Structure):
                 ("moe_router", _i), ("moe_gated", _i), ("moe_scale_input", _i), ("moe_shared_sg", _i),
                 ("w_in_bias_dev", _vp), ("window", _i), ("qk_head_norm", _i), ("diff_maps", _i), ("diff_lambda", _f), ("diff_init", _f),
                 ("decay_dev", _vp), ("post_norm_dev", _vp), ("post_norm2_dev", _vp),
-                ("side_gate_dev", _vp), ("side_proj_dev", _vp), ("side_norm_dev", _vp), ("side_col0", _i)]
+                ("side_gate_dev", _vp), ("side_proj_dev", _vp), ("side_norm_dev", _vp), ("side_col0", _i),
+                ("softcap", _f), ("bias_slope_dev", _vp), ("q_temp_coef", _f), ("q_temp_every", _f),
+                ("rec_silu", _i), ("rec_plain_k", _i), ("rec_joint_norm", _i), ("rec_sigmoid_gate", _i), ("router_bias_dev", _vp),
+                ("beside", _vp), ("mix_scale", _f)]
 
 
 class TlHybridConfig(ctypes.Structure):
@@ -63,7 +66,9 @@ class TlHybridConfig(ctypes.Structure):
                 ("final_norm_offset", _f), ("head_dev", _vp),
                 ("embed_scale", _f), ("final_norm_kind", _i), ("final_norm_alpha", _f), ("final_norm_bias_dev", _vp),
                 ("page_size", _i), ("num_pages", _i), ("max_slots", _i), ("max_pages_per_seq", _i), ("max_rows", _i),
-                ("logit_scale", _f), ("embed_norm_dev", _vp), ("side_embed_dev", _vp), ("side_cols", _i), ("side_dim", _i)]
+                ("logit_scale", _f), ("embed_norm_dev", _vp), ("side_embed_dev", _vp), ("side_cols", _i), ("side_dim", _i),
+                ("pair_embed_dev", _vp), ("pair_buckets", ctypes.c_int64), ("pair_mul_prev", ctypes.c_int64), ("pair_mul_cur", ctypes.c_int64),
+                ("logit_softcap", _f)]
 
 
 class TlHybridStats(ctypes.Structure):

@@ -25,7 +25,7 @@ _NORM = {"rms": 0, "dyt": 1}
 _FF_KIND = {"plain": 0, "gated": 1, "moe": 2}
 _BLOCK = {"sequential": 0, "parallel": 1, "postnorm": 2, "sandwich": 3}
 _VMIX = {"none": 0, "first": 1, "blend": 2}
-_ROUTER = {"softmax": 0, "sigmoid": 1}
+_ROUTER = {"softmax": 0, "sigmoid": 1, "chosen_softmax": 2}
 
 
 class HybridEngine:
@@ -52,53 +52,33 @@ class HybridEngine:
         self.page_size, self.max_batch, self.vocab_size = int(page_size), int(max_batch), cfg.vocab
         self.max_prefill_rows = max(int(max_prefill_rows), self.max_batch)
         self.num_hidden_layers = len(cfg.layers)
-        self.has_recurrent_state = any(L.kind in ("delta", "linrec") for L in cfg.layers)
+        self.has_recurrent_state = cfg.pair_embed is not None or any(M.kind in ("delta", "linrec") for L in cfg.layers for M in (L, L.beside) if M is not None)
         for i, L in enumerate(cfg.layers):  # a size the configuration leaves to the tensors
             if L.a_rank < 0:
                 L.a_rank = int(model.tensors[cfg.prefix(i) + "mix.a1"].shape[0])
         w = self._weights = pack_layer_list(cfg, model.tensors, dtype, self.device)
         layers = (ext.TlHybridLayer * len(cfg.layers))()
+        self._beside: list = []  # descriptions of second mixers
         for i, (L, t) in enumerate(zip(cfg.layers, w["layers"])):
             s = layers[i]
-            s.kind = _MIX[L.kind]
-            s.heads, s.kv_heads, s.dim, s.vdim, s.ff, s.ff_act = L.heads, L.kv_heads, L.dim, L.vdim, L.ff, _FF_ACT[L.ff_act]
-            s.w_in_dev, s.w_out_dev, s.norm_dev, s.norm_offset = t["w_in"].data_ptr(), t["w_out"].data_ptr(), t["norm"].data_ptr(), cfg.norm_offset
-            s.rot_dims, s.rot_base, s.scale = L.rot_dims, L.rot_base, L.scale
-            s.qk_unit_rms, s.sink, s.gated = int(L.qk_unit_rms), int(L.sink), (2 if L.head_gate else 1) if L.gated else 0
-            s.conv_taps, s.unit_eps = L.conv_taps, L.unit_eps
-            if L.kind == "delta":
-                s.conv_dev, s.a_log_dev, s.dt_bias_dev, s.out_norm_dev = (t["conv"].data_ptr(), t["a_log"].data_ptr(),
-                                                                          t["dt_bias"].data_ptr(), t["out_norm"].data_ptr())
             ptr = lambda key: t[key].data_ptr() if key in t else None
+            self._describe_mixer(s, L, t)
+            if L.beside is not None:
+                second = ext.TlHybridLayer()
+                self._describe_mixer(second, L.beside, t["beside"])
+                self._beside.append(second)  # read by create only
+                s.beside = ctypes.addressof(second)
+            s.ff, s.ff_act = L.ff, _FF_ACT[L.ff_act]
+            s.w_in_dev, s.w_out_dev, s.norm_dev, s.norm_offset = t["w_in"].data_ptr(), t["w_out"].data_ptr(), t["norm"].data_ptr(), cfg.norm_offset
             s.norm_kind, s.norm_alpha, s.norm2_alpha = _NORM[cfg.norm_kind], t.get("norm_alpha", 0.0), t.get("norm2_alpha", 0.0)
             s.norm_bias_dev, s.norm2_bias_dev, s.norm2_dev = ptr("norm_bias"), ptr("norm2_bias"), ptr("norm2")
             s.w_in2_dev, s.w_out2_dev, s.ls1_dev, s.ls2_dev = ptr("w_in2"), ptr("w_out2"), ptr("ls1"), ptr("ls2")
             s.ff_kind, s.experts, s.identity, s.top, s.groups, s.keep = _FF_KIND[L.ff_kind], L.experts, L.identity, L.top, L.groups, L.keep
-            s.expert_ff, s.shared_ff, s.correction_dev = L.expert_ff, L.shared_ff, ptr("correction")
-            s.kv_from = -1
+            s.expert_ff, s.shared_ff, s.correction_dev, s.router_bias_dev = L.expert_ff, L.shared_ff, ptr("correction"), ptr("router_bias")
             s.moe_router, s.moe_gated, s.moe_scale_input = _ROUTER[L.router], int(L.moe_gated), int(L.moe_scale_input)
             s.moe_shared_sg = int(L.moe_gated and L.moe_shared_sg)
-            if L.kind == "attention":
-                s.qk_norm, s.q_norm_dev, s.k_norm_dev, s.rot_half = int(L.qk_norm), ptr("q_norm"), ptr("k_norm"), int(L.rot_half)
-                s.talk_dev, s.sink_dev, s.chunk = ptr("talk"), ptr("sink"), L.chunk
-                s.v_mix, s.v_mix_lambda = _VMIX[L.v_mix], t.get("v_mix_lambda", 0.0)
-                s.w_in_bias_dev, s.window, s.qk_head_norm = ptr("w_in_bias"), L.window, int(L.qk_head_norm)
-                if L.diff is not None:
-                    s.diff_maps, s.diff_lambda, s.diff_init = 1, t["diff_lambda"], L.diff
-            if L.kind in ("attention", "linrec") and L.rot_scaling:
-                s.rot_factor, s.rot_original, s.rot_fast, s.rot_slow = L.rot_scaling
-                s.rot_scaling_kind = 1 if L.rot_scaling_kind == "wavelength" else 0
             s.post_norm_dev, s.post_norm2_dev = ptr("post_norm"), ptr("post_norm2")
             s.side_gate_dev, s.side_proj_dev, s.side_norm_dev, s.side_col0 = ptr("side_gate"), ptr("side_proj"), ptr("side_norm"), i * cfg.side_dim
-            if L.kind == "linrec":
-                s.rec_kind, s.gate_cap, s.tau, s.a_rank, s.out_norm_dev = _REC[L.rec_kind], L.gate_cap, L.tau, max(L.a_rank, 0), ptr("out_norm")
-                s.decay_dev, s.rot_half = ptr("decay"), int(L.rot_half)
-                s.a2_dev, s.a2_bias_dev, s.i_bias_dev, s.f_bias_dev = ptr("a2"), ptr("a2_bias"), ptr("i_bias"), ptr("f_bias")
-            elif L.kind == "latent":
-                s.q_rank, s.kv_rank, s.rot_dim, s.kv_from = L.q_rank, L.kv_rank, L.rot_dim, L.kv_from
-                s.dq_norm_dev, s.dkv_norm_dev, s.uq_dev, s.uk_t_dev, s.uv_dev = ptr("dq_norm"), ptr("dkv_norm"), ptr("uq"), ptr("uk_t"), ptr("uv")
-                if L.rot_scaling:
-                    s.rot_factor, s.rot_original, s.rot_fast, s.rot_slow = L.rot_scaling
         c = ext.TlHybridConfig()
         c.dtype = ext.HY_BF16 if dtype == torch.bfloat16 else ext.HY_F32
         c.width, c.vocab, c.num_layers, c.norm_eps, c.residual_mult = cfg.width, cfg.vocab, len(cfg.layers), cfg.norm_eps, cfg.residual_mult
@@ -110,6 +90,10 @@ class HybridEngine:
             c.loop_in_dev, c.loop_step_dev = (w["loop_in"].data_ptr() if "loop_in" in w else None), w["loop_step"].data_ptr()
         c.embed_dev, c.final_norm_dev, c.final_norm_offset, c.head_dev = w["embed"].data_ptr(), w["final_norm"].data_ptr(), cfg.norm_offset, w["head"].data_ptr()
         c.embed_norm_dev = w["embed_norm"].data_ptr() if "embed_norm" in w else None
+        c.logit_softcap = cfg.logit_softcap
+        if cfg.pair_embed:
+            c.pair_embed_dev = w["pair_embed"].data_ptr()
+            c.pair_buckets, c.pair_mul_prev, c.pair_mul_cur = cfg.pair_embed
         if cfg.side_dim:
             c.side_embed_dev, c.side_cols, c.side_dim = w["side_embed"].data_ptr(), w["side_embed"].shape[1], cfg.side_dim
         c.page_size, c.num_pages, c.max_slots = self.page_size, int(num_pages), self.max_batch
@@ -120,6 +104,39 @@ class HybridEngine:
         ext.check(self._lib.tl_hybrid_create(ctypes.byref(c), layers, None, ctypes.byref(handle)))
         self._h = handle
         self._produced: dict[int, list[int]] = {}
+
+    @staticmethod
+    def _describe_mixer(s: Any, L: Any, t: dict) -> None:
+        """The mixer fields of a layer description (``s``: a TlHybridLayer) from a LayerSpec and its packed tensors."""
+        ptr = lambda key: t[key].data_ptr() if key in t else None
+        s.kind, s.heads, s.kv_heads, s.dim, s.vdim, s.kv_from, s.mix_scale = _MIX[L.kind], L.heads, L.kv_heads, L.dim, L.vdim, -1, L.mix_scale
+        s.rot_dims, s.rot_base, s.scale = L.rot_dims, L.rot_base, L.scale
+        s.qk_unit_rms, s.sink, s.gated = int(L.qk_unit_rms), int(L.sink), (2 if L.head_gate else 1) if L.gated else 0
+        s.sink_dev, s.window = ptr("sink"), L.window
+        if L.rot_scaling:
+            s.rot_factor, s.rot_original, s.rot_fast, s.rot_slow = L.rot_scaling
+            s.rot_scaling_kind = 1 if L.kind in ("attention", "linrec") and L.rot_scaling_kind == "wavelength" else 0
+        if L.kind == "delta":
+            s.conv_taps, s.unit_eps = L.conv_taps, L.unit_eps
+            s.conv_dev, s.a_log_dev, s.dt_bias_dev, s.out_norm_dev = ptr("conv"), ptr("a_log"), ptr("dt_bias"), ptr("out_norm")
+        elif L.kind == "attention":
+            s.qk_norm, s.q_norm_dev, s.k_norm_dev, s.rot_half = int(L.qk_norm), ptr("q_norm"), ptr("k_norm"), int(L.rot_half)
+            s.talk_dev, s.chunk = ptr("talk"), L.chunk
+            s.v_mix, s.v_mix_lambda = _VMIX[L.v_mix], t.get("v_mix_lambda", 0.0)
+            s.w_in_bias_dev, s.qk_head_norm = ptr("w_in_bias"), int(L.qk_head_norm)
+            if L.diff is not None:
+                s.diff_maps, s.diff_lambda, s.diff_init = 1, t["diff_lambda"], L.diff
+            s.softcap, s.bias_slope_dev = L.softcap, ptr("bias_slope")
+            if L.q_temp:
+                s.q_temp_coef, s.q_temp_every = L.q_temp
+        elif L.kind == "linrec":
+            s.rec_kind, s.gate_cap, s.tau, s.a_rank, s.out_norm_dev = _REC[L.rec_kind], L.gate_cap, L.tau, max(L.a_rank, 0), ptr("out_norm")
+            s.decay_dev, s.rot_half = ptr("decay"), int(L.rot_half)
+            s.rec_silu, s.rec_plain_k, s.rec_joint_norm, s.rec_sigmoid_gate = int(L.rec_silu), int(L.rec_plain_k), int(L.rec_joint_norm), int(L.rec_sigmoid_gate)
+            s.a2_dev, s.a2_bias_dev, s.i_bias_dev, s.f_bias_dev = ptr("a2"), ptr("a2_bias"), ptr("i_bias"), ptr("f_bias")
+        elif L.kind == "latent":
+            s.q_rank, s.kv_rank, s.rot_dim, s.kv_from = L.q_rank, L.kv_rank, L.rot_dim, L.kv_from
+            s.dq_norm_dev, s.dkv_norm_dev, s.uq_dev, s.uk_t_dev, s.uv_dev = ptr("dq_norm"), ptr("dkv_norm"), ptr("uq"), ptr("uk_t"), ptr("uv")
 
     @classmethod
     def from_model(cls, model: Any, **kwargs) -> "HybridEngine":

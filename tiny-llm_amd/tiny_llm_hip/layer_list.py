@@ -69,6 +69,20 @@ per-layer token input:
     mixer "retention": q, k, v per head, q and k rotated (pairs (i, i + dims/2)), k * dim^-1/2;  S <- decay_h S + k v^T;  o = S^T q;
         o / rms(o) * silu(W_g h); W_o.
     loop {start, stop, times}: as Fonapel's, entered by x <- x + step[t] alone.
+
+Karorax -- x = embed[token] + bigram[(previous token * mul_prev + token * mul_cur) mod buckets] (row `buckets` for a first token);
+sequential pre-norm blocks, norms with weights around zero, per-channel layer scales:
+
+    x <- x + ls1 * mixer(norm1 x);   x <- x + ls2 * ff(norm2 x)       norm: y / sqrt(mean y^2 + eps) * (1 + w);  logits = cap tanh(head norm(x) / cap)
+
+    mixer "latent_attention": q = W_q h directly ([plain | rotated] per head); latent and rotated key part as Zefapel's with plain frequencies;
+        keys j with 0 <= i - j < mask.size; weights exp(s) / (exp(sink_h) + sum exp(s)); one sigmoid gate per head; "kv_from" as Zefapel's.
+    mixer "parallel": left_scale * left(h) + right_scale * right(h).  left: grouped-query attention without rotation; q times
+        1 + coef ln(floor((p + 1) / every) + 1); s = cap tanh(q.k scale / cap) - 2^(-8 (h + 1) / H) (i - j); causal softmax; W_o.
+        right (lightning attention): q, k, v pass SiLU; S <- decay_h S + k v^T; o = S^T q; rms_norm over all heads * norm * sigmoid(W_g h); W_o.
+    ff "dense": W_down relu(W_up h)^2.
+    ff "moe": z = W_router h + b; the `top` largest z are taken, weights = softmax over those; expert = W_down (silu(W_gate h) * W_up h);
+        plus a shared expert of the same form.
 """
 
 from __future__ import annotations
@@ -78,7 +92,7 @@ from typing import Any, Callable
 
 import torch
 
-__all__ = ["LayerSpec", "LayerListConfig", "FAMILIES", "fonapel_config", "zefapel_config", "lovulix_config", "muduvik_config", "pack_layer_list"]
+__all__ = ["LayerSpec", "LayerListConfig", "FAMILIES", "fonapel_config", "zefapel_config", "lovulix_config", "muduvik_config", "karorax_config", "pack_layer_list"]
 
 
 @dataclass
@@ -143,6 +157,21 @@ class LayerSpec:
     # linrec "fixed": a constant decay per head
     decay: tuple[float, ...] = ()
     out_norm_weight: bool = True    # linrec: the read-out's unit-RMS norm has a weight (tensor mix.norm)
+    # linrec "fixed", further options
+    rec_silu: bool = False          # q, k and v pass SiLU
+    rec_plain_k: bool = False       # k is not scaled by dim^-1/2
+    rec_joint_norm: bool = False    # the read-out of all heads is normed together (mix.norm [heads*vdim])
+    rec_sigmoid_gate: bool = False  # the gate is a sigmoid (SiLU otherwise)
+    # attention, further options (3)
+    softcap: float = 0.0            # > 0: scores s <- softcap tanh(s / softcap)
+    distance_bias: bool = False     # scores -= 2^(-8 (h + 1) / heads) * (query position - key position)
+    q_temp: tuple[float, float] | None = None  # (coef, every): q *= 1 + coef ln(floor((p + 1) / every) + 1)
+    # mixture of experts, further options (2)
+    moe_bias: bool = False          # the router's logits carry a bias (tensor mlp.router.b)
+    # two mixers side by side on one input
+    beside: LayerSpec | None = None # the second mixer (its sizes and options only; the feed-forward is the layer's)
+    mix_scale: float = 1.0          # factor on this mixer's result
+    mix_prefix: str = "mix."        # where this mixer's tensors lie behind the layer's prefix
 
 
 @dataclass
@@ -164,6 +193,9 @@ class LayerListConfig:
     embed_norm: bool = False        # the embedding output passes the model's norm (tensor embed.norm)
     loop_projection: bool = True    # a loop pass is entered through loop.in [width, 2 width]; False: only loop.step is added
     side_dim: int = 0               # > 0: per-layer token input of this many columns a layer (tensors side.embed, <layer>.side.*)
+    pair_embed: tuple[int, int, int] | None = None  # (buckets, factor of the previous token, factor of the token): a second embedding table
+                                    # [buckets + 1, width] indexed by a hash of both is added (tensor bigram; the last row for a first token)
+    logit_softcap: float = 0.0      # > 0: logits <- cap tanh(logits / cap)
     prefix: Callable[[int], str] = field(default=lambda i: f"l{i}.")
 
     @property
@@ -421,6 +453,92 @@ def _muduvik_tensor_shapes(cfg: LayerListConfig) -> dict[str, tuple[int, ...]]:
     return want
 
 
+def karorax_config(config: dict) -> LayerListConfig:
+    """config.json of a Karorax checkpoint -> LayerListConfig.  Every size and every constant the file gives is read from it."""
+    for key in ("layers", "norm", "vocab", "width"):
+        if key not in config:
+            raise ValueError(f"config.json lacks {key!r}")
+    layers = []
+    for i, entry in enumerate(config["layers"]):
+        kind, mc, mlp = entry.get("type"), entry.get("mixer") or {}, entry.get("mlp")
+        ff: dict[str, Any] = {}
+        if mlp is not None:
+            if mlp.get("kind", "dense") == "dense":
+                ff = dict(ff=int(mlp["ff"]), ff_kind="plain", ff_act="relu2")
+            elif mlp["kind"] == "moe":
+                r, shared = mlp["router"], mlp.get("shared")
+                experts, expert_ff = int(r["experts"]), int(mlp["expert"]["ff"])
+                shared_ff = int(shared["ff"]) if shared else 0
+                if not 1 <= int(r["top"]) <= experts:
+                    raise ValueError(f"layer {i}: top={r['top']} of {experts} experts")
+                ff = dict(ff=shared_ff + experts * expert_ff, ff_kind="moe", ff_act="silu", experts=experts, top=int(r["top"]), expert_ff=expert_ff,
+                          shared_ff=shared_ff, router="chosen_softmax", moe_gated=True, moe_shared_sg=False, moe_correction=False, moe_bias=True)
+            else:
+                raise ValueError(f"layer {i}: unsupported mlp.kind={mlp.get('kind')!r}")
+        if kind == "latent_attention":
+            rot, rot_dim = mc.get("rot") or {}, int(mc.get("rot_dim", 0))
+            kv_from = int(mc["kv_from"]) if mc.get("kv_from") is not None else -1
+            if kv_from >= i or kv_from < -1:
+                raise ValueError(f"layer {i}: kv_from={kv_from} must name an earlier layer")
+            layers.append(LayerSpec(kind="latent", heads=int(mc["heads"]), kv_heads=1, dim=int(mc["dim"]), vdim=int(mc["vdim"]), kv_rank=int(mc["kv_rank"]),
+                                    rot_dim=rot_dim, rot_dims=int(rot.get("dims", 0)), rot_base=float(rot.get("base", 10000.0)), scale=float(mc["scale"]),
+                                    window=int((mc.get("mask") or {}).get("size", 0)), sink=True, learned_sink=True, gated=True, head_gate=True,
+                                    kv_from=kv_from, **ff))
+        elif kind == "parallel":
+            a, r, temp = mc["left"], mc["right"], mc["left"].get("q_temp")
+            if int(a["heads"]) % int(a["kv_heads"]):
+                raise ValueError(f"layer {i}: {a['heads']} heads do not form {a['kv_heads']} equal groups")
+            decay = tuple(float(d) for d in r["decay"])
+            if len(decay) != int(r["heads"]):
+                raise ValueError(f"layer {i}: {len(decay)} decays for {r['heads']} heads")
+            right = LayerSpec(kind="linrec", rec_kind="fixed", heads=int(r["heads"]), kv_heads=int(r["heads"]), dim=int(r["dim"]), vdim=int(r["vdim"]), decay=decay,
+                              rec_silu=True, rec_plain_k=True, rec_joint_norm=True, rec_sigmoid_gate=True, mix_scale=float(mc["right_scale"]), mix_prefix="mix.right.")
+            layers.append(LayerSpec(kind="attention", heads=int(a["heads"]), kv_heads=int(a["kv_heads"]), dim=int(a["dim"]), vdim=int(a["vdim"]),
+                                    scale=float(a["scale"]), softcap=float(a.get("softcap") or 0.0), distance_bias=True,
+                                    q_temp=(float(temp["coef"]), float(temp["every"])) if temp else None, mix_scale=float(mc["left_scale"]), mix_prefix="mix.left.",
+                                    beside=right, **ff))
+        else:
+            raise ValueError(f"layer {i}: unknown mixer type {kind!r}")
+    big = (config.get("embedding") or {}).get("bigram")
+    return LayerListConfig(family="Karorax", width=int(config["width"]), vocab=int(config["vocab"]), norm_eps=float(config["norm"]["eps"]), residual_mult=1.0,
+                           layers=layers, norm_offset=1.0, block="sequential", layer_scale=True,
+                           pair_embed=(int(big["buckets"]), int(big["mul_prev"]), int(big["mul_cur"])) if big else None,
+                           logit_softcap=float(config.get("logit_softcap") or 0.0))
+
+
+def _karorax_tensor_shapes(cfg: LayerListConfig) -> dict[str, tuple[int, ...]]:
+    """Every tensor a Karorax checkpoint must hold, with its shape."""
+    W = cfg.width
+    want: dict[str, tuple[int, ...]] = {"embed": (cfg.vocab, W), "final.norm": (W,), "head": (cfg.vocab, W)}
+    if cfg.pair_embed:
+        want["bigram"] = (cfg.pair_embed[0] + 1, W)
+    for i, L in enumerate(cfg.layers):
+        p = cfg.prefix(i)
+        want.update({p + "norm1": (W,), p + "ls1": (W,)})
+        m = p + L.mix_prefix
+        if L.kind == "latent":
+            hv = L.heads * L.vdim
+            want.update({m + "q": (L.heads * (L.dim + L.rot_dim), W), m + "uk": (L.heads * L.dim, L.kv_rank), m + "uv": (hv, L.kv_rank), m + "sink": (L.heads,),
+                         m + "g": (L.heads, W), m + "o": (W, hv)})
+            if L.kv_from < 0:
+                want.update({m + "dkv": (L.kv_rank + L.rot_dim, W), m + "dkv.norm": (L.kv_rank,)})
+        else:
+            R, r = L.beside, p + L.beside.mix_prefix
+            want.update({m + "q": (L.heads * L.dim, W), m + "k": (L.kv_heads * L.dim, W), m + "v": (L.kv_heads * L.vdim, W), m + "o": (W, L.heads * L.vdim)})
+            hd, hv = R.heads * R.dim, R.heads * R.vdim
+            want.update({r + "q": (hd, W), r + "k": (hd, W), r + "v": (hv, W), r + "g": (hv, W), r + "norm": (hv,), r + "o": (W, hv)})
+        if L.ff:
+            f = p + "mlp."
+            want.update({p + "norm2": (W,), p + "ls2": (W,)})
+            if L.ff_kind == "plain":
+                want.update({f + "up": (L.ff, W), f + "down": (W, L.ff)})
+            else:
+                want.update({f + "router": (L.experts, W), f + "router.b": (L.experts,)})
+                for name, n in [(f"e{e}.", L.expert_ff) for e in range(L.experts)] + ([("shared.", L.shared_ff)] if L.shared_ff else []):
+                    want.update({f + name + "gate": (n, W), f + name + "up": (n, W), f + name + "down": (W, n)})
+    return want
+
+
 def _norm_shapes(cfg: LayerListConfig, name: str) -> dict[str, tuple[int, ...]]:
     if cfg.norm_kind == "dyt":
         return {name: (cfg.width,), name + ".b": (cfg.width,), name + ".alpha": ()}
@@ -469,7 +587,64 @@ FAMILIES: dict[str, tuple[Callable[[dict], LayerListConfig], Callable[[LayerList
     "Zefapel": (zefapel_config, _zefapel_tensor_shapes),
     "Lovulix": (lovulix_config, _lovulix_tensor_shapes),
     "Muduvik": (muduvik_config, _muduvik_tensor_shapes),
+    "Karorax": (karorax_config, _karorax_tensor_shapes),
 }
+
+
+def _pack_mixer(entry: dict, L: LayerSpec, m: str, mat: Callable, vec: Callable, tensors: dict[str, torch.Tensor], device: Any) -> tuple[list, list]:
+    """One mixer's tensors (names ``m`` + ...): its vectors and per-head matrices go into ``entry``; returns its rows of the layer's input matrix
+    and its columns of the output matrix, in the engine's order."""
+    if L.kind == "latent":
+        if L.q_rank:
+            rows = [mat(m + "dq")]
+            entry["dq_norm"], entry["uq"] = vec(m + "dq.norm"), mat(m + "uq").contiguous()
+        else:
+            rows = [mat(m + "q")]
+        rows += ([mat(m + "dkv")] if L.kv_from < 0 else []) + ([mat(m + "g")] if L.gated else [])
+        if L.kv_from < 0:
+            entry["dkv_norm"] = vec(m + "dkv.norm")
+        # per head: W_uk transposed ([kv_rank, dim]: the key projection is applied to the query), W_uv as stored ([vdim, kv_rank])
+        entry["uk_t"] = mat(m + "uk").reshape(L.heads, L.dim, L.kv_rank).transpose(1, 2).contiguous()
+        entry["uv"] = mat(m + "uv").reshape(L.heads, L.vdim, L.kv_rank).contiguous()
+        if L.learned_sink:
+            entry["sink"] = vec(m + "sink")
+    else:
+        rows = [mat(m + "q"), mat(m + "k"), mat(m + "v")]
+        if L.kind != "attention" or L.gated:
+            rows.append(mat(m + "g"))
+    if L.kind == "attention":
+        if L.qk_norm or L.qk_head_norm:
+            entry["q_norm"], entry["k_norm"] = vec(m + "q.norm"), vec(m + "k.norm")
+        if L.bias:  # one vector over the mixer's rows of w_in: q | k | v biases, zeros behind them (the gate has none)
+            b = torch.cat([vec(m + "q.b"), vec(m + "k.b"), vec(m + "v.b")])
+            entry["w_in_bias"] = torch.cat([b, torch.zeros(sum(r.shape[0] for r in rows) - b.numel(), device=device)]).contiguous()
+        if L.diff is not None:  # one number for the layer, from four [dim] vectors, in float32
+            t32 = lambda name: tensors[m + name].to(torch.float32)
+            entry["diff_lambda"] = float(torch.exp((t32("lq1") * t32("lk1")).sum()) - torch.exp((t32("lq2") * t32("lk2")).sum()) + torch.tensor(L.diff, dtype=torch.float32))
+        if L.talk:
+            entry["talk"] = vec(m + "talk")
+        if L.learned_sink:
+            entry["sink"] = vec(m + "sink")
+        if L.v_mix == "blend":
+            entry["v_mix_lambda"] = float(tensors[m + "vmix"].float())
+        if L.distance_bias:
+            entry["bias_slope"] = torch.tensor([2.0 ** (-8.0 * (h + 1) / L.heads) for h in range(L.heads)], dtype=torch.float32, device=device)
+    if L.kind == "delta":
+        rows += [mat(m + "a"), mat(m + "b")]
+        entry["conv"] = torch.cat([vec(m + "q.conv"), vec(m + "k.conv"), vec(m + "v.conv")], 0).contiguous()
+        entry["a_log"], entry["dt_bias"], entry["out_norm"] = vec(m + "A_log"), vec(m + "dt_bias"), vec(m + "norm")
+    elif L.kind == "linrec":
+        if L.out_norm_weight:
+            entry["out_norm"] = vec(m + "norm")
+        if L.rec_kind == "fixed":
+            entry["decay"] = torch.tensor(L.decay, dtype=torch.float32, device=device)
+        elif L.rec_kind == "expgate":
+            rows += [mat(m + "i"), mat(m + "f")]
+            entry["i_bias"], entry["f_bias"] = vec(m + "i.b"), vec(m + "f.b")
+        else:
+            rows.append(mat(m + "a1"))
+            entry["a2"], entry["a2_bias"] = mat(m + "a2").contiguous(), vec(m + "a2.b")
+    return rows, [mat(m + "o")]
 
 
 def pack_layer_list(cfg: LayerListConfig, tensors: dict[str, torch.Tensor], dtype: torch.dtype, device: Any) -> dict:
@@ -492,6 +667,8 @@ def pack_layer_list(cfg: LayerListConfig, tensors: dict[str, torch.Tensor], dtyp
     norm(packed, "final_norm", "final.norm")
     if cfg.embed_norm:
         packed["embed_norm"] = vec("embed.norm")
+    if cfg.pair_embed:
+        packed["pair_embed"] = mat("bigram").contiguous()
     if cfg.side_dim:
         packed["side_embed"] = mat("side.embed").contiguous()
     if cfg.loop:
@@ -502,49 +679,11 @@ def pack_layer_list(cfg: LayerListConfig, tensors: dict[str, torch.Tensor], dtyp
         p = cfg.prefix(i)
         entry: dict[str, Any] = {}
         norm(entry, "norm", p + "norm1")
-        if L.kind == "latent":
-            rows = [mat(p + "mix.dq")] + ([mat(p + "mix.dkv")] if L.kv_from < 0 else []) + ([mat(p + "mix.g")] if L.gated else [])
-            entry["dq_norm"], entry["uq"] = vec(p + "mix.dq.norm"), mat(p + "mix.uq").contiguous()
-            if L.kv_from < 0:
-                entry["dkv_norm"] = vec(p + "mix.dkv.norm")
-            # per head: W_uk transposed ([kv_rank, dim]: the key projection is applied to the query), W_uv as stored ([vdim, kv_rank])
-            entry["uk_t"] = mat(p + "mix.uk").reshape(L.heads, L.dim, L.kv_rank).transpose(1, 2).contiguous()
-            entry["uv"] = mat(p + "mix.uv").reshape(L.heads, L.vdim, L.kv_rank).contiguous()
-        else:
-            rows = [mat(p + "mix.q"), mat(p + "mix.k"), mat(p + "mix.v")]
-            if L.kind != "attention" or L.gated:
-                rows.append(mat(p + "mix.g"))
-        if L.kind == "attention":
-            if L.qk_norm or L.qk_head_norm:
-                entry["q_norm"], entry["k_norm"] = vec(p + "mix.q.norm"), vec(p + "mix.k.norm")
-            if L.bias:  # one vector over the mixer's rows of w_in: q | k | v biases, zeros behind them (the gate has none)
-                b = torch.cat([vec(p + "mix.q.b"), vec(p + "mix.k.b"), vec(p + "mix.v.b")])
-                entry["w_in_bias"] = torch.cat([b, torch.zeros(sum(r.shape[0] for r in rows) - b.numel(), device=device)]).contiguous()
-            if L.diff is not None:  # one number for the layer, from four [dim] vectors, in float32
-                t32 = lambda name: tensors[p + "mix." + name].to(torch.float32)
-                entry["diff_lambda"] = float(torch.exp((t32("lq1") * t32("lk1")).sum()) - torch.exp((t32("lq2") * t32("lk2")).sum()) + torch.tensor(L.diff, dtype=torch.float32))
-            if L.talk:
-                entry["talk"] = vec(p + "mix.talk")
-            if L.learned_sink:
-                entry["sink"] = vec(p + "mix.sink")
-            if L.v_mix == "blend":
-                entry["v_mix_lambda"] = float(tensors[p + "mix.vmix"].float())
-        if L.kind == "delta":
-            rows += [mat(p + "mix.a"), mat(p + "mix.b")]
-            entry["conv"] = torch.cat([vec(p + "mix.q.conv"), vec(p + "mix.k.conv"), vec(p + "mix.v.conv")], 0).contiguous()
-            entry["a_log"], entry["dt_bias"], entry["out_norm"] = vec(p + "mix.A_log"), vec(p + "mix.dt_bias"), vec(p + "mix.norm")
-        elif L.kind == "linrec":
-            if L.out_norm_weight:
-                entry["out_norm"] = vec(p + "mix.norm")
-            if L.rec_kind == "fixed":
-                entry["decay"] = torch.tensor(L.decay, dtype=torch.float32, device=device)
-            elif L.rec_kind == "expgate":
-                rows += [mat(p + "mix.i"), mat(p + "mix.f")]
-                entry["i_bias"], entry["f_bias"] = vec(p + "mix.i.b"), vec(p + "mix.f.b")
-            else:
-                rows.append(mat(p + "mix.a1"))
-                entry["a2"], entry["a2_bias"] = mat(p + "mix.a2").contiguous(), vec(p + "mix.a2.b")
-        out = [mat(p + "mix.o")]
+        rows, out = _pack_mixer(entry, L, p + L.mix_prefix, mat, vec, tensors, device)
+        if L.beside is not None:  # the second mixer's rows and columns follow the first's; its vectors wait in an entry of their own
+            entry["beside"] = {}
+            more_rows, more_out = _pack_mixer(entry["beside"], L.beside, p + L.beside.mix_prefix, mat, vec, tensors, device)
+            rows, out = rows + more_rows, out + more_out
         if L.ff:
             f = p + "mlp."
             if L.ff_kind == "plain":
@@ -564,6 +703,8 @@ def pack_layer_list(cfg: LayerListConfig, tensors: dict[str, torch.Tensor], dtyp
                 ff_out = [mat(f + n + "down") for n in names]
                 if L.moe_correction:
                     entry["correction"] = vec(f + "correction")
+                if L.moe_bias:
+                    entry["router_bias"] = vec(f + "router.b")
             else:
                 W = cfg.width
                 shared = [mat(f + "shared.up")] if L.shared_ff else []
