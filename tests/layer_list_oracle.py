@@ -963,11 +963,16 @@ def chosen_softmax_route(z, top):
     return {j: e[j] / sum(e.values()) for j in chosen}
 
 
-def karorax_feed_forward(mlp, W, f, h):
+def karorax_feed_forward(mlp, W, f, h, margins=None):
+    """``margins`` (a list) receives, per token, how far the last logit taken lies above the first one left out."""
     if mlp["kind"] == "dense":
         return relu2(h @ W[f + "up"].T) @ W[f + "down"].T
     out = np.zeros_like(h)
     z = h @ W[f + "router"].T + W[f + "router.b"]
+    top = mlp["router"]["top"]
+    if margins is not None and top < z.shape[1]:
+        s = -np.sort(-z, axis=1)
+        margins.append(s[:, top - 1] - s[:, top])
     for t in range(h.shape[0]):
         for j, w in chosen_softmax_route(z[t], mlp["router"]["top"]).items():
             out[t] += w * gated_expert(W, f + f"e{j}.", h[t])
@@ -976,8 +981,9 @@ def karorax_feed_forward(mlp, W, f, h):
     return out
 
 
-def karorax_forward(config, W, tokens, streams=None):
-    """Logits [L, vocab] of a whole sequence; ``streams`` (a list) receives the residual stream after every layer."""
+def karorax_forward(config, W, tokens, streams=None, margins=None):
+    """Logits [L, vocab] of a whole sequence; ``streams`` (a list) receives the residual stream after every layer, ``margins`` one row of router
+    margins per mixture of experts."""
     W = {k: np.asarray(v, dtype=np.float64) for k, v in W.items()}
     eps = config["norm"]["eps"]
     tokens = [int(t) for t in tokens]
@@ -999,7 +1005,7 @@ def karorax_forward(config, W, tokens, streams=None):
             raise ValueError(spec["type"])
         x = x + y * W[p + "ls1"]
         if spec.get("mlp"):
-            x = x + karorax_feed_forward(spec["mlp"], W, p + "mlp.", rms_norm(x, W[p + "norm2"], eps, 1.0)) * W[p + "ls2"]
+            x = x + karorax_feed_forward(spec["mlp"], W, p + "mlp.", rms_norm(x, W[p + "norm2"], eps, 1.0), margins) * W[p + "ls2"]
         if streams is not None:
             streams.append(x.copy())
     logits = rms_norm(x, W["final.norm"], eps, 1.0) @ W["head"].T
