@@ -23,6 +23,12 @@ values blended from the second layer on) with 8 gated experts of W / 2 (2 taken)
 sequential block with layer scales, latent attention over the same 192-wide cache rows, a linear recurrence over 128 x 128 states, the
 same gated feed-forward of 2 W) and, for its attention layers, beside Fonapel's attention: 4 layers (retention, differential attention with
 a window of 4,096 positions, latent attention, differential attention), a per-layer token input of 256 columns.
+
+`--layer-list-family Karorax` measures the Karorax family beside Zefapel (the closest existing model: sequential blocks with layer scales, latent
+attention over the same 192 + 64-wide cache rows, a second layer on the first one's cache, a linear recurrence over 128 x 128 states, 8 experts of
+W / 2 beside a shared one of W) and, for the capped attention, beside Fonapel's attention layers: 4 layers (parallel + squared-ReLU feed-forward of
+3 W, latent attention with a window of 1,024 + experts, latent attention on that cache + experts, parallel + experts); a parallel layer holds 16 heads of
+attention (a quarter of them K/V heads) AND 16 heads of lightning attention at width 2048.
 """
 
 from __future__ import annotations
@@ -118,6 +124,57 @@ def muduvik_costs(cfg: dict, ctx: int, dtype_bytes: int = 2) -> dict:
 
     return {"matrix_elems": fixed, "head_elems": head, "attn_macs": attn_macs,
             "decode_bytes": lambda b: (fixed + head) * dtype_bytes + b * (sum(per * (min(ctx, win) if win else ctx) for per, win in terms) * dtype_bytes + 2 * state * 4)}
+
+
+def karorax_config(width: int, vocab: int = 32768, window: int = 1024) -> dict:
+    heads = max(1, width // 128)
+    kv = max(1, heads // 4)
+    moe = {"kind": "moe", "expert": {"ff": width // 2}, "router": {"experts": 8, "top": 2}, "shared": {"ff": width}}
+    par = {"left": {"heads": heads, "kv_heads": kv, "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "softcap": 30.0, "q_temp": {"coef": 0.1, "every": 512}}, "left_scale": 0.9,
+           "right": {"heads": heads, "dim": 128, "vdim": 128, "decay": [1.0 - 2.0 ** (-3 - 6 * h / max(1, heads - 1)) for h in range(heads)]}, "right_scale": 0.9}
+    lat = {"heads": heads, "dim": 128, "vdim": 128, "rot_dim": 64, "kv_rank": 192, "rot": {"base": 1e6, "dims": 64}, "scale": 192 ** -0.5, "mask": {"size": window}}
+    layers = [{"type": "parallel", "mixer": par, "mlp": {"kind": "dense", "ff": 3 * width}}, {"type": "latent_attention", "mixer": lat, "mlp": moe},
+              {"type": "latent_attention", "mixer": dict(lat, kv_from=1), "mlp": moe}, {"type": "parallel", "mixer": par, "mlp": moe}]
+    return {"architecture": "Karorax", "embedding": {"bigram": {"buckets": 65521, "mul_prev": 40503, "mul_cur": 10007}}, "layers": layers, "logit_softcap": 30.0,
+            "norm": {"eps": 1e-6}, "vocab": vocab, "width": width}
+
+
+def karorax_costs(cfg: dict, ctx: int, dtype_bytes: int = 2) -> dict:
+    """What the design needs: matrix elements a token multiplies (the experts it takes), attention multiply-adds per (query, key) pair in the per-head
+    form and the pairs a window leaves, the bytes a decode step of b sequences streams: every matrix once, of the experts those b tokens can take; keys and
+    values of the causal layers, the latent rows inside the window (once per cache), the recurrent states read and written."""
+    W, fixed, state, causal, windowed, terms, per_expert, taken = cfg["width"], 0, 0, 0, [], [], [], []
+    for L in cfg["layers"]:
+        m, mlp = L["mixer"], L["mlp"]
+        if L["type"] == "parallel":
+            a, r = m["left"], m["right"]
+            fixed += W * (a["heads"] * a["dim"] + a["kv_heads"] * (a["dim"] + a["vdim"])) + a["heads"] * a["vdim"] * W
+            fixed += W * r["heads"] * (2 * r["dim"] + 2 * r["vdim"]) + r["heads"] * r["vdim"] * W
+            state += r["heads"] * r["dim"] * r["vdim"]
+            causal += a["heads"] * (a["dim"] + a["vdim"])
+            terms.append((a["kv_heads"] * (a["dim"] + a["vdim"]), 0))
+        else:
+            H, D, V, R, C, win = m["heads"], m["dim"], m["vdim"], m["rot_dim"], m["kv_rank"], (m.get("mask") or {}).get("size", 0)
+            fixed += W * H * (D + R) + H * (D + V) * C + W * H + H * V * W
+            windowed.append((H * (D + R + V), win))
+            if "kv_from" not in m:
+                fixed += W * (C + R)
+                terms.append((C + R, win))
+        if mlp and mlp["kind"] == "dense":
+            fixed += 2 * W * mlp["ff"]
+        elif mlp:
+            fixed += W * mlp["router"]["experts"] + (3 * W * mlp["shared"]["ff"] if mlp.get("shared") else 0)
+            per_expert.append(3 * W * mlp["expert"]["ff"])
+            taken.append((mlp["router"]["top"], mlp["router"]["experts"]))
+    head = cfg["vocab"] * W
+
+    def attn_macs(n):
+        full = n * (n + 1) / 2
+        return causal * full + sum(macs * (full if not win or win >= n else win * (win + 1) / 2 + (n - win) * win) for macs, win in windowed)
+
+    return {"matrix_elems": fixed + sum(pe * top for pe, (top, _) in zip(per_expert, taken)), "head_elems": head, "attn_macs": attn_macs,
+            "decode_bytes": lambda b: (fixed + head + sum(pe * min(n, b * top) for pe, (top, n) in zip(per_expert, taken))) * dtype_bytes
+            + b * (sum(per * (min(ctx, win) if win else ctx) for per, win in terms) * dtype_bytes + 2 * state * 4)}
 
 
 def zefapel_dense_config(width: int, vocab: int = 32768) -> dict:
@@ -266,7 +323,7 @@ def measure(engine, prompt, decode_steps: int, batches=(1, 4), free_running=None
 
 
 def run_family_pair(widths, prompt_len: int = 2048, decode_steps: int = 64, seed: int = 0, device: str = "cuda", family: str = "Zefapel") -> dict:
-    """Zefapel or Lovulix beside Fonapel (Lovulix: beside its attention layers only), all on the layer-list engine."""
+    """A family beside the closest existing ones (module docstring), all on the layer-list engine."""
     import torch
 
     from tiny_llm_hip.models import engine_for
@@ -281,10 +338,12 @@ def run_family_pair(widths, prompt_len: int = 2048, decode_steps: int = 64, seed
         pages = 4 * ((prompt_len + 3 * decode_steps) // page + 2)
         row = {"width": W, "prompt_len": prompt_len, "decode_steps": decode_steps}
         new = {"Zefapel": ("zefapel", zefapel_config(W), zefapel_costs), "Lovulix": ("lovulix", lovulix_config(W), lovulix_costs),
-               "Muduvik": ("muduvik", muduvik_config(W), muduvik_costs)}[family]
+               "Muduvik": ("muduvik", muduvik_config(W), muduvik_costs), "Karorax": ("karorax", karorax_config(W), karorax_costs)}[family]
         others = [("fonapel", fonapel_config(W, order="mixed" if family == "Zefapel" else "attention"), fonapel_costs)]
         if family == "Muduvik":
             others.insert(0, ("zefapel_dense", zefapel_dense_config(W), zefapel_costs))
+        elif family == "Karorax":
+            others.insert(0, ("zefapel", zefapel_config(W), zefapel_costs))
         for key, cfg, costs in [new] + others:
             model = synthetic_layer_list(cfg, seed=seed, device=device)
             eng = engine_for(model, dtype=torch.bfloat16, page_size=page, num_pages=pages, max_batch=4, max_pages_per_seq=pages // 4, max_prefill_rows=prompt_len)
@@ -366,7 +425,7 @@ def summarize(got: dict, costs: dict, prompt_len: int) -> dict:
 
 
 def main(widths, prompt_len=2048, decode_steps=64, family="Fonapel") -> None:
-    if family not in ("Fonapel", "Zefapel", "Lovulix", "Muduvik"):
+    if family not in ("Fonapel", "Zefapel", "Lovulix", "Muduvik", "Karorax"):
         raise SystemExit(f"--layer-list-family: unknown family {family!r}")
     out = run(widths, prompt_len, decode_steps) if family == "Fonapel" else run_family_pair(widths, prompt_len, decode_steps, family=family)
     print(json.dumps(out), flush=True)
