@@ -385,6 +385,53 @@ static int attention_core(tl_hybrid *e, const tl_hybrid_layer &L, const void *kp
     return launch_attn_tile<D, 64, 16>(e, L, kpool, vpool, v_row, m, sh, gate, ldg, out, ldo, x);
 }
 
+template <int DK8, int VT>
+static int launch_latent_tile(tl_hybrid *e, const tl_hybrid_layer &L, const void *pool, const Meta &m, const StepShape &sh, void *out) {
+    const tl_hybrid_config &c = e->cfg;
+    int HGB = 1;
+    while (HGB < L.heads && HGB < 16) HGB *= 2;
+    const int n_hblk = (L.heads + HGB - 1) / HGB, TQ = 64 / HGB;
+    int page_shift = -1;
+    for (int b = 0; b < 30; ++b)
+        if ((1 << b) == c.page_size) page_shift = b;
+    const bool wsplit = sh.max_len * HGB <= 16;
+    const size_t lds_tile = (size_t)64 * (32 * DK8 + 8) * 2, lds = wsplit ? std::max(lds_tile, (size_t)(128 + 4 * 64 * 4 * VT) * 4) : lds_tile;
+    auto kern = wsplit ? latent_tile_kernel<DK8, VT, true> : latent_tile_kernel<DK8, VT, false>;
+    (void)hipFuncSetAttribute(reinterpret_cast<const void *>(kern), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+    dim3 grid((sh.max_len + TQ - 1) / TQ, n_hblk, sh.n_seqs * sh.n_splits);
+    hipLaunchKernelGGL(kern, grid, dim3(256), lds, e->stream, e->qbuf, (const uint16_t *)pool, m.seq_row0, m.seq_slot, m.row_pos, e->table_dev, c.max_pages_per_seq,
+                       c.page_size, page_shift, L.heads, L.kv_rank + L.rot_dim, L.kv_rank, L.scale, L.sink, L.sink_dev, L.window, HGB, n_hblk, sh.keys_per_split,
+                       sh.n_splits, (uint16_t *)out, L.heads * L.kv_rank, e->part_acc, e->part_ml);
+    TL_CHECK_LAUNCH("hybrid latent attention tile");
+    if (sh.n_splits > 1) {
+        hipLaunchKernelGGL((attn_merge_kernel<BF16>), dim3(sh.rows, L.heads), dim3(64), 0, e->stream, e->part_acc, e->part_ml, sh.n_splits, L.heads, L.kv_rank,
+                           (const float *)nullptr, 0, (uint16_t *)out, L.heads * L.kv_rank, 0, (float *)nullptr, 1.f);
+        TL_CHECK_LAUNCH("hybrid attention merge");
+    }
+    return TL_OK;
+}
+
+// latent attention over its one cached row per token: bfloat16 rows of whole 16-byte chunks up to 256 wide on the kernel that reads keys and values from
+// one staged tile, everything else through the general core (one K/V head whose values are the keys' leading columns)
+template <typename D>
+static int latent_core(tl_hybrid *e, const tl_hybrid_layer &L, const void *pool, const Meta &m, const StepShape &sh0, void *out) {
+    const int DT = L.kv_rank + L.rot_dim;
+    if constexpr (sizeof(typename D::storage) == 2) {
+        if (!e->attn_rows_only && DT % 8 == 0 && DT <= 256) {
+            const StepShape sh = window_shape(sh0, L.window);
+            if (DT <= 64) return launch_latent_tile<2, 4>(e, L, pool, m, sh, out);
+            if (DT <= 128) return launch_latent_tile<4, 8>(e, L, pool, m, sh, out);
+            if (L.kv_rank <= 192) return launch_latent_tile<8, 12>(e, L, pool, m, sh, out);
+            return launch_latent_tile<8, 16>(e, L, pool, m, sh, out);
+        }
+    }
+    tl_hybrid_layer A = L;
+    A.kv_heads = 1, A.dim = DT, A.vdim = L.kv_rank;
+    AttnExtra x;
+    x.window = L.window, x.sinks = L.sink ? L.sink_dev : nullptr;
+    return attention_core<D>(e, A, pool, pool, DT, m, sh0, nullptr, 0, out, L.heads * L.kv_rank, x);
+}
+
 static size_t attn_talk_lds(int es, int DK4, int VT, int G, int HGB) {
     const size_t HP = (size_t)G * HGB, QP = es == 2 ? (4 * DK4 + 8) / 2 : 4 * DK4 + 4;
     return std::max(HP * HP + (size_t)G * 16 * QP + 4 * (size_t)(16 * (16 * VT + 4) + 16 * (16 * G + 4)), (size_t)128 + 4 * 64 * 4 * VT + 4 * 16 * (16 * VT + 4)) * sizeof(float);
@@ -578,11 +625,7 @@ static int mixer_part_t(tl_hybrid *e, size_t ri, int part, float *proj, typename
         TL_CHECK_LAUNCH("hybrid latent prep");
         // the keys' per-head projection moves onto the query: q_h' = W_uk,h^T q_h  -> qbuf[t, h, 0 .. kv_rank)
         HY_TRY(linear_t<D>(e->db, H * L.dim, L.uk_t_dev, e->qbuf, H * DT, rows, L.kv_rank, L.dim, 0, 1.f, nullptr, 0, st, H, L.dim, (long)L.kv_rank * L.dim, DT));
-        tl_hybrid_layer A = L;  // one K/V head: keys [c | rotated part], values = the keys' leading kv_rank columns
-        A.kv_heads = 1, A.dim = DT, A.vdim = L.kv_rank;
-        AttnExtra x;
-        x.window = L.window, x.sinks = L.sink ? L.sink_dev : nullptr;
-        HY_TRY(attention_core<D>(e, A, run.kpool, run.kpool, DT, m, sh, nullptr, 0, e->da, H * L.kv_rank, x));
+        HY_TRY(latent_core<D>(e, L, run.kpool, m, sh, e->da));  // one K/V head: keys [c | rotated part], values = the keys' leading kv_rank columns
         // ... and the values' onto the read-out: o_h = W_uv,h (sum_j p_j c_j)
         HY_TRY(linear_t<D>(e->da, H * L.kv_rank, L.uv_dev, e->obuf, HV, rows, L.vdim, L.kv_rank, 0, 1.f, nullptr, 0, st, H, L.kv_rank, (long)L.vdim * L.kv_rank, L.vdim));
         const size_t n = (size_t)rows * HV;

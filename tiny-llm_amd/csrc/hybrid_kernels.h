@@ -781,6 +781,211 @@ __global__ __launch_bounds__(64) void attn_merge_kernel(const float *part_acc, c
     }
 }
 
+// ---- latent attention, step 2: flash attention over ONE K/V head whose values are the leading columns of its key rows (bfloat16 pages) -------------
+// pool: [pages, page, width] rows [latent (rank) | rotated part], width a multiple of 8, at most 32 DK8; rank at most 16 VT.  A workgroup owns 64 query rows
+// of one sequence (row = (token, head), as in attn_tile_kernel with one K/V head); a 64-key tile is staged ONCE in LDS as it lies in its page (rows of
+// 32 DK8 + 8 16-bit elements, zeros behind `width` and behind the last key) and serves both products:
+//   S^T[key, row]  = K . Q^T      v_mfma_f32_16x16x32_bf16, float32 sums and scale
+//   O^T[vcol, row] = V^T . P^T    the weights stay float32 numbers: each enters as a bfloat16 pair hi + lo (16 mantissa bits), so one 16x16x32 product covers
+//                                 16 keys -- k-slots 8 g .. 8 g + 3 of lane group g hold hi and 8 g + 4 .. 8 g + 7 hold lo of its keys 4 g .. 4 g + 3, where
+//                                 the first product left them -- against V^T read transposed from the row-major tile (ds_read_b64_tr_b16: in a 16-lane
+//                                 group lane c hands in the address of [row c >> 2][4 columns from 4 (c & 3)] and receives column c of the 4 x 16 block)
+// window > 0: keys j with qpos - j < window.  sink: the running pair starts at (sinks[head], or 0, 1).  WSPLIT and split key ranges as in attn_tile_kernel.
+template <int DK8, int VT, bool WSPLIT>
+__global__ __launch_bounds__(256) void latent_tile_kernel(const float *qbuf, const uint16_t *pool, const int32_t *seq_row0, const int32_t *seq_slot,
+                                                          const int32_t *row_pos, const int32_t *block_table, int max_pages, int page_size, int page_shift,
+                                                          int H, int width, int rank, float scale, int sink, const float *sinks, int window, int HGB,
+                                                          int n_hblk, int keys_per_split, int n_splits, uint16_t *out, int ldo, float *part_acc,
+                                                          float *part_ml) {
+    typedef short v4s16 __attribute__((ext_vector_type(4)));
+    typedef __attribute__((address_space(3))) v4s16 lds_v4s16;
+    extern __shared__ float smem[];
+    constexpr int RS = 32 * DK8 + 8;   // elements of a key row in LDS
+    constexpr int CK = 4 * DK8;        // 16-byte chunks of a key row
+    constexpr int NIT = 64 * CK / 256; // chunks a thread stages per tile (= DK8)
+    uint16_t *Ks = reinterpret_cast<uint16_t *>(smem);
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, g4 = lane >> 4, col = lane & 15;
+    const int seq = blockIdx.z / n_splits, split = blockIdx.z % n_splits, hblk = blockIdx.y, TQ = 64 / HGB;
+    const int r0 = seq_row0[seq], len = seq_row0[seq + 1] - r0, t0 = ((int)gridDim.x - 1 - (int)blockIdx.x) * TQ;  // (late tokens see the most keys: first)
+    if (t0 >= len) return;
+    const int pos0 = row_pos[r0];
+    const int32_t *bt = block_table + (size_t)seq_slot[seq] * max_pages;
+    const int k_lo = window > 0 ? max(0, pos0 + t0 - window + 1) : 0;
+    const int k_begin = k_lo + split * keys_per_split, k_end = min(pos0 + min(t0 + TQ, len), k_lo + (split + 1) * keys_per_split);
+    const int rho = (WSPLIT ? 0 : wave * 16) + col, tl = rho / HGB, head = hblk * HGB + rho % HGB;
+    constexpr int NN = WSPLIT ? 1 : 4;
+    const int nb = WSPLIT ? wave : 0;
+    const bool row_ok = t0 + tl < len && head < H;
+    const int trow = r0 + t0 + tl, qpos = pos0 + t0 + tl;
+    const bool owns_sink = sink && split == 0 && (!WSPLIT || wave == 0);
+    float m_run = owns_sink ? (sinks && row_ok ? sinks[head] : 0.f) : -INFINITY, l_run = owns_sink ? 1.f : 0.f;
+    f32x4 o[VT];
+#pragma unroll
+    for (int v = 0; v < VT; ++v) o[v] = f32x4{0.f, 0.f, 0.f, 0.f};
+    if (k_begin < k_end) {
+        u32x4 raw[NIT];
+        auto load_tile = [&](int kb) __attribute__((always_inline)) {
+#pragma unroll
+            for (int it = 0; it < NIT; ++it) {
+                const int q = tid + 256 * it, j = kb + q / CK, c8 = 8 * (q % CK);
+                raw[it] = u32x4{0u, 0u, 0u, 0u};
+                if (j < k_end && c8 < width) {
+                    const int pg = page_shift >= 0 ? (j >> page_shift) : (j / page_size);
+                    raw[it] = *reinterpret_cast<const u32x4 *>(pool + ((size_t)bt[pg] * page_size + (j - pg * page_size)) * width + c8);
+                }
+            }
+        };
+        load_tile(k_begin);
+        u32x4 qb[DK8];
+        const float *qrow = qbuf + ((size_t)(row_ok ? trow : r0) * H + (row_ok ? head : 0)) * width;
+#pragma unroll
+        for (int ks = 0; ks < DK8; ++ks) {
+            const int d = 32 * ks + 8 * g4;
+            qb[ks] = u32x4{0u, 0u, 0u, 0u};
+            if (row_ok && d < width) {
+                const f32x4 a = *reinterpret_cast<const f32x4 *>(qrow + d), b = *reinterpret_cast<const f32x4 *>(qrow + d + 4);
+                qb[ks] = u32x4{BF16::pack2(a[0], a[1]), BF16::pack2(a[2], a[3]), BF16::pack2(b[0], b[1]), BF16::pack2(b[2], b[3])};
+            }
+        }
+        const uint16_t *vtr = Ks + (4 * g4 + (col >> 2)) * RS + 4 * (col & 3);  // this lane's address inside a 16-key x 16-column block of values
+        for (int kb = k_begin; kb < k_end; kb += 64) {
+            __syncthreads();  // every wave is done with the previous tile
+#pragma unroll
+            for (int it = 0; it < NIT; ++it) {
+                const int q = tid + 256 * it;
+                *reinterpret_cast<u32x4 *>(Ks + (q / CK) * RS + 8 * (q % CK)) = raw[it];
+            }
+            __syncthreads();
+            if (kb + 64 < k_end) load_tile(kb + 64);
+            const bool inside = kb + 64 <= k_end && kb + 63 <= pos0 + t0 && (window <= 0 || pos0 + min(t0 + TQ, len) - 1 - kb < window);  // no key of the tile is masked for any row
+            f32x4 sc[NN];
+            float m_tile = -INFINITY;
+#pragma unroll
+            for (int nn = 0; nn < NN; ++nn) {
+                f32x4 a4{0.f, 0.f, 0.f, 0.f};
+                const uint16_t *kr = Ks + (16 * (nb + nn) + col) * RS + 8 * g4;
+#pragma unroll
+                for (int ks = 0; ks < DK8; ++ks)
+                    a4 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, *reinterpret_cast<const u32x4 *>(kr + 32 * ks)),
+                                                                 __builtin_bit_cast(bf16x8_t, qb[ks]), a4, 0, 0, 0);
+#pragma unroll
+                for (int r = 0; r < 4; ++r) {
+                    const int j = kb + 16 * (nb + nn) + 4 * g4 + r;
+                    const bool seen = inside || (row_ok && j <= qpos && j < k_end && (window <= 0 || qpos - j < window));
+                    a4[r] = seen ? a4[r] * scale : -INFINITY;
+                    m_tile = fmaxf(m_tile, a4[r]);
+                }
+                sc[nn] = a4;
+            }
+            m_tile = fmaxf(m_tile, __shfl_xor(m_tile, 16, 64));
+            m_tile = fmaxf(m_tile, __shfl_xor(m_tile, 32, 64));
+            const float m_new = fmaxf(m_run, m_tile);
+            const float corr = (m_run == -INFINITY) ? 0.f : (m_new == m_run ? 1.f : __expf(m_run - m_new));
+            float psum = 0.f;
+#pragma unroll
+            for (int nn = 0; nn < NN; ++nn)
+#pragma unroll
+                for (int r = 0; r < 4; ++r) {
+                    const float p = (sc[nn][r] == -INFINITY) ? 0.f : __expf(sc[nn][r] - m_new);
+                    sc[nn][r] = p;
+                    psum += p;
+                }
+            psum += __shfl_xor(psum, 16, 64);
+            psum += __shfl_xor(psum, 32, 64);
+            if (__any(corr != 1.f && l_run != 0.f)) {  // (most tiles move no row's maximum: the sums keep their scale)
+#pragma unroll
+                for (int v = 0; v < VT; ++v)
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) o[v][r] *= corr;
+            }
+            l_run = l_run * corr + psum;
+            m_run = m_new;
+#pragma unroll
+            for (int nn = 0; nn < NN; ++nn) {
+                const uint32_t h0 = BF16::pack2(sc[nn][0], sc[nn][1]), h1 = BF16::pack2(sc[nn][2], sc[nn][3]);
+                const uint32_t l0 = BF16::pack2(sc[nn][0] - __uint_as_float(h0 << 16), sc[nn][1] - __uint_as_float(h0 & 0xffff0000u));
+                const uint32_t l1 = BF16::pack2(sc[nn][2] - __uint_as_float(h1 << 16), sc[nn][3] - __uint_as_float(h1 & 0xffff0000u));
+                const u32x4 pf{h0, h1, l0, l1};
+                const uint16_t *vr = vtr + 16 * (nb + nn) * RS;
+#pragma unroll
+                for (int v = 0; v < VT; ++v) {
+                    const u32x2 x = __builtin_bit_cast(u32x2, __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_v4s16 *)(vr + 16 * v)));
+                    o[v] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, u32x4{x[0], x[1], x[0], x[1]}), __builtin_bit_cast(bf16x8_t, pf), o[v], 0, 0, 0);
+                }
+            }
+        }
+    }
+    if constexpr (WSPLIT) {  // four waves, four partial sets of the same 16 rows: through LDS (the tile is no longer needed); wave w finishes the value tiles w, w + 4, ...
+        float *xm = smem, *xl = smem + 64, *xo = smem + 128;  // [4][16], [4][16], [4][VT][64][4]
+        __syncthreads();
+        if (g4 == 0) {
+            xm[wave * 16 + col] = m_run;
+            xl[wave * 16 + col] = l_run;
+        }
+#pragma unroll
+        for (int v = 0; v < VT; ++v) *reinterpret_cast<f32x4 *>(xo + ((size_t)(wave * VT + v) * 64 + lane) * 4) = o[v];
+        __syncthreads();
+        float M = -INFINITY, L = 0.f, f[4];
+#pragma unroll
+        for (int w = 0; w < 4; ++w) M = fmaxf(M, xm[w * 16 + col]);
+#pragma unroll
+        for (int w = 0; w < 4; ++w) {
+            const float mw = xm[w * 16 + col];
+            f[w] = (mw == -INFINITY) ? 0.f : __expf(mw - M);
+            L += xl[w * 16 + col] * f[w];
+        }
+        if (!row_ok) return;
+        const float invl = n_splits == 1 ? (L > 0.f ? 1.f / L : 0.f) : 1.f;
+        const size_t pi = ((size_t)trow * H + head) * n_splits + split;
+        for (int v = wave; v < VT; v += 4) {
+            f32x4 s{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int w = 0; w < 4; ++w) {
+                const f32x4 ow = *reinterpret_cast<const f32x4 *>(xo + ((size_t)(w * VT + v) * 64 + lane) * 4);
+#pragma unroll
+                for (int r = 0; r < 4; ++r) s[r] += ow[r] * f[w];
+            }
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                const int c = 16 * v + 4 * g4 + r;
+                if (c >= rank) continue;
+                if (n_splits == 1) out[(size_t)trow * ldo + (size_t)head * rank + c] = BF16::from_float(s[r] * invl);
+                else part_acc[pi * rank + c] = s[r];
+            }
+        }
+        if (n_splits > 1 && wave == 0 && g4 == 0) {
+            part_ml[2 * pi] = M;
+            part_ml[2 * pi + 1] = L;
+        }
+        return;
+    }
+    if (!row_ok) return;
+    const float invl = l_run > 0.f ? 1.f / l_run : 0.f;
+    const size_t pi = ((size_t)trow * H + head) * n_splits + split;
+#pragma unroll
+    for (int v = 0; v < VT; ++v) {
+        const int c = 16 * v + 4 * g4;
+        if (n_splits == 1) {
+            uint16_t *dst = out + (size_t)trow * ldo + (size_t)head * rank + c;
+            if ((rank & 3) == 0 && (ldo & 3) == 0) {
+                if (c < rank) *reinterpret_cast<u32x2 *>(dst) = u32x2{BF16::pack2(o[v][0] * invl, o[v][1] * invl), BF16::pack2(o[v][2] * invl, o[v][3] * invl)};
+            } else {
+#pragma unroll
+                for (int r = 0; r < 4; ++r)
+                    if (c + r < rank) dst[r] = BF16::from_float(o[v][r] * invl);
+            }
+        } else {
+#pragma unroll
+            for (int r = 0; r < 4; ++r)
+                if (c + r < rank) part_acc[pi * rank + c + r] = o[v][r];
+        }
+    }
+    if (n_splits > 1 && g4 == 0) {
+        part_ml[2 * pi] = m_run;
+        part_ml[2 * pi + 1] = l_run;
+    }
+}
+
 // ---- attention, step 1 (head form with a norm ahead of the rotation): one wave per (row, head and map of q | k, value head) ------------------
 // proj: q | k | v at columns 0 | H*M*dim | (H+G)*M*dim; M maps per head lie side by side ([map 1 | map 2] with M = 2).  Every (head, map) of q and
 // k: x / sqrt(mean x^2 + eps) * w over dim (qw / kw [dim], shared by all heads and maps; head_norm 0: none), then the rotation of the first
