@@ -381,7 +381,7 @@ static int attention_core(tl_hybrid *e, const tl_hybrid_layer &L, const void *kp
     }
     if (dk4 <= 16 && vt_n <= 4) return launch_attn_tile<D, 16, 4>(e, L, kpool, vpool, v_row, m, sh, gate, ldg, out, ldo, x);
     if (dk4 <= 32 && vt_n <= 8) return launch_attn_tile<D, 32, 8>(e, L, kpool, vpool, v_row, m, sh, gate, ldg, out, ldo, x);
-    if (vt_n <= 12 && sizeof(S) == 2) return launch_attn_tile<D, 64, 12>(e, L, kpool, vpool, v_row, m, sh, gate, ldg, out, ldo, x);  // (a 192-wide latent beside a 64-wide rotated part)
+    if (vt_n <= 12 && sizeof(S) == 2) return launch_attn_tile<D, 64, 12>(e, L, kpool, vpool, v_row, m, sh, gate, ldg, out, ldo, x);  // (values up to 192 wide)
     return launch_attn_tile<D, 64, 16>(e, L, kpool, vpool, v_row, m, sh, gate, ldg, out, ldo, x);
 }
 

@@ -27,6 +27,8 @@ __device__ __forceinline__ float block_sum(float v, float *red) {
 
 __device__ __forceinline__ float sigmoid_f(float x) { return 1.f / (1.f + expf(-x)); }
 __device__ __forceinline__ float silu_f(float x) { return x / (1.f + expf(-x)); }
+// SiLU through the hardware's exponential and reciprocal (relative error of a few 1e-7), where every workgroup that reads a row forms it again
+__device__ __forceinline__ float silu_hw(float x) { return x * __builtin_amdgcn_rcpf(1.f + __expf(-x)); }
 __device__ __forceinline__ float softplus_f(float x) { return x > 20.f ? x : log1pf(expf(x)); }
 __device__ __forceinline__ float act_f(float z, int kind) {
     if (kind == 0) return 0.5f * z * (1.f + erff(z * 0.70710678118654752440f));
@@ -2080,13 +2082,13 @@ __global__ __launch_bounds__(256) void linrec_kernel(const float *proj, int ldp,
         __syncthreads();  // the previous tile's recurrence is done with the LDS
 #pragma unroll
         for (int it = 0; it < NIT; ++it) {
-            qs[tid + 256 * it] = (silu & 1) ? silu_f(rq[it]) : rq[it];  // (silu(0) = 0: padding stays zero)
-            ks[tid + 256 * it] = ((silu & 1) ? silu_f(rk[it]) : rk[it]) * k_mul;
+            qs[tid + 256 * it] = (silu & 1) ? silu_hw(rq[it]) : rq[it];  // (silu(0) = 0: padding stays zero)
+            ks[tid + 256 * it] = ((silu & 1) ? silu_hw(rk[it]) : rk[it]) * k_mul;
             if constexpr (CHAN) as[tid + 256 * it] = ra[it];
         }
 #pragma unroll
         for (int it = 0; it < NV; ++it)
-            if (tid + 256 * it < TB * CPB) vs[tid + 256 * it] = (silu & 2) ? silu_f(rv[it]) : rv[it];
+            if (tid + 256 * it < TB * CPB) vs[tid + 256 * it] = (silu & 2) ? silu_hw(rv[it]) : rv[it];
         if (tid < TB) {
             if constexpr (!CHAN) as[tid] = rg;
             bs[tid] = rb;
