@@ -23,6 +23,8 @@
  *                      as a1 - lambda a2, are divided by their RMS over vdim and multiplied by 1 - diff_init.
  *                      Also: scores capped by softcap tanh(s / softcap), a distance bias taken off the scores (bias_slope_dev[h] times
  *                      the distance between query and key), and a query temperature 1 + q_temp_coef ln(floor((p + 1) / q_temp_every) + 1).
+ *                      Also: the first keys of a sequence kept visible beside a window (keep_first), and a short causal depthwise convolution
+ *                      without an activation on q, k and v ahead of everything else (conv_taps; its last inputs live in the state slot).
  *   TL_MIX_DELTA       gated delta rule: a [key_dim, value_dim] float32 state per head that decays, is corrected
  *                      towards the new value along the new key and is read with the query; q/k/v pass a short
  *                      causal depthwise convolution + SiLU first.  The state and the convolution's last inputs
@@ -48,7 +50,7 @@
  *                      W_uv,h (sum_j p_j c_j) -- one K/V head of width kv_rank + rot_dim whose values are its leading
  *                      kv_rank columns.  Rotation frequencies may be rescaled (YaRN: rot_factor > 0).  kv_from >= 0: the
  *                      layer has no latent projection of its own and reads the pages of that earlier layer.  Options: a sliding
- *                      window (window), learned sinks (sink + sink_dev), one gate per head (gated 2).
+ *                      window (window), learned sinks (sink + sink_dev), one gate per head (gated 2), half-split rotation pairs (rot_half).
  *
  * A layer may hold TWO mixers side by side (beside): both read the same normed input, their results are summed with the factors
  * mix_scale.  Their projections share one input product and their output projections one output product.
@@ -56,18 +58,18 @@
  * Block forms: parallel_block 1 is x += m (mixer(h) + ff(h)) with one norm; 0 is the sequential pre-norm block
  * x += ls1 * mixer(norm1 x); x += ls2 * ff(norm2 x) with optional per-channel scales ls1 / ls2; 2 is the block with the norm on
  * the branch's OUTPUT, x += m norm1(mixer(x)); x += m norm2(ff(x)), whose sublayers read the stream itself; 3 has a norm on both sides
- * of every sublayer, x += m ls1 post1(mixer(norm1 x)); x += m ls2 post2(ff(norm2 x)).  A layer may end with a per-layer token input
+ * of every sublayer, x += m ls1 post1(mixer(norm1 x)); x += m ls2 post2(ff(norm2 x)), all of them RMS or all Dynamic Tanh; its dense feed-forwards may have biases.  A layer may end with a per-layer token input
  * (side_*): e = the layer's columns of a second embedding table, y = W_proj (gelu_tanh(W_gate x) * e), x += y / rms(y) * side_norm.
  * The embedding output may pass an RMS norm (embed_norm_dev); a second table indexed by a hash of the token and the one before it may
  * be added to it first (pair_embed_dev).  Norms: RMS or
  * Dynamic Tanh (tanh(alpha x) w + b).  Feed-forward kinds: W_down act(W_up h), W_down (act(W_gate h) * W_up h), or a
  * mixture of experts (softmax or sigmoid router with a selection-only correction, groups of neighbouring experts, identity
- * experts, a shared expert with or without a scalar gate; experts W_down act(W_up h) or, with moe_gated, W_down (act(W_gate h) *
+ * experts, group scores by the largest or the two largest choices, weights renormalised and scaled, a shared expert with or without a scalar gate; experts W_down act(W_up h) or, with moe_gated, W_down (act(W_gate h) *
  * W_up h); the router's weight on the expert's output or, with moe_scale_input, on its input).
  *
  * A contiguous range of layers may be repeated ("loop"): each pass has its own K/V pages / state slots, and is
  * entered through a [width, 2 width] projection of the running stream beside the embedding output (loop_in_dev; NULL:
- * the stream passes as it is) plus a per-pass offset vector.
+ * the stream passes as it is, or with the embedding output added from the second pass on: loop_add_embed) plus a per-pass offset vector.
  *
  * One step function serves prefill, decode and any mixture: tl_hybrid_step takes chunks of token ids for several
  * sequence slots (a chunk of one token is a decode step), runs them as one packed batch of rows and returns the
@@ -213,6 +215,18 @@ typedef struct tl_hybrid_layer {
     /* a second mixer on the same input: its kind, sizes, options and vectors (matrices of the layer itself are not read from it) */
     const struct tl_hybrid_layer *beside;
     float mix_scale;            /* factor on this mixer's result (0 is read as 1) */
+    /* attention: with a window, keys j < keep_first stay visible.  conv_taps > 0 (conv_dev over q | k | v, conv_channels = their columns): q, k and v pass a short causal
+     * depthwise convolution without an activation, ahead of the per-head norm and the rotation; its last inputs live in the sequence's slot */
+    int keep_first;
+    /* mixture of experts, further options */
+    int moe_group_top2;         /* a group scores the sum of its two largest choices (0: its largest) */
+    int moe_renorm;             /* the weights of the experts taken are divided by their sum + 1e-20 */
+    float moe_scale;            /* factor on the weights, behind that (0 is read as 1) */
+    /* biases of a dense feed-forward (TL_BLOCK_SANDWICH): [rows of w_in2], [width]; NULL: none */
+    const float *ff_in_bias_dev, *ff_out_bias_dev;
+    /* Dynamic Tanh as the norm on a branch's result (TL_BLOCK_SANDWICH with norm_kind TL_NORM_DYT) */
+    const float *post_norm_bias_dev, *post_norm2_bias_dev; /* [width] */
+    float post_norm_alpha, post_norm2_alpha;
 } tl_hybrid_layer;
 
 typedef struct tl_hybrid_config {
@@ -241,6 +255,7 @@ typedef struct tl_hybrid_config {
                                     pair_buckets, row pair_buckets for a sequence's first token; NULL: none */
     int64_t pair_buckets, pair_mul_prev, pair_mul_cur;
     float logit_softcap;         /* > 0: logits <- logit_softcap tanh(logits / logit_softcap), after logit_scale */
+    int loop_add_embed;          /* a loop without loop_in_dev: the embedding output is added to the stream ahead of every pass but the first */
 } tl_hybrid_config;
 
 typedef struct tl_hybrid_stats {

@@ -1094,3 +1094,191 @@ def karorax_config(layers, width=64, vocab=101, eps=1e-5, bigram=(53, 5, 3), log
     if logit_softcap:
         cfg["logit_softcap"] = logit_softcap
     return cfg
+
+
+# ---- Vabuzen: x = embed[token]; a Dynamic Tanh norm before AND after every sublayer, one residual factor for the whole model; a looped range whose
+# ---- later passes get the embedding output added back, and every pass its own vector.  Mixers: short convolutions on q, k and v ahead of
+# ---- sliding-window attention that keeps the first tokens, with a one in the softmax denominator; latent attention with direct queries.
+# ---- Feed-forwards with biases, and experts chosen by groups.  Same conventions: float64, whole sequences, one function per mechanism. ---------
+
+def short_conv(z, w):
+    """z [L, C], w [C, taps]: out_t = sum_j w[:, j] z_(t - taps + 1 + j), nothing before the start.  No activation."""
+    L, taps = z.shape[0], w.shape[1]
+    out = np.zeros_like(z)
+    for t in range(L):
+        for back in range(min(taps, t + 1)):
+            out[t] += w[:, taps - 1 - back] * z[t - back]
+    return out
+
+
+def keep_first_window_attention(q, k, v, scale, window, keep_first):
+    """q [L, H, D], k [L, G, D], v [L, G, V]: query i sees key j <= i where i - j < window or j < keep_first; weights exp(s) / (1 + sum exp(s))."""
+    L, H, _ = q.shape
+    G = k.shape[1]
+    out = np.zeros((L, H, v.shape[2]))
+    for i in range(L):
+        seen = [j for j in range(i + 1) if i - j < window or j < keep_first]
+        for h in range(H):
+            s = (k[seen, h // (H // G)] @ q[i, h]) * scale
+            top = max(0.0, s.max())
+            e = np.exp(s - top)
+            out[i, h] = (e / (np.exp(-top) + e.sum())) @ v[seen, h // (H // G)]
+    return out
+
+
+def vabuzen_attention(W, m, mc, h, pos):
+    L, H, G, D, V = h.shape[0], mc["heads"], mc["kv_heads"], mc["dim"], mc["vdim"]
+    q, k, v = (short_conv(h @ W[m + n].T, W[m + n + ".conv"]) for n in "qkv")
+    rot = mc["rot"]
+    q = rotate_pairs(q.reshape(L, H, D), pos, rot["dims"], rot["base"])
+    k = rotate_pairs(k.reshape(L, G, D), pos, rot["dims"], rot["base"])
+    o = keep_first_window_attention(q, k, v.reshape(L, G, V), mc["scale"], mc["mask"]["size"], mc["mask"]["keep_first"])
+    return o.reshape(L, H * V) @ W[m + "o"].T
+
+
+def vabuzen_latent(W, m, mc, h, pos, eps):
+    L, H, D, R, V, C = h.shape[0], mc["heads"], mc["dim"], mc["rot_dim"], mc["vdim"], mc["kv_rank"]
+    f = [mc["rot"]["base"] ** (-2.0 * i / R) for i in range(R // 2)]
+    q = (h @ W[m + "q"].T).reshape(L, H, D + R)
+    down = h @ W[m + "dkv"].T
+    c, kr = rms_norm(down[:, :C], W[m + "dkv.norm"], eps), rotate_halves_by(down[:, None, C:], pos, f)
+    k, v = (c @ W[m + "uk"].T).reshape(L, H, D), (c @ W[m + "uv"].T).reshape(L, H, V)
+    o = causal_softmax_attention(np.concatenate([q[..., :D], rotate_halves_by(q[..., D:], pos, f)], -1), np.concatenate([k, np.repeat(kr, H, 1)], -1), v, mc["scale"])
+    return o.reshape(L, H * V) @ W[m + "o"].T
+
+
+def grouped_sigmoid_route(z, top, count, keep, scale):
+    """Scores s = sigmoid(z); `count` equal runs of neighbouring experts, a run scores the sum of its two largest s; the `top` largest s inside the `keep`
+    best runs are taken (ties: the lower index); weights s / (sum of the taken s + 1e-20) * scale.  Returns ({expert: weight}, margin): the margin is
+    how far the closest comparison that decided the choice was from going the other way (in units of s)."""
+    s = sigmoid(z)
+    per = len(z) // count
+    group = [np.sort(s[g * per:(g + 1) * per])[::-1][:2].sum() for g in range(count)]
+    order = sorted(range(count), key=lambda g: (-group[g], g))
+    margin = group[order[keep - 1]] - group[order[keep]] if keep < count else np.inf
+    allowed = sorted((j for j in range(len(z)) if j // per in order[:keep]), key=lambda j: (-s[j], j))
+    if top < len(allowed):
+        margin = min(margin, s[allowed[top - 1]] - s[allowed[top]])
+    total = sum(s[j] for j in allowed[:top]) + 1e-20
+    return {j: s[j] / total * scale for j in allowed[:top]}, margin
+
+
+def vabuzen_feed_forward(mlp, W, f, h, margins=None):
+    if mlp["kind"] == "dense":
+        return gelu_tanh(h @ W[f + "up"].T + W[f + "up.b"]) @ W[f + "down"].T + W[f + "down.b"]
+    r, out, row = mlp["router"], np.zeros_like(h), []
+    groups = r.get("groups") or {"count": 1, "keep": 1}
+    for t in range(h.shape[0]):
+        weights, margin = grouped_sigmoid_route(h[t] @ W[f + "router"].T, r["top"], groups["count"], groups["keep"], r["scale"])
+        row.append(margin)
+        for j, w in weights.items():
+            out[t] += w * gated_expert(W, f + f"e{j}.", h[t])
+    if margins is not None:
+        margins.append(np.array(row))
+    return out + gated_expert(W, f + "shared.", h) if mlp.get("shared") else out
+
+
+def vabuzen_forward(config, W, tokens, streams=None, margins=None):
+    """Logits [L, vocab] of a whole sequence; ``streams`` (a list) receives the residual stream after every layer run, ``margins`` one row of router
+    margins per run of a mixture of experts."""
+    W = {k: np.asarray(v, dtype=np.float64) for k, v in W.items()}
+    eps, mult = config["norm"]["eps"], config["residual_mult"]
+    pos = np.arange(len(tokens), dtype=np.float64)
+    dyt = lambda z, name: dyt_norm(z, W[name + ".alpha"], W[name], W[name + ".b"])
+    x = x0 = W["embed"][np.asarray(tokens)]
+    for i, t, first in muduvik_layer_order(config):
+        if first:
+            x = (x + x0 if t > 0 else x) + W["loop.step"][t]
+        spec, p = config["layers"][i], f"l{i}."
+        h = dyt(x, p + "norm1")
+        if spec["type"] == "attention":
+            y = vabuzen_attention(W, p + "mix.", spec["mixer"], h, pos)
+        elif spec["type"] == "latent_attention":
+            y = vabuzen_latent(W, p + "mix.", spec["mixer"], h, pos, eps)
+        else:
+            raise ValueError(spec["type"])
+        x = x + mult * dyt(y, p + "norm1b")
+        if spec.get("mlp"):
+            x = x + mult * dyt(vabuzen_feed_forward(spec["mlp"], W, p + "mlp.", dyt(x, p + "norm2"), margins), p + "norm2b")
+        if streams is not None:
+            streams.append(x.copy())
+    logits = dyt(x, "final.norm") @ W["head"].T
+    cap = config.get("logit_softcap")
+    return cap * np.tanh(logits / cap) if cap else logits
+
+
+def make_vabuzen_weights(config, seed=0):
+    """Random bf16-representable weights by tensor name (float32 arrays) for a Vabuzen config dict."""
+    import torch
+
+    gen = torch.Generator().manual_seed(seed)
+    Wd, out = config["width"], {}
+
+    def mat(rows, cols, scale=None):
+        s = scale if scale is not None else cols ** -0.5
+        return (torch.randn(rows, cols, generator=gen) * s).to(torch.bfloat16).float().numpy()
+
+    def vec(n, scale=0.1, shift=0.0):
+        return (torch.randn(n, generator=gen) * scale + shift).to(torch.bfloat16).float().numpy()
+
+    def norm(name, alpha):
+        out[name], out[name + ".b"] = vec(Wd, 0.2, 1.0), vec(Wd, 0.1)
+        out[name + ".alpha"] = torch.tensor(alpha * (0.8 + 0.4 * float(torch.rand((), generator=gen)))).to(torch.bfloat16).float().numpy()
+
+    out["embed"], out["head"] = mat(config["vocab"], Wd, 1.0), mat(config["vocab"], Wd)
+    norm("final.norm", 0.6)
+    if config.get("loop"):
+        out["loop.step"] = mat(config["loop"]["times"], Wd, 0.4)
+    for i, spec in enumerate(config["layers"]):
+        p, m, mc = f"l{i}.", f"l{i}.mix.", spec["mixer"]
+        norm(p + "norm1", 0.7)
+        norm(p + "norm1b", 0.9)
+        H, D, V = mc["heads"], mc["dim"], mc["vdim"]
+        out[m + "o"] = mat(Wd, H * V)
+        if spec["type"] == "attention":
+            for name, n in (("q", H * D), ("k", mc["kv_heads"] * D), ("v", mc["kv_heads"] * V)):
+                out[m + name], out[m + name + ".conv"] = mat(n, Wd, 1.4 * Wd ** -0.5), mat(n, mc["conv"], 0.7)
+        else:
+            R, C = mc["rot_dim"], mc["kv_rank"]
+            out[m + "q"], out[m + "dkv"], out[m + "dkv.norm"] = mat(H * (D + R), Wd, 1.4 * Wd ** -0.5), mat(C + R, Wd), vec(C, 0.1, 1.0)
+            out[m + "uk"], out[m + "uv"] = mat(H * D, C), mat(H * V, C)
+        mlp, f = spec.get("mlp"), p + "mlp."
+        if mlp:
+            norm(p + "norm2", 0.7)
+            norm(p + "norm2b", 0.9)
+            if mlp["kind"] == "dense":
+                out[f + "up"], out[f + "up.b"], out[f + "down"], out[f + "down.b"] = mat(mlp["ff"], Wd), vec(mlp["ff"], 0.3), mat(Wd, mlp["ff"]), vec(Wd, 0.3)
+            else:
+                E = mlp["router"]["experts"]
+                out[f + "router"] = mat(E, Wd, 2.0 * Wd ** -0.5)
+                names = [(f"e{e}.", mlp["expert"]["ff"]) for e in range(E)] + ([("shared.", mlp["shared"]["ff"])] if mlp.get("shared") else [])
+                for name, n in names:
+                    out[f + name + "gate"], out[f + name + "up"], out[f + name + "down"] = mat(n, Wd), mat(n, Wd), mat(Wd, n)
+    return out
+
+
+def vabuzen_moe(experts=6, top=2, ff=24, shared=40, groups=(3, 2), scale=1.3):
+    mlp = {"kind": "moe", "expert": {"ff": ff}, "router": {"experts": experts, "groups": {"count": groups[0], "keep": groups[1]}, "scale": scale, "top": top}}
+    if shared:
+        mlp["shared"] = {"ff": shared}
+    return mlp
+
+
+def vabuzen_attention_layer(heads=4, kv_heads=2, dim=16, vdim=24, conv=4, rot_dims=12, base=3000.0, scale=0.3, window=20, keep_first=3, mlp="default"):
+    mixer = {"conv": conv, "dim": dim, "heads": heads, "kv_heads": kv_heads, "mask": {"keep_first": keep_first, "size": window}, "rot": {"base": base, "dims": rot_dims},
+             "scale": scale, "vdim": vdim}
+    return {"type": "attention", "mixer": mixer, "mlp": {"kind": "dense", "ff": 72} if mlp == "default" else mlp}
+
+
+def vabuzen_latent_layer(heads=4, dim=16, vdim=24, rot_dim=8, kv_rank=40, base=5000.0, scale=0.2, mlp="default"):
+    mixer = {"dim": dim, "heads": heads, "kv_rank": kv_rank, "rot": {"base": base, "dims": rot_dim}, "rot_dim": rot_dim, "scale": scale, "vdim": vdim}
+    return {"type": "latent_attention", "mixer": mixer, "mlp": vabuzen_moe() if mlp == "default" else mlp}
+
+
+def vabuzen_config(layers, width=64, vocab=101, eps=1e-5, residual_mult=0.8, loop=None, logit_softcap=6.0):
+    cfg = {"architecture": "Vabuzen", "layers": layers, "norm": {"eps": eps}, "residual_mult": residual_mult, "vocab": vocab, "width": width}
+    if loop:
+        cfg["loop"] = {"start": loop[0], "stop": loop[1], "times": loop[2]}
+    if logit_softcap:
+        cfg["logit_softcap"] = logit_softcap
+    return cfg

@@ -43,7 +43,7 @@ namespace hy {
 
 struct MixState {             // what one mixer of a layer run keeps per sequence
     void *kpool = nullptr, *vpool = nullptr;      // attention: [pages, G, page, dim] / [pages, G, page, vdim] of the engine dtype
-    float *state = nullptr, *conv_state = nullptr; // delta: [slots, H, vdim, dim] / [slots, taps-1, C]
+    float *state = nullptr, *conv_state = nullptr; // delta: [slots, H, vdim, dim] / [slots, taps-1, C];  attention with a short convolution: - / [slots, taps-1, C]
                                                    // linrec: [slots, H, vdim (+1), dim] / the gates' running maximum [slots, H]
     // latent: kpool = [pages, page, kv_rank + rot_dim] (vpool unused); with kv_from the pages of an earlier run (not owned)
 };
@@ -132,9 +132,21 @@ static int layer_read_cols(const tl_hybrid *e, int layer) {
     const tl_hybrid_layer &L = e->layers[layer], &B = e->beside[layer];
     return L.heads * L.vdim + (B.kind >= 0 ? B.heads * B.vdim : 0);
 }
-static int conv_channels(const tl_hybrid_layer &L) { return 2 * L.kv_heads * L.dim + L.heads * L.vdim; }
-// floats of one sequence's recurrent state, and of what travels beside it (delta: the convolution's last inputs; expgate: the running maximum)
+static int conv_channels(const tl_hybrid_layer &L) {
+    if (L.kind == TL_MIX_ATTENTION) return attn_maps(L) * (L.heads + L.kv_heads) * L.dim + L.kv_heads * L.vdim;
+    return 2 * L.kv_heads * L.dim + L.heads * L.vdim;
+}
+// mixers that keep something in the sequence's slot (beside or instead of pages)
+static bool has_slot_state(const tl_hybrid_layer &L) {
+    return L.kind == TL_MIX_DELTA || L.kind == TL_MIX_LINREC || (L.kind == TL_MIX_ATTENTION && L.conv_taps > 1);
+}
+// an attention layer whose options only the per-head preparation has
+static bool head_prep(const tl_hybrid_layer &L) {
+    return L.kind == TL_MIX_ATTENTION && (L.diff_maps || L.qk_head_norm || L.window > 0 || L.gated == 2 || L.conv_taps > 0);
+}
+// floats of one sequence's recurrent state, and of what travels beside it (the convolution's last inputs; expgate: the running maximum)
 static size_t state_floats(const tl_hybrid_layer &L) {
+    if (L.kind == TL_MIX_ATTENTION) return 0;
     if (L.kind == TL_MIX_LINREC) return (size_t)L.heads * L.dim * (L.vdim + (L.rec_kind == TL_REC_EXPGATE ? 1 : 0));
     return (size_t)L.heads * L.dim * L.vdim;
 }
@@ -178,7 +190,8 @@ struct NormTail {
 // out (+)= A . W^T by shape: a few rows stream the weights once per column (row kernel), more go through the MFMA tile kernel
 template <typename D>
 static int linear_t(const void *A, int lda, const void *W, float *out, int ldc, int M, int N, int K, int epi, float alpha, const float *bias,
-                    int force, hipStream_t st, int batch = 1, long sa = 0, long sw = 0, long sc = 0, NormTail *tail = nullptr, const SegSkip *skip = nullptr) {
+                    int force, hipStream_t st, int batch = 1, long sa = 0, long sw = 0, long sc = 0, NormTail *tail = nullptr, const SegSkip *skip = nullptr,
+                    const BranchTail *branch = nullptr, bool *branch_done = nullptr) {
     using S = typename D::storage;
     if (M <= 0 || N <= 0 || batch <= 0) return TL_OK;
     const int vec_ok = (K % 8 == 0) && (lda % 8 == 0) && ((uintptr_t)A % 16 == 0) && ((uintptr_t)W % 16 == 0) && sa % 8 == 0 && sw % 8 == 0;
@@ -207,21 +220,25 @@ static int linear_t(const void *A, int lda, const void *W, float *out, int ldc, 
     const float *nw = with_tail ? tail->w : nullptr, *nb = with_tail ? tail->b : nullptr;
     const float nalpha = with_tail ? tail->alpha : 0.f;
     S *nout = with_tail ? (S *)tail->out : nullptr;
+    const bool with_branch = branch && epi == 0 && batch == 1 && ldc == N;  // (the product forms a whole branch: its tail leaves with it, `out` is not written)
+    const BranchTail bt = with_branch ? *branch : BranchTail{};
 #define HY_GEMM(KERN, E) \
-    hipLaunchKernelGGL((KERN<D, E>), grid, block, 0, st, (const S *)A, lda, (const S *)W, out, ldc, M, N, K, alpha, bias, vec_ok, sa, sw, sc, nw, nb, nalpha, nout)
+    hipLaunchKernelGGL((KERN<D, E>), grid, block, 0, st, (const S *)A, lda, (const S *)W, out, ldc, M, N, K, alpha, bias, vec_ok, sa, sw, sc, nw, nb, nalpha, nout, bt)
 #define HY_GEMM_ROWS(E) \
-    hipLaunchKernelGGL((gemm_rows_kernel<D, E>), grid, block, 0, st, (const S *)A, lda, (const S *)W, out, ldc, M, N, K, alpha, bias, vec_ok, sa, sw, sc, nw, nb, nalpha, nout, sk)
+    hipLaunchKernelGGL((gemm_rows_kernel<D, E>), grid, block, 0, st, (const S *)A, lda, (const S *)W, out, ldc, M, N, K, alpha, bias, vec_ok, sa, sw, sc, nw, nb, nalpha, nout, sk, bt)
     if (rows) {
         dim3 grid((N + 3) / 4, batch), block(256);
         const SegSkip sk = skip ? *skip : SegSkip{};
-        if (epi == 0) HY_GEMM_ROWS(0);
+        if (with_branch) HY_GEMM_ROWS(5);
+        else if (epi == 0) HY_GEMM_ROWS(0);
         else if (epi == 1) HY_GEMM_ROWS(1);
         else if (epi == 2) HY_GEMM_ROWS(2);
         else if (!with_tail) HY_GEMM_ROWS(3);
         else HY_GEMM_ROWS(4);
     } else {
         dim3 grid(((M + 63) / 64) * ((N + 63) / 64), batch), block(256);
-        if (epi == 0) HY_GEMM(gemm_tile_kernel, 0);
+        if (with_branch) HY_GEMM(gemm_tile_kernel, 5);
+        else if (epi == 0) HY_GEMM(gemm_tile_kernel, 0);
         else if (epi == 1) HY_GEMM(gemm_tile_kernel, 1);
         else if (epi == 2) HY_GEMM(gemm_tile_kernel, 2);
         else if (!with_tail) HY_GEMM(gemm_tile_kernel, 3);
@@ -230,6 +247,7 @@ static int linear_t(const void *A, int lda, const void *W, float *out, int ldc, 
 #undef HY_GEMM
 #undef HY_GEMM_ROWS
     if (with_tail) tail->done = true;
+    if (branch_done) *branch_done = with_branch;
     TL_CHECK_LAUNCH("hybrid linear");
     return TL_OK;
 }
@@ -307,10 +325,11 @@ struct AttnExtra {
     const float *slopes = nullptr;  // [heads] distance bias: s -= slope (i - j)
     const float *sinks = nullptr;   // [heads] learned sinks (with L.sink)
     float out_scale = 1.f;   // factor on the read-out
+    int keep_first = 0;      // with a window: the first keys of a sequence stay visible
     bool any() const { return window > 0 || vshare != 1 || gate_per_head || out32 || softcap > 0.f || slopes || sinks || out_scale != 1.f; }
 };
 
-// a windowed layer's split of the keys: a decode step sees at most `window` keys, whatever the context
+// a windowed layer's split of the keys: a decode step sees at most `window` keys (a window's and the kept first ones), whatever the context
 static StepShape window_shape(const StepShape &sh, int window) {
     StepShape w = sh;
     if (window > 0 && sh.n_splits > 1) {
@@ -345,7 +364,7 @@ static int launch_attn_tile(tl_hybrid *e, const tl_hybrid_layer &L, const void *
     hipLaunchKernelGGL(kern, grid, dim3(256), lds, e->stream, e->qbuf, (const S *)kpool, (const S *)vpool, m.seq_row0, m.seq_slot, m.row_pos,
                        e->table_dev, c.max_pages_per_seq, c.page_size, L.heads, L.kv_heads, L.dim, L.vdim, L.scale, L.sink, HGB, n_hblk, sh.keys_per_split,
                        sh.n_splits, gate, ldg, (S *)out, ldo, e->part_acc, e->part_ml, page_shift, vec_ok, v_row, x.window, x.vshare, x.gate_per_head, x.out32,
-                       x.softcap, x.slopes, x.sinks, x.out_scale);
+                       x.softcap, x.slopes, x.sinks, x.out_scale, x.keep_first);
     TL_CHECK_LAUNCH("hybrid attention tile");
     if (sh.n_splits > 1) {
         hipLaunchKernelGGL((attn_merge_kernel<D>), dim3(sh.rows, L.heads), dim3(64), 0, e->stream, e->part_acc, e->part_ml, sh.n_splits, L.heads, L.vdim, gate,
@@ -361,7 +380,7 @@ static int attention_core(tl_hybrid *e, const tl_hybrid_layer &L, const void *kp
                           const float *gate, int ldg, void *out, int ldo, const AttnExtra &x = AttnExtra{}) {
     using S = typename D::storage;
     const tl_hybrid_config &c = e->cfg;
-    const StepShape sh = window_shape(sh0, x.window);
+    const StepShape sh = window_shape(sh0, x.window > 0 ? x.window + x.keep_first : 0);
     const int dk4 = (L.dim + 3) / 4, vt_n = (L.vdim + 15) / 16;
     // the two 64-wide tile templates serve widths that are multiples of 8 (whole 16-byte chunks); other widths beyond the 32-wide template
     // take the row kernel (the tile kernel faulted on a 136 / 130-wide head in float32, cause not found), and float32 pages take the 16-tile
@@ -375,7 +394,7 @@ static int attention_core(tl_hybrid *e, const tl_hybrid_layer &L, const void *kp
         hipLaunchKernelGGL((attn_rows_kernel<D>), dim3(sh.rows, L.heads), dim3(64), (L.dim + 64) * sizeof(float), e->stream, e->qbuf, (const S *)kpool,
                            (const S *)vpool, m.row_seq, m.row_pos, m.seq_slot, e->table_dev, c.max_pages_per_seq, c.page_size, L.heads, L.kv_heads, L.dim,
                            L.vdim, L.scale, L.sink, gate, ldg, (S *)out, ldo, v_row, x.window, x.vshare, x.gate_per_head, x.out32, x.softcap, x.slopes,
-                           x.sinks, x.out_scale);
+                           x.sinks, x.out_scale, x.keep_first);
         TL_CHECK_LAUNCH("hybrid attention");
         return TL_OK;
     }
@@ -570,18 +589,25 @@ static int mixer_part_t(tl_hybrid *e, size_t ri, int part, float *proj, typename
     const int rows = sh.rows, n_seqs = sh.n_seqs, H = L.heads, HV = L.heads * L.vdim;
     if (L.kind == TL_MIX_ATTENTION) {
         const int G = L.kv_heads;
-        if (L.diff_maps || L.qk_head_norm || L.window > 0 || L.gated == 2) {
-            // q / k normed per head ahead of the rotation, maps side by side, a window on the keys, one gate per head
+        if (head_prep(L)) {
+            // q / k normed per head ahead of the rotation, maps side by side, a window on the keys, one gate per head, short convolutions
             const int M = attn_maps(L);
+            ShortConv conv;
+            conv.taps = L.conv_taps, conv.w = L.conv_dev, conv.state = run.conv_state, conv.columns = conv_channels(L), conv.move = sh.max_len == 1;
             hipLaunchKernelGGL((attn_prep_head_kernel<D>), dim3(rows, M * (H + G) + G), dim3(64), 0, st, proj, ldp, m.row_seq, m.row_pos, m.seq_slot, e->table_dev,
                                c.max_pages_per_seq, c.page_size, inv_freq, L.rot_dims, L.rot_half, L.qk_head_norm, L.q_norm_dev, L.k_norm_dev, c.norm_eps,
                                H, G, M, L.dim, L.vdim, e->qbuf, (S *)run.kpool, (S *)run.vpool, L.w_in_bias_dev,
-                               L.q_temp_coef, L.q_temp_every);
-            TL_CHECK_LAUNCH("hybrid attention prep (per-head norm)");
+                               L.q_temp_coef, L.q_temp_every, m.seq_row0, conv);
+            TL_CHECK_LAUNCH("hybrid attention prep (per head)");
+            if (conv.taps > 1 && !conv.move) {
+                hipLaunchKernelGGL(conv_state_kernel, dim3((unsigned)(((size_t)n_seqs * conv.columns + 255) / 256)), dim3(256), 0, st, proj, ldp, conv.taps, conv.columns,
+                                   m.seq_row0, m.seq_slot, run.conv_state, n_seqs);
+                TL_CHECK_LAUNCH("hybrid conv state");
+            }
             const float *gate = L.gated ? proj + (size_t)M * (H + G) * L.dim + (size_t)G * L.vdim : nullptr;
             AttnExtra x;
             x.window = L.window, x.vshare = M, x.gate_per_head = L.gated == 2, x.out_scale = out_scale;
-            x.softcap = L.softcap, x.slopes = L.bias_slope_dev;
+            x.softcap = L.softcap, x.slopes = L.bias_slope_dev, x.keep_first = L.keep_first;
             if (!L.diff_maps) return attention_core<D>(e, L, run.kpool, run.vpool, L.vdim, m, sh, gate, ldp, cat, ldcat, x);
             tl_hybrid_layer A = L;  // every map is a head of its own over M * G K/V heads; the read-outs stay float32 for the combination
             A.heads = M * H, A.kv_heads = M * G;
@@ -621,7 +647,7 @@ static int mixer_part_t(tl_hybrid *e, size_t ri, int part, float *proj, typename
         }
         hipLaunchKernelGGL((latent_prep_kernel<D>), dim3(rows, H + 1), dim3(64), 0, st, q, ldq, H, L.dim, L.rot_dim, L.kv_rank, proj, ldp, kv0,
                            L.dkv_norm_dev, c.norm_eps, own, m.row_seq, m.row_pos, m.seq_slot, e->table_dev, c.max_pages_per_seq, c.page_size,
-                           inv_freq, L.rot_dims, e->rot_mult[2 * layer + part], (S *)e->db, e->qbuf, (S *)run.kpool);
+                           inv_freq, L.rot_dims, L.rot_half, e->rot_mult[2 * layer + part], (S *)e->db, e->qbuf, (S *)run.kpool);
         TL_CHECK_LAUNCH("hybrid latent prep");
         // the keys' per-head projection moves onto the query: q_h' = W_uk,h^T q_h  -> qbuf[t, h, 0 .. kv_rank)
         HY_TRY(linear_t<D>(e->db, H * L.dim, L.uk_t_dev, e->qbuf, H * DT, rows, L.kv_rank, L.dim, 0, 1.f, nullptr, 0, st, H, L.dim, (long)L.kv_rank * L.dim, DT));
@@ -705,6 +731,12 @@ static int mixer_t(tl_hybrid *e, size_t ri, const Meta &m, const StepShape &sh, 
 }
 
 
+static RouteOpts route_opts(const tl_hybrid_layer &L) {
+    RouteOpts o;
+    o.group_top2 = L.moe_group_top2, o.renorm = L.moe_renorm, o.scale = L.moe_scale != 0.f ? L.moe_scale : 1.f;
+    return o;
+}
+
 // the feed-forward's activation: proj columns up0 .. -> cat columns col0 .. col0 + L.ff
 template <typename D>
 static int ff_act_t(tl_hybrid *e, const tl_hybrid_layer &L, int rows, int ldp, int up0, int ldcat, int col0) {
@@ -716,23 +748,24 @@ static int ff_act_t(tl_hybrid *e, const tl_hybrid_layer &L, int rows, int ldp, i
             const int ET = L.experts + L.identity, r0 = up0 + 2 * L.ff;
             hipLaunchKernelGGL((moe_gated_act_kernel<D>), grid, dim3(256), 0, st, e->proj, ldp, r0, L.moe_shared_sg ? r0 + ET : -1, up0, up0 + L.ff, L.experts,
                                L.identity, L.top, L.groups, L.keep, L.expert_ff, L.shared_ff, L.correction_dev, L.router_bias_dev, (S *)e->cat, ldcat, col0, e->idw, L.moe_router,
-                               L.moe_scale_input, L.ff_act);
+                               route_opts(L), L.moe_scale_input, L.ff_act);
             TL_CHECK_LAUNCH("hybrid moe route (gated experts)");
             return TL_OK;
         }
         const int ET = L.experts + L.identity, r0 = up0 + L.ff;  // shared up | expert ups | router | shared gate | padding
         hipLaunchKernelGGL((moe_route_act_kernel<D>), grid, dim3(256), 0, st, e->proj, ldp, r0, r0 + ET, up0, up0 + L.shared_ff,
-                           L.experts, L.identity, L.top, L.groups, L.keep, L.expert_ff, L.shared_ff, L.correction_dev, L.router_bias_dev, (S *)e->cat, ldcat, col0, e->idw, L.moe_router);
+                           L.experts, L.identity, L.top, L.groups, L.keep, L.expert_ff, L.shared_ff, L.correction_dev, L.router_bias_dev, (S *)e->cat, ldcat, col0, e->idw, L.moe_router,
+                           route_opts(L));
         TL_CHECK_LAUNCH("hybrid moe route");
         return TL_OK;
     }
     const size_t n = (size_t)rows * L.ff;
     if (L.ff_kind == TL_FF_GATED)
         hipLaunchKernelGGL((ff_gated_act_kernel<D>), dim3((unsigned)((n + 255) / 256)), dim3(256), 0, st, e->proj, ldp, up0, up0 + L.ff, L.ff, L.ff_act,
-                           (S *)e->cat, ldcat, col0, rows);
+                           (S *)e->cat, ldcat, col0, rows, L.ff_in_bias_dev);
     else
         hipLaunchKernelGGL((ff_act_kernel<D>), dim3((unsigned)((n + 255) / 256)), dim3(256), 0, st, e->proj, ldp, up0, L.ff, L.ff_act, (S *)e->cat, ldcat, col0,
-                           rows);
+                           rows, L.ff_in_bias_dev);
     TL_CHECK_LAUNCH("hybrid ff act");
     return TL_OK;
 }
@@ -740,7 +773,8 @@ static int ff_act_t(tl_hybrid *e, const tl_hybrid_layer &L, int rows, int ldp, i
 // a feed-forward of its own matrices on the D rows e->h: out (+)= (epi, alpha, col as in linear_t) its result.  Where the result is added (epi 1 / 3) the
 // identity experts' part is added too; a caller that takes the bare result (epi 0) adds it itself.
 template <typename D>
-static int ff_t(tl_hybrid *e, const tl_hybrid_layer &L, int rows, float *out, int epi, float alpha, const float *col, NormTail *tail) {
+static int ff_t(tl_hybrid *e, const tl_hybrid_layer &L, int rows, float *out, int epi, float alpha, const float *col, NormTail *tail, const BranchTail *branch = nullptr,
+                bool *branch_done = nullptr) {
     using S = typename D::storage;
     const int W = e->cfg.width, nin2 = ff_in_cols(L);
     hipStream_t st = e->stream;
@@ -750,7 +784,7 @@ static int ff_t(tl_hybrid *e, const tl_hybrid_layer &L, int rows, float *out, in
     if (few) {
         HY_TRY(linear_t<D>(e->h, W, (const S *)L.w_in2_dev + (size_t)2 * L.ff * W, e->proj + 2 * L.ff, nin2, rows, nin2 - 2 * L.ff, W, 0, 1.f, nullptr, 0, st));
         hipLaunchKernelGGL(moe_taken_mask_kernel, dim3(1), dim3(256), 0, st, e->proj, nin2, 2 * L.ff, rows, L.experts, L.identity, L.top, L.groups, L.keep,
-                           L.correction_dev, L.router_bias_dev, L.moe_router, e->moe_mask);
+                           L.correction_dev, L.router_bias_dev, L.moe_router, route_opts(L), e->moe_mask);
         TL_CHECK_LAUNCH("hybrid moe taken experts");
         in_skip.mask = out_skip.mask = e->moe_mask;
         in_skip.lead = out_skip.lead = L.shared_ff, in_skip.len = out_skip.len = L.expert_ff;
@@ -763,7 +797,63 @@ static int ff_t(tl_hybrid *e, const tl_hybrid_layer &L, int rows, float *out, in
         hipLaunchKernelGGL((identity_axpy_kernel<D>), dim3((unsigned)((n + 255) / 256)), dim3(256), 0, st, out, (const S *)e->h, e->idw, col, alpha, W, rows);
         TL_CHECK_LAUNCH("hybrid identity experts");
     }
-    return linear_t<D>(e->cat, L.ff, L.w_out2_dev, out, W, rows, W, L.ff, epi, alpha, col, 0, st, 1, 0, 0, 0, tail, few ? &out_skip : nullptr);
+    return linear_t<D>(e->cat, L.ff, L.w_out2_dev, out, W, rows, W, L.ff, epi, alpha, col, 0, st, 1, 0, 0, 0, tail, few ? &out_skip : nullptr, branch, branch_done);
+}
+
+// one run of the block with norms on both sides where the norms are Dynamic Tanh (no statistics of a row): a branch's norm, its sum, the entry of the loop pass that
+// comes next and the norm that reads the new stream are one element-wise tail.  It rides the product that forms the branch (row and 64-wide tile kernels); behind the
+// 256-wide tile GEMM it is a launch of its own.  h_ready / entered: what the run leaves behind for the next one.
+template <typename D>
+static int dyt_sandwich_t(tl_hybrid *e, size_t ri, const Meta &m, const StepShape &sh, bool &h_ready, bool &entered) {
+    const tl_hybrid_config &c = e->cfg;
+    const tl_hybrid_layer &L = e->layers[e->runs[ri].layer];
+    hipStream_t st = e->stream;
+    const int rows = sh.rows, W = c.width, nmix = layer_mixer_cols(e, e->runs[ri].layer), HV = layer_read_cols(e, e->runs[ri].layer);
+    const Run *next = ri + 1 < e->runs.size() ? &e->runs[ri + 1] : nullptr;
+    if (next && next->enters_pass && (c.loop_in_dev || e->trace)) next = nullptr;  // (a projection comes between, or the stream is kept as it is ahead of the entry)
+    auto tail = [&](bool second) {  // of the mixer's (false) or the feed-forward's result
+        BranchTail t;
+        t.x = e->x, t.mult = c.residual_mult;
+        t.bias = second ? L.ff_out_bias_dev : nullptr, t.ls = second ? L.ls2_dev : L.ls1_dev;
+        t.pw = second ? L.post_norm2_dev : L.post_norm_dev, t.pb = second ? L.post_norm2_bias_dev : L.post_norm_bias_dev;
+        t.palpha = second ? L.post_norm2_alpha : L.post_norm_alpha;
+        if (!second && L.ff > 0) t.h = e->h, t.nw = L.norm2_dev, t.nb = L.norm2_bias_dev, t.nalpha = L.norm2_alpha;
+        else if (next) {
+            const tl_hybrid_layer &Nx = e->layers[next->layer];
+            t.h = e->h, t.nw = Nx.norm_dev, t.nb = Nx.norm_bias_dev, t.nalpha = Nx.norm_alpha;
+            if (next->enters_pass) t.vec = c.loop_step_dev + (size_t)next->pass * W, t.add = c.loop_add_embed && next->pass > 0 ? e->x0 : nullptr;
+        }
+        return t;
+    };
+    auto finish = [&](const BranchTail &t, bool done) -> int {
+        if (done) return TL_OK;
+        const size_t n = (size_t)rows * W;
+        if (W % 4 == 0) hipLaunchKernelGGL((branch_tail_kernel<D, 4>), dim3((unsigned)((n / 4 + 255) / 256)), dim3(256), 0, st, e->y, t, W, n);
+        else hipLaunchKernelGGL((branch_tail_kernel<D, 1>), dim3((unsigned)((n + 255) / 256)), dim3(256), 0, st, e->y, t, W, n);
+        TL_CHECK_LAUNCH("hybrid branch tail");
+        return TL_OK;
+    };
+    bool done = false;
+    HY_TRY(linear_t<D>(e->h, W, L.w_in_dev, e->proj, nmix, rows, nmix, W, L.w_in_bias_dev && !head_prep(L) ? 2 : 0, 1.f, L.w_in_bias_dev, 0, st));
+    HY_TRY(mixer_t<D>(e, ri, m, sh, nmix, HV));
+    const BranchTail t1 = tail(false);
+    HY_TRY(linear_t<D>(e->cat, HV, L.w_out_dev, e->y, W, rows, W, HV, 0, 1.f, nullptr, 0, st, 1, 0, 0, 0, nullptr, nullptr, &t1, &done));
+    HY_TRY(finish(t1, done));
+    if (L.ff > 0) {
+        const BranchTail t2 = tail(true);
+        const bool identity = L.ff_kind == TL_FF_MOE && L.identity > 0;  // (their part joins the branch ahead of its norm)
+        done = false;
+        HY_TRY(ff_t<D>(e, L, rows, e->y, 0, 1.f, nullptr, nullptr, identity ? nullptr : &t2, &done));
+        if (identity) {
+            const size_t n = (size_t)rows * W;
+            hipLaunchKernelGGL((identity_axpy_kernel<D>), dim3((unsigned)((n + 255) / 256)), dim3(256), 0, st, e->y, (const typename D::storage *)e->h, e->idw,
+                               (const float *)nullptr, 1.f, W, rows);
+            TL_CHECK_LAUNCH("hybrid identity experts");
+        }
+        HY_TRY(finish(t2, done));
+    }
+    h_ready = next != nullptr, entered = next && next->enters_pass;
+    return TL_OK;
 }
 
 // every layer run over the packed rows described by m
@@ -783,6 +873,7 @@ static int forward_t(tl_hybrid *e, const Meta &m, const StepShape &sh) {
                        c.embed_scale != 0.f ? c.embed_scale : 1.f, c.embed_norm_dev, c.final_norm_offset, c.norm_eps, pe);
     TL_CHECK_LAUNCH("hybrid embed");
     bool h_ready = false;  // e->h already holds this run's first norm (it left with the product that completed the previous residual sum)
+    bool entered = false;  // e->x already holds this run's loop-pass entry (likewise)
     // the Dynamic Tanh norm that follows a residual sum: element-wise, so it can ride the completing product's epilogue
     auto tail_for = [&](const float *w, const float *b, float alpha) {
         NormTail t;
@@ -798,10 +889,12 @@ static int forward_t(tl_hybrid *e, const Meta &m, const StepShape &sh) {
             const tl_hybrid_layer &Nx = e->layers[e->runs[ri + 1].layer];
             if (Nx.norm_kind == TL_NORM_DYT) next_first = tail_for(Nx.norm_dev, Nx.norm_bias_dev, Nx.norm_alpha);
         }
-        if (run.enters_pass && !c.loop_in_dev) {  // x <- x + step[pass]
+        if (run.enters_pass && entered) {
+        } else if (run.enters_pass && !c.loop_in_dev) {  // x <- x [+ x0 from the second pass on] + step[pass]
             const size_t n = (size_t)rows * W;
-            hipLaunchKernelGGL(add_rowvec_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, st, e->x, c.loop_step_dev + (size_t)run.pass * W, W, rows);
-            TL_CHECK_LAUNCH("hybrid pass offset");
+            hipLaunchKernelGGL(pass_entry_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, st, e->x, c.loop_add_embed && run.pass > 0 ? e->x0 : (const float *)nullptr,
+                               c.loop_step_dev + (size_t)run.pass * W, W, rows);
+            TL_CHECK_LAUNCH("hybrid pass entry");
         } else if (run.enters_pass) {  // x <- W_in [x ; x0] + step[pass]
             hipLaunchKernelGGL((pack2_kernel<D>), dim3(rows), dim3(256), 0, st, e->x, e->x0, (S *)e->cat2, W);
             TL_CHECK_LAUNCH("hybrid pack2");
@@ -838,15 +931,17 @@ static int forward_t(tl_hybrid *e, const Meta &m, const StepShape &sh) {
             continue;
         }
         if (!h_ready) HY_TRY(norm_t<D>(e, L.norm_kind, L.norm_dev, L.norm_bias_dev, L.norm_alpha, L.norm_offset, e->h, nullptr, rows));
-        h_ready = false;
-        if (c.parallel_block == TL_BLOCK_SANDWICH) {
+        h_ready = entered = false;
+        if (c.parallel_block == TL_BLOCK_SANDWICH && L.norm_kind == TL_NORM_DYT) {
+            HY_TRY(dyt_sandwich_t<D>(e, ri, m, sh, h_ready, entered));
+        } else if (c.parallel_block == TL_BLOCK_SANDWICH) {
             // x += m ls1 post1(W_o mixer(norm1 x));  x += m ls2 post2(ff(norm2 x));  x += side(x).  Each sum's kernel also writes what reads the new
             // stream next: the feed-forward's norm, the stream itself for the token input, or the next run's first norm.
             const tl_hybrid_layer *Nx = (ri + 1 < e->runs.size() && !e->runs[ri + 1].enters_pass) ? &e->layers[e->runs[ri + 1].layer] : nullptr;
             const bool side = L.side_gate_dev != nullptr;
             const int threads = rows < 64 ? 1024 : 256;
             // (biases: the per-head preparation of an attention layer adds them where it reads q, k and v; any other mixer gets them with the product)
-            const bool prep_adds_bias = L.kind == TL_MIX_ATTENTION && (L.diff_maps || L.qk_head_norm || L.window > 0 || L.gated == 2);
+            const bool prep_adds_bias = head_prep(L);
             HY_TRY(linear_t<D>(e->h, W, L.w_in_dev, e->proj, nmix, rows, nmix, W, L.w_in_bias_dev && !prep_adds_bias ? 2 : 0, 1.f, L.w_in_bias_dev, 0, st));
             HY_TRY(mixer_t<D>(e, ri, m, sh, nmix, HV));
             HY_TRY(linear_t<D>(e->cat, HV, L.w_out_dev, e->y, W, rows, W, HV, 0, 1.f, nullptr, 0, st));
@@ -854,15 +949,22 @@ static int forward_t(tl_hybrid *e, const Meta &m, const StepShape &sh) {
                 const int next = L.ff > 0 ? 2 : (side ? 1 : (Nx ? 2 : 0));
                 const float *nw = L.ff > 0 ? L.norm2_dev : (Nx ? Nx->norm_dev : nullptr);
                 hipLaunchKernelGGL((sandwich_add_kernel<D>), dim3(rows), dim3(threads), 0, st, e->x, e->y, L.post_norm_dev, L.norm_offset, c.norm_eps, c.residual_mult,
-                                   L.ls1_dev, next, nw, L.ff > 0 ? L.norm_offset : (Nx ? Nx->norm_offset : 0.f), (S *)e->h, W);
+                                   L.ls1_dev, next, nw, L.ff > 0 ? L.norm_offset : (Nx ? Nx->norm_offset : 0.f), (S *)e->h, W,
+                                   (const float *)nullptr);
                 TL_CHECK_LAUNCH("hybrid norm on the mixer's output");
                 h_ready = L.ff <= 0 && !side && next == 2;
             }
             if (L.ff > 0) {
                 HY_TRY(ff_t<D>(e, L, rows, e->y, 0, 1.f, nullptr, nullptr));
+                if (L.ff_kind == TL_FF_MOE && L.identity > 0) {
+                    const size_t n = (size_t)rows * W;
+                    hipLaunchKernelGGL((identity_axpy_kernel<D>), dim3((unsigned)((n + 255) / 256)), dim3(256), 0, st, e->y, (const S *)e->h, e->idw,
+                                       (const float *)nullptr, 1.f, W, rows);
+                    TL_CHECK_LAUNCH("hybrid identity experts");
+                }
                 const int next = side ? 1 : (Nx ? 2 : 0);
                 hipLaunchKernelGGL((sandwich_add_kernel<D>), dim3(rows), dim3(threads), 0, st, e->x, e->y, L.post_norm2_dev, L.norm_offset, c.norm_eps, c.residual_mult,
-                                   L.ls2_dev, next, Nx ? Nx->norm_dev : nullptr, Nx ? Nx->norm_offset : 0.f, (S *)e->h, W);
+                                   L.ls2_dev, next, Nx ? Nx->norm_dev : nullptr, Nx ? Nx->norm_offset : 0.f, (S *)e->h, W, L.ff_out_bias_dev);
                 TL_CHECK_LAUNCH("hybrid norm on the feed-forward's output");
                 h_ready = !side && next == 2;
             }
@@ -875,7 +977,7 @@ static int forward_t(tl_hybrid *e, const Meta &m, const StepShape &sh) {
                 TL_CHECK_LAUNCH("hybrid token input");
                 HY_TRY(linear_t<D>(e->cat, sd, L.side_proj_dev, e->y, W, rows, W, sd, 0, 1.f, nullptr, 0, st));
                 hipLaunchKernelGGL((sandwich_add_kernel<D>), dim3(rows), dim3(threads), 0, st, e->x, e->y, L.side_norm_dev, 0.f, c.norm_eps, 1.f, (const float *)nullptr,
-                                   Nx ? 2 : 0, Nx ? Nx->norm_dev : nullptr, Nx ? Nx->norm_offset : 0.f, (S *)e->h, W);
+                                   Nx ? 2 : 0, Nx ? Nx->norm_dev : nullptr, Nx ? Nx->norm_offset : 0.f, (S *)e->h, W, (const float *)nullptr);
                 TL_CHECK_LAUNCH("hybrid norm on the token input");
                 h_ready = Nx != nullptr;
             }
@@ -978,10 +1080,12 @@ static int check_mixer(const tl_hybrid_layer *layers, int i, const tl_hybrid_lay
         TL_REQUIRE(!(L.qk_unit_rms && (L.qk_norm || L.rot_half || L.v_mix != TL_VMIX_NONE)),
                    "hybrid_create: unit-RMS heads after the rotation do not combine with the whole-projection norm, half-split rotation pairs or value mixing");
         TL_REQUIRE(L.chunk >= 0 && L.v_mix >= TL_VMIX_NONE && L.v_mix <= TL_VMIX_BLEND, "hybrid_create: chunk >= 0, v_mix 0..2");
-        TL_REQUIRE(L.gated >= 0 && L.gated <= 2 && L.window >= 0, "hybrid_create: gated 0..2, window >= 0");
-        if (L.diff_maps || L.qk_head_norm || L.window > 0 || L.gated == 2) {
+        TL_REQUIRE(L.gated >= 0 && L.gated <= 2 && L.window >= 0 && L.keep_first >= 0, "hybrid_create: gated 0..2, window >= 0, keep_first >= 0");
+        TL_REQUIRE(L.conv_taps >= 0 && L.conv_taps <= 64 && (L.conv_taps == 0 || (L.conv_dev && !L.w_in_bias_dev)),
+                   "hybrid_create: an attention layer's short convolution needs its weights (at most 64 taps) and takes no projection biases");
+        if (head_prep(L)) {
             TL_REQUIRE(!L.qk_unit_rms && !L.qk_norm && L.v_mix == TL_VMIX_NONE && !L.talk_dev && !L.sink_dev && L.chunk == 0,
-                       "hybrid_create: per-head norms, maps, a window and per-head gates do not combine with unit-RMS heads, the whole-projection norm, value mixing, "
+                       "hybrid_create: per-head norms, maps, a window, per-head gates and short convolutions do not combine with unit-RMS heads, the whole-projection norm, value mixing, "
                        "mixed scores, learned sinks or a chunked mask");
             TL_REQUIRE(!L.qk_head_norm || (L.q_norm_dev && L.k_norm_dev), "hybrid_create: a norm per head needs its weights");
             TL_REQUIRE(!L.diff_maps || !L.sink, "hybrid_create: differential attention takes no sink");
@@ -1088,9 +1192,15 @@ extern "C" int tl_hybrid_create(const tl_hybrid_config *cfg, const tl_hybrid_lay
         if (c.parallel_block == TL_BLOCK_POSTNORM)
             TL_REQUIRE(L.norm_kind == TL_NORM_RMS && !L.ls1_dev && !L.ls2_dev && !looped, "hybrid_create: the block with the norm on the branch's output takes RMS norms, no layer scale and no loop");
         if (c.parallel_block == TL_BLOCK_SANDWICH) {
-            TL_REQUIRE(L.norm_kind == TL_NORM_RMS && L.post_norm_dev && (L.ff <= 0 || L.post_norm2_dev), "hybrid_create: the block with norms on both sides takes RMS norms and a weight for every branch's result");
-            TL_REQUIRE(L.ff <= 0 || L.ff_kind == TL_FF_PLAIN || L.ff_kind == TL_FF_GATED, "hybrid_create: the block with norms on both sides takes a dense feed-forward");
+            TL_REQUIRE(L.post_norm_dev && (L.ff <= 0 || L.post_norm2_dev), "hybrid_create: the block with norms on both sides takes a weight for every branch's result");
+            TL_REQUIRE(L.norm_kind == e->layers[0].norm_kind, "hybrid_create: the block with norms on both sides takes one kind of norm in all layers");
+            TL_REQUIRE(L.norm_kind == TL_NORM_RMS || (L.post_norm_bias_dev && (L.ff <= 0 || L.post_norm2_bias_dev) && !L.side_gate_dev),
+                       "hybrid_create: Dynamic Tanh norms on both sides need their biases and take no per-layer token input");
         }
+        TL_REQUIRE((!L.ff_in_bias_dev && !L.ff_out_bias_dev) || (L.ff_kind != TL_FF_MOE && c.parallel_block == TL_BLOCK_SANDWICH),
+                   "hybrid_create: feed-forward biases are read by dense feed-forwards in the block with norms on both sides only");
+        TL_REQUIRE((!L.moe_group_top2 && !L.moe_renorm && (L.moe_scale == 0.f || L.moe_scale == 1.f)) || (L.ff_kind == TL_FF_MOE && L.moe_router != TL_ROUTER_CHOSEN_SOFTMAX),
+                   "hybrid_create: group scores of two choices, renormalised and scaled weights belong to a router with scores");
         TL_REQUIRE((!L.side_gate_dev && !L.side_proj_dev && !L.side_norm_dev) ||
                        (c.parallel_block == TL_BLOCK_SANDWICH && L.side_gate_dev && L.side_proj_dev && L.side_norm_dev && c.side_dim > 0 && L.side_col0 >= 0 &&
                         L.side_col0 + c.side_dim <= c.side_cols),
@@ -1218,6 +1328,11 @@ extern "C" int tl_hybrid_create(const tl_hybrid_config *cfg, const tl_hybrid_lay
             HY_TRY(dev_alloc(p, &r.conv_state, mb, true));
             e->stats.state_bytes += (sb + mb) * 4;
         } else if (L.kind == TL_MIX_ATTENTION) {
+            if (has_slot_state(L)) {
+                const size_t cb = (size_t)c.max_slots * aux_floats(L);
+                HY_TRY(dev_alloc(p, &r.conv_state, cb, true));
+                e->stats.state_bytes += cb * 4;
+            }
             const size_t kb = (size_t)c.num_pages * attn_maps(L) * L.kv_heads * c.page_size * L.dim * es, vb = (size_t)c.num_pages * L.kv_heads * c.page_size * L.vdim * es;
             HY_TRY(dev_alloc(p, (char **)&r.kpool, kb, true));
             HY_TRY(dev_alloc(p, (char **)&r.vpool, vb, true));
@@ -1303,9 +1418,9 @@ extern "C" int tl_hybrid_begin(tl_hybrid *e, int slot) {
     for (size_t rm = 0; rm < 2 * e->runs.size(); ++rm) {  // the slot's recurrent state starts at zero (fill kernels: a caller may have a capture open on this stream)
         MixState &r = e->runs[rm / 2].mix[rm % 2];
         const tl_hybrid_layer &L = rm % 2 ? e->beside[e->runs[rm / 2].layer] : e->layers[e->runs[rm / 2].layer];
-        if (L.kind != TL_MIX_DELTA && L.kind != TL_MIX_LINREC) continue;
+        if (L.kind < 0 || !has_slot_state(L)) continue;
         const size_t sn = state_floats(L), cn = aux_floats(L);
-        hipLaunchKernelGGL(fill_kernel, dim3((unsigned)std::min<size_t>(1024, (sn + 255) / 256)), dim3(256), 0, e->stream, r.state + slot * sn, sn, 0.f);
+        if (sn) hipLaunchKernelGGL(fill_kernel, dim3((unsigned)std::min<size_t>(1024, (sn + 255) / 256)), dim3(256), 0, e->stream, r.state + slot * sn, sn, 0.f);
         hipLaunchKernelGGL(fill_kernel, dim3((unsigned)std::min<size_t>(1024, (cn + 255) / 256)), dim3(256), 0, e->stream, r.conv_state + slot * cn, cn, 0.f);
         TL_CHECK_LAUNCH("hybrid_begin: state fill");
     }
@@ -1328,9 +1443,9 @@ extern "C" int tl_hybrid_move(tl_hybrid *e, int src, int dst) {
     for (size_t rm = 0; rm < 2 * e->runs.size(); ++rm) {  // recurrent state and convolution inputs travel with the sequence; K/V pages stay where they are
         MixState &r = e->runs[rm / 2].mix[rm % 2];
         const tl_hybrid_layer &L = rm % 2 ? e->beside[e->runs[rm / 2].layer] : e->layers[e->runs[rm / 2].layer];
-        if (L.kind != TL_MIX_DELTA && L.kind != TL_MIX_LINREC) continue;
+        if (L.kind < 0 || !has_slot_state(L)) continue;
         const size_t sn = state_floats(L), cn = aux_floats(L);
-        HY_HIP(hipMemcpyAsync(r.state + dst * sn, r.state + src * sn, sn * 4, hipMemcpyDeviceToDevice, e->stream));
+        if (sn) HY_HIP(hipMemcpyAsync(r.state + dst * sn, r.state + src * sn, sn * 4, hipMemcpyDeviceToDevice, e->stream));
         HY_HIP(hipMemcpyAsync(r.conv_state + dst * cn, r.conv_state + src * cn, cn * 4, hipMemcpyDeviceToDevice, e->stream));
     }
     HY_HIP(hipMemcpyAsync(e->last_tok_dev + dst, e->last_tok_dev + src, 4, hipMemcpyDeviceToDevice, e->stream));

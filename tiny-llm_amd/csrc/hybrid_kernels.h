@@ -129,17 +129,38 @@ __global__ void pack2_kernel(const float *x, const float *x0, typename D::storag
         out[(size_t)t * 2 * width + c] = D::from_float(c < width ? x[(size_t)t * width + c] : x0[(size_t)t * width + c - width]);
 }
 
+// What happens to a branch's result y in the block with Dynamic Tanh norms on both sides, element by element, so that it can ride the product that forms y:
+//   x += mult * ls * (tanh(palpha * (y + bias)) * pw + pb);   x += add + vec  (the entry of a loop pass);   h = tanh(nalpha * x) * nw + nb  (the next sublayer's input)
+// bias, ls, vec, pw, pb, nw, nb: [N]; x, add: [M, N]; bias / ls / add / vec NULL: left out; h NULL: no next norm.
+struct BranchTail {
+    float *x = nullptr;
+    const float *bias = nullptr, *pw = nullptr, *pb = nullptr, *ls = nullptr, *add = nullptr, *vec = nullptr, *nw = nullptr, *nb = nullptr;
+    float palpha = 0.f, mult = 1.f, nalpha = 0.f;
+    void *h = nullptr;
+};
+template <typename D>
+__device__ __forceinline__ void branch_tail(const BranchTail &t, size_t i, int n, float y) {
+    const float b = (t.ls ? t.mult * t.ls[n] : t.mult) * (tanhf(t.palpha * (y + (t.bias ? t.bias[n] : 0.f))) * t.pw[n] + t.pb[n]);
+    float v = t.x[i] + b;
+    if (t.add) v += t.add[i];
+    if (t.vec) v += t.vec[n];
+    t.x[i] = v;
+    if (t.h) reinterpret_cast<typename D::storage *>(t.h)[i] = D::from_float(tanhf(t.nalpha * v) * t.nw[n] + t.nb[n]);
+}
+
 // ---- tile matrix product: out[M, N] (+)= A[M, K] . W[N, K]^T, float32 accumulation on the matrix cores ------------
 // 64 x 64 output tile per 256-thread workgroup, 4 waves of 32 x 32 (2 x 2 MFMA 16x16 tiles), K in steps of 32 through LDS.
 // bf16: v_mfma_f32_16x16x32_bf16; fp32: v_mfma_f32_16x16x4_f32 (full fp32 products).  Any M, N, K: edges are zero-filled in LDS.
 // EPI 0: out = acc   1: out += alpha * acc   2: out = acc + bias[n]   3: out += alpha * bias[n] * acc (a per-column scale on the way into the sum)
 //     4: as 3, and the Dynamic Tanh norm of the new sum leaves with it: nout[m, n] = tanh(nalpha * out) * nw[n] + nb[n] (D rows of N; the norm is
 //        element-wise, so the product that completes a residual sum can hand the next product its input)
+//     5: acc is a branch's result: BranchTail (out is not written)
 // blockIdx.y = a batch of independent products of one shape (the heads of a per-head projection): operands advance by sa / sw / sc elements.
 template <typename D, int EPI>
 __global__ __launch_bounds__(256) void gemm_tile_kernel(const typename D::storage *A, int lda, const typename D::storage *W, float *out,
                                                         int ldc, int M, int N, int K, float alpha, const float *bias, int vec_ok, long sa, long sw,
-                                                        long sc, const float *nw, const float *nb, float nalpha, typename D::storage *nout) {
+                                                        long sc, const float *nw, const float *nb, float nalpha, typename D::storage *nout,
+                                                        BranchTail tail) {
     using S = typename D::storage;
     A += (size_t)blockIdx.y * sa, W += (size_t)blockIdx.y * sw, out += (size_t)blockIdx.y * sc;
     constexpr bool BF = sizeof(S) == 2;
@@ -240,6 +261,7 @@ __global__ __launch_bounds__(256) void gemm_tile_kernel(const typename D::storag
                     else if constexpr (EPI == 1) *o += alpha * v;
                     else if constexpr (EPI == 2) *o = v + bias[gn];
                     else if constexpr (EPI == 3) *o += alpha * bias[gn] * v;
+                    else if constexpr (EPI == 5) branch_tail<D>(tail, (size_t)gm * N + gn, gn, v);
                     else {
                         const float xn = *o + alpha * bias[gn] * v;
                         *o = xn;
@@ -264,7 +286,7 @@ template <typename D, int EPI>
 __global__ __launch_bounds__(256) void gemm_rows_kernel(const typename D::storage *A, int lda, const typename D::storage *W, float *out,
                                                         int ldc, int M, int N, int K, float alpha, const float *bias, int vec_ok, long sa, long sw,
                                                         long sc, const float *nw, const float *nb, float nalpha, typename D::storage *nout,
-                                                        SegSkip skip) {
+                                                        SegSkip skip, BranchTail tail) {
     using S = typename D::storage;
     A += (size_t)blockIdx.y * sa, W += (size_t)blockIdx.y * sw, out += (size_t)blockIdx.y * sc;
     const int lane = threadIdx.x & 63;
@@ -328,6 +350,7 @@ __global__ __launch_bounds__(256) void gemm_rows_kernel(const typename D::storag
                 else if constexpr (EPI == 1) *o += alpha * v;
                 else if constexpr (EPI == 2) *o = v + bias[n];
                 else if constexpr (EPI == 3) *o += alpha * bias[n] * v;
+                else if constexpr (EPI == 5) branch_tail<D>(tail, (size_t)m * N + n, n, v);
                 else {
                     const float xn = *o + alpha * bias[n] * v;
                     *o = xn;
@@ -413,24 +436,25 @@ __global__ __launch_bounds__(64) void attn_rows_kernel(const float *qbuf, const 
                                                        const int32_t *block_table, int max_pages, int page_size, int H, int G, int dim, int vdim,
                                                        float scale, int sink, const float *gate, int ldg, typename D::storage *out, int ldo, int v_row,
                                                        int window, int vshare, int gate_per_head, float *out32, float softcap, const float *slopes,
-                                                       const float *sinks, float out_scale) {
+                                                       const float *sinks, float out_scale, int keep_first) {
     extern __shared__ float smem[];
     float *qs = smem;        // [dim]
     float *ps = smem + dim;  // [64]
     const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
     const int pos = row_pos[t], slot = seq_slot[row_seq[t]], g = h / (H / G);
-    // window > 0: the keys start window - 1 positions before the query.  vshare K/V heads in a row read one value head.
-    const int Gv = G / vshare, gv = g / vshare, k_lo = window > 0 ? max(0, pos - window + 1) : 0;
+    // window > 0: the keys are the first keep_first of the sequence and those from window - 1 positions before the query on, walked without the `gap`
+    // between them.  vshare K/V heads in a row read one value head.
+    const int Gv = G / vshare, gv = g / vshare, gap = window > 0 ? max(0, pos - window + 1 - keep_first) : 0, n_keys = pos + 1 - gap;
     const int32_t *bt = block_table + (size_t)slot * max_pages;
     for (int c = lane; c < dim; c += 64) qs[c] = qbuf[((size_t)t * H + h) * dim + c];
     __syncthreads();
     float m = sink ? (sinks ? sinks[h] : 0.f) : -INFINITY, l = sink ? 1.f : 0.f;
     const float slope = slopes ? slopes[h] : 0.f;
     float acc[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};  // vdim <= 512
-    for (int kb = k_lo; kb <= pos; kb += 64) {
-        const int j = kb + lane;
+    for (int kb = 0; kb < n_keys; kb += 64) {
+        const int jc = kb + lane, j = jc + (jc >= keep_first ? gap : 0);
         float s = -INFINITY;
-        if (j <= pos) {
+        if (jc < n_keys) {
             const typename D::storage *kr = kpool + (((size_t)bt[j / page_size] * G + g) * page_size + j % page_size) * dim;
             float d = 0.f;
             for (int c = 0; c < dim; ++c) d += qs[c] * D::to_float(kr[c]);
@@ -439,18 +463,18 @@ __global__ __launch_bounds__(64) void attn_rows_kernel(const float *qbuf, const 
             s -= slope * (float)(pos - j);
         }
         const float m_new = fmaxf(m, wave_max(s));
-        const float p = (j <= pos) ? expf(s - m_new) : 0.f;
+        const float p = (jc < n_keys) ? expf(s - m_new) : 0.f;
         const float corr = (m == -INFINITY) ? 0.f : expf(m - m_new);
         l = l * corr + wave_sum(p);
         m = m_new;
         __syncthreads();
         ps[lane] = p;
         __syncthreads();
-        const int cnt = min(64, pos - kb + 1);
+        const int cnt = min(64, n_keys - kb);
 #pragma unroll
         for (int i = 0; i < 8; ++i) acc[i] *= corr;
         for (int jj = 0; jj < cnt; ++jj) {
-            const int jg = kb + jj;
+            const int jg = kb + jj + (kb + jj >= keep_first ? gap : 0);
             const typename D::storage *vr = vpool + (((size_t)bt[jg / page_size] * Gv + gv) * page_size + jg % page_size) * v_row;
             const float pj = ps[jj];
 #pragma unroll
@@ -498,7 +522,7 @@ __global__ __launch_bounds__(256) void attn_tile_kernel(const float *qbuf, const
                                                         float scale, int sink, int HGB, int n_hblk, int keys_per_split, int n_splits, const float *gate,
                                                         int ldg, typename D::storage *out, int ldo, float *part_acc, float *part_ml, int page_shift,
                                                         int vec_ok, int v_row, int window_, int vshare_, int gate_per_head_, float *out32_,
-                                                        float softcap_, const float *slopes_, const float *sinks_, float out_scale_) {
+                                                        float softcap_, const float *slopes_, const float *sinks_, float out_scale_, int keep_first_) {
     using S = typename D::storage;
     extern __shared__ float smem[];
     // EXT false: plain causal attention into D rows, the options folded away at compile time
@@ -506,8 +530,10 @@ __global__ __launch_bounds__(256) void attn_tile_kernel(const float *qbuf, const
     const float *const slopes = EXT ? slopes_ : nullptr, *const sinks = EXT ? sinks_ : nullptr;
     const int window = EXT ? window_ : 0, vshare = EXT ? vshare_ : 1, gate_per_head = EXT ? gate_per_head_ : 0;
     float *const out32 = EXT ? out32_ : nullptr;
-    // window > 0: a query sees key j <= its position only if position - j < window; the walk starts at the first key the tile's first row sees,
-    // and a split key range (decode steps) is counted from there.  vshare: that many K/V heads in a row read one value head (maps over shared
+    const int keep_first = EXT ? keep_first_ : 0;
+    // window > 0: a query sees key j <= its position only if position - j < window or j < keep_first; the walk takes the first keep_first keys and then, over
+    // a `gap` no row of the tile sees, those from the first key of the tile's first row on.  Key ranges (kb, k_begin, k_end; a split of them in decode steps)
+    // count the walked keys: number jc is key jc below keep_first and key jc + gap from there on.  vshare: that many K/V heads in a row read one value head (maps over shared
     // values).  out32: the read-out as float32 rows [row, head, vdim] instead of D rows of `out` (no gate).
     // LDS rows as wide as the template: zeros behind dim / vdim, no guards in the product loops.  bfloat16 pages: the K tile stays bfloat16
     // in LDS ([64][4 DK4 + 8] 16-bit elements) and S^T runs on v_mfma_f32_16x16x32_bf16 (q rounded to bfloat16 like every other input of a
@@ -523,9 +549,9 @@ __global__ __launch_bounds__(256) void attn_tile_kernel(const float *qbuf, const
     if (t0 >= len) return;
     const int pos0 = row_pos[r0], slot = seq_slot[seq];
     const int32_t *bt = block_table + (size_t)slot * max_pages;
-    const int k_end_tile = pos0 + min(t0 + TQ, len);  // keys the tile's last query row sees
-    const int k_lo = window > 0 ? max(0, pos0 + t0 - window + 1) : 0;
-    const int k_begin = k_lo + split * keys_per_split, k_end = min(k_end_tile, k_lo + (split + 1) * keys_per_split);
+    const int gap = window > 0 ? max(0, pos0 + t0 - window + 1 - keep_first) : 0;
+    const int k_end_tile = pos0 + min(t0 + TQ, len) - gap;  // keys up to the one of the tile's last query row
+    const int k_begin = split * keys_per_split, k_end = min(k_end_tile, (split + 1) * keys_per_split);
     const int Gv = G / vshare, kvh_v = kvh / vshare;
     // this lane's query row (column of the transposed products)
     // WSPLIT (a tile with at most 16 query rows, i.e. decode steps): every wave holds the SAME 16 rows and takes the 16 keys `wave` of each
@@ -578,11 +604,11 @@ __global__ __launch_bounds__(256) void attn_tile_kernel(const float *qbuf, const
         auto load_tile = [&](int kb) __attribute__((always_inline)) {
 #pragma unroll
             for (int it = 0; it < NIT; ++it) {
-                const int pl = place[it], j = kb + (pl & 255), c8 = 8 * ((pl >> 8) & 0xffff);
+                const int pl = place[it], jc = kb + (pl & 255), j = jc + (jc >= keep_first ? gap : 0), c8 = 8 * ((pl >> 8) & 0xffff);
                 const bool is_v = (pl >> 24) & 1;
 #pragma unroll
                 for (int e = 0; e < 8; ++e) raw[it][e] = (S)0;
-                if (pl >= 0 && j < k_end && c8 < (is_v ? vdim : dim)) {
+                if (pl >= 0 && jc < k_end && c8 < (is_v ? vdim : dim)) {
                     const int pg = page_shift >= 0 ? (j >> page_shift) : (j / page_size), in_pg = j - pg * page_size;
                     const int wd = is_v ? vdim : dim;  // v_row: the width of a row of vpool (vdim, or the key row's when the values are its leading columns)
                     const S *src = (is_v ? vpool + (((size_t)bt[pg] * Gv + kvh_v) * page_size + in_pg) * v_row
@@ -652,10 +678,10 @@ __global__ __launch_bounds__(256) void attn_tile_kernel(const float *qbuf, const
                 }
 #pragma unroll
                 for (int r = 0; r < 4; ++r) {
-                    const int j = kb + 16 * n + 4 * g4 + r;
+                    const int jc = kb + 16 * n + 4 * g4 + r, j = jc + (jc >= keep_first ? gap : 0);
                     if (softcap > 0.f) a4[r] = softcap * tanh_t<KB16>(a4[r] * inv_cap);
                     if (slopes) a4[r] -= slope * (float)(qpos - j);
-                    a4[r] = (row_ok && j <= qpos && j < k_end && (window <= 0 || qpos - j < window)) ? a4[r] : -INFINITY;
+                    a4[r] = (row_ok && j <= qpos && jc < k_end && (window <= 0 || qpos - j < window || j < keep_first)) ? a4[r] : -INFINITY;
                     m_tile = fmaxf(m_tile, a4[r]);
                 }
                 sc[nn] = a4;
@@ -992,35 +1018,62 @@ __global__ __launch_bounds__(256) void latent_tile_kernel(const float *qbuf, con
 // proj: q | k | v at columns 0 | H*M*dim | (H+G)*M*dim; M maps per head lie side by side ([map 1 | map 2] with M = 2).  Every (head, map) of q and
 // k: x / sqrt(mean x^2 + eps) * w over dim (qw / kw [dim], shared by all heads and maps; head_norm 0: none), then the rotation of the first
 // rot_dims dimensions by pos * inv_freq[i]: pairs (i, i + rot_dims/2) with rot_half, (2i, 2i+1) without.
+// conv (taps > 0): q, k and v first pass a causal depthwise convolution without an activation, conv.w [columns, taps] over the mixer's columns of proj and, before the
+// chunk's first row, the sequence's last taps - 1 projected rows (conv.state [slots, taps-1, columns], oldest first, zeros at its start).  conv.move: every chunk is
+// one token; the lane that reads a column's inputs moves them on (longer chunks: conv_state_kernel, behind this kernel).
 // q goes to qbuf as H*M heads ordered [K/V head][map][head in group], k to kpool as G*M K/V heads [K/V head][map]: query head e of that order reads
 // K/V head e / (H/G), and K/V head g reads value head g / M.
+struct ShortConv {
+    const float *w = nullptr;
+    float *state = nullptr;
+    int taps = 0, columns = 0, move = 0;
+};
 template <typename D>
 __global__ __launch_bounds__(64) void attn_prep_head_kernel(const float *proj, int ldp, const int32_t *row_seq, const int32_t *row_pos, const int32_t *seq_slot,
                                                             const int32_t *block_table, int max_pages, int page_size, const float *inv_freq, int rot_dims,
                                                             int rot_half, int head_norm, const float *qw, const float *kw, float eps, int H, int G, int M, int dim,
                                                             int vdim, float *qbuf, typename D::storage *kpool, typename D::storage *vpool, const float *bias,
-                                                            float temp_coef, float temp_every) {
+                                                            float temp_coef, float temp_every, const int32_t *seq_row0, ShortConv conv) {
     const int t = blockIdx.x, hh = blockIdx.y, lane = threadIdx.x;
-    const int pos = row_pos[t], slot = seq_slot[row_seq[t]];
+    const int seq = row_seq[t], pos = row_pos[t], slot = seq_slot[seq];
     const int page = block_table[(size_t)slot * max_pages + pos / page_size], in_page = pos % page_size;
     const int HM = H * M, GM = G * M;
+    const int before = conv.taps > 0 ? t - seq_row0[seq] : 0;  // rows of the chunk ahead of this one
+    float *const past = conv.taps > 1 ? conv.state + (size_t)slot * (conv.taps - 1) * conv.columns : nullptr;
+    // column `col` of the row: the projection, its bias (NULL: none), or the convolution over it
+    auto input = [&](int col) __attribute__((always_inline)) {
+        float v = proj[(size_t)t * ldp + col];
+        if (conv.taps <= 0) return v + (bias ? bias[col] : 0.f);
+        const float *w = conv.w + (size_t)col * conv.taps;
+        float acc = w[conv.taps - 1] * v;
+        for (int back = 1; back < conv.taps; ++back) {
+            const float u = back <= before ? proj[(size_t)(t - back) * ldp + col] : past[(size_t)(conv.taps - 1 + before - back) * conv.columns + col];
+            acc += w[conv.taps - 1 - back] * u;
+        }
+        return acc;
+    };
+    auto move_on = [&](int col) __attribute__((always_inline)) {
+        if (!conv.move || conv.taps <= 1) return;
+        for (int j = 0; j + 2 < conv.taps; ++j) past[(size_t)j * conv.columns + col] = past[(size_t)(j + 1) * conv.columns + col];
+        past[(size_t)(conv.taps - 2) * conv.columns + col] = proj[(size_t)t * ldp + col];
+    };
     if (hh >= HM + GM) {  // a value head: copy
-        const int g = hh - HM - GM;
-        const size_t col = (size_t)(HM + GM) * dim + (size_t)g * vdim;
-        const float *src = proj + (size_t)t * ldp + col;
+        const int g = hh - HM - GM, col = (HM + GM) * dim + g * vdim;
         typename D::storage *dst = vpool + (((size_t)page * G + g) * page_size + in_page) * vdim;
-        for (int c = lane; c < vdim; c += 64) dst[c] = D::from_float(src[c] + (bias ? bias[col + c] : 0.f));
+        for (int c = lane; c < vdim; c += 64) {
+            dst[c] = D::from_float(input(col + c));
+            move_on(col + c);
+        }
         return;
     }
     const bool is_q = hh < HM;
-    const float *src = proj + (size_t)t * ldp + (size_t)hh * dim;
-    const float *bs = bias ? bias + (size_t)hh * dim : nullptr;  // bias (NULL: none): the projection's, over the columns of proj, added here
+    const int col0 = hh * dim;
     const float *w = head_norm ? (is_q ? qw : kw) : nullptr;
     float inv = 1.f;
     if (head_norm) {
         float ss = 0.f;
         for (int c = lane; c < dim; c += 64) {
-            const float v = src[c] + (bs ? bs[c] : 0.f);
+            const float v = input(col0 + c);
             ss += v * v;
         }
         ss = wave_sum(ss);
@@ -1039,14 +1092,16 @@ __global__ __launch_bounds__(64) void attn_prep_head_kernel(const float *proj, i
         int c0, c1 = -1;
         if (u < half) c0 = rot_half ? u : 2 * u, c1 = rot_half ? u + half : 2 * u + 1;
         else c0 = u + half;
-        float a = (src[c0] + (bs ? bs[c0] : 0.f)) * inv * (w ? w[c0] : 1.f), b2 = 0.f;
+        float a = input(col0 + c0) * inv * (w ? w[c0] : 1.f), b2 = 0.f;
         if (c1 >= 0) {
-            b2 = (src[c1] + (bs ? bs[c1] : 0.f)) * inv * (w ? w[c1] : 1.f);
+            b2 = input(col0 + c1) * inv * (w ? w[c1] : 1.f);
             float sn, cs;
             sincosf((float)pos * inv_freq[u], &sn, &cs);
             const float na = a * cs - b2 * sn, nb = b2 * cs + a * sn;
             a = na, b2 = nb;
         }
+        move_on(col0 + c0);
+        if (c1 >= 0) move_on(col0 + c1);
         if (is_q) {
             qdst[c0] = a * temp;
             if (c1 >= 0) qdst[c1] = b2 * temp;
@@ -1611,22 +1666,25 @@ __global__ void postnorm_add_kernel(float *x, const float *y, const float *w, fl
         h[(size_t)r * width + c] = D::from_float(v);
     }
 }
-// ---- the block with norms on both sides: x += mult * ls * (y / sqrt(mean y^2 + eps) * (offset + w))  (ls NULL: 1), and what reads the new
+// ---- the block with norms on both sides: y += ybias (NULL: none), x += mult * ls * (y / sqrt(mean y^2 + eps) * (offset + w))  (ls NULL: 1), and what reads the new
 // stream next leaves with it: next 1: h = x as D rows;  next 2: h = x / sqrt(mean x^2 + eps) * (noffset + nw) as D rows;  0: nothing ----
 template <typename D>
 __global__ void sandwich_add_kernel(float *x, const float *y, const float *w, float offset, float eps, float mult, const float *ls, int next,
-                                    const float *nw, float noffset, typename D::storage *h, int width) {
+                                    const float *nw, float noffset, typename D::storage *h, int width, const float *ybias) {
     __shared__ float red[16];
     const int r = blockIdx.x;
     const float *src = y + (size_t)r * width;
     float *xr = x + (size_t)r * width;
     float ss = 0.f;
-    for (int c = threadIdx.x; c < width; c += blockDim.x) ss += src[c] * src[c];
+    for (int c = threadIdx.x; c < width; c += blockDim.x) {
+        const float v = src[c] + (ybias ? ybias[c] : 0.f);
+        ss += v * v;
+    }
     ss = block_sum(ss, red);
     const float inv = 1.f / sqrtf(ss / (float)width + eps);
     float s2 = 0.f;
     for (int c = threadIdx.x; c < width; c += blockDim.x) {
-        const float v = xr[c] + mult * (ls ? ls[c] : 1.f) * (src[c] * inv * (offset + w[c]));
+        const float v = xr[c] + mult * (ls ? ls[c] : 1.f) * ((src[c] + (ybias ? ybias[c] : 0.f)) * inv * (offset + w[c]));
         xr[c] = v;
         s2 += v * v;
         if (next == 1) h[(size_t)r * width + c] = D::from_float(v);
@@ -1635,6 +1693,33 @@ __global__ void sandwich_add_kernel(float *x, const float *y, const float *w, fl
     s2 = block_sum(s2, red);
     const float inv2 = 1.f / sqrtf(s2 / (float)width + eps);
     for (int c = threadIdx.x; c < width; c += blockDim.x) h[(size_t)r * width + c] = D::from_float(xr[c] * inv2 * (noffset + nw[c]));  // (this thread's own writes)
+}
+// the same block with Dynamic Tanh norms, where the product that forms the branch's result y [rows, width] did not carry the tail itself; VEC columns a thread
+template <typename D, int VEC>
+__global__ void branch_tail_kernel(const float *y, BranchTail t, int width, size_t n) {
+    const size_t i = ((size_t)blockIdx.x * blockDim.x + threadIdx.x) * VEC;
+    if (i >= n) return;
+    const int c = (int)(i % width);
+    if constexpr (VEC == 4) {  // (width a multiple of 4: the columns lie in one row)
+        typedef const f32x4 *V;
+        f32x4 v = *(V)(y + i);
+        if (t.bias) v += *(V)(t.bias + c);
+        const f32x4 pw = *(V)(t.pw + c), pb = *(V)(t.pb + c);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[e] = t.mult * (tanhf(t.palpha * v[e]) * pw[e] + pb[e]);
+        if (t.ls) v *= *(V)(t.ls + c);
+        v += *(V)(t.x + i);
+        if (t.add) v += *(V)(t.add + i);
+        if (t.vec) v += *(V)(t.vec + c);
+        *(f32x4 *)(t.x + i) = v;
+        if (t.h) {
+            const f32x4 nw = *(V)(t.nw + c), nb = *(V)(t.nb + c);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) v[e] = tanhf(t.nalpha * v[e]) * nw[e] + nb[e];
+            if constexpr (sizeof(typename D::storage) == 2) *(u32x2 *)((uint16_t *)t.h + i) = u32x2{BF16::pack2(v[0], v[1]), BF16::pack2(v[2], v[3])};
+            else *(f32x4 *)((float *)t.h + i) = v;
+        }
+    } else branch_tail<D>(t, i, c, y[i]);
 }
 // per-layer token input, middle step: cat[t, c] = gelu_tanh(proj[t, c]) * table[token[t], col0 + c], c < n
 template <typename D>
@@ -1661,13 +1746,13 @@ __global__ void logit_scale_kernel(float *x, float a, float cap, size_t n) {
     x[i] = cap > 0.f ? cap * tanhf(v / cap) : v;
 }
 
-// ---- feed-forward activation: cat[t, col0 + c] = act(proj[t, up0 + c]) ---------------------------------------------------
+// ---- feed-forward activation: cat[t, col0 + c] = act(proj[t, up0 + c] + bias[c])  (bias NULL: none) ---------------------------------------------------
 template <typename D>
-__global__ void ff_act_kernel(const float *proj, int ldp, int up0, int ff, int kind, typename D::storage *out, int ldo, int col0, int rows) {
+__global__ void ff_act_kernel(const float *proj, int ldp, int up0, int ff, int kind, typename D::storage *out, int ldo, int col0, int rows, const float *bias) {
     const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
     if (i >= (size_t)rows * ff) return;
     const int t = (int)(i / ff), c = (int)(i % ff);
-    out[(size_t)t * ldo + col0 + c] = D::from_float(act_f(proj[(size_t)t * ldp + up0 + c], kind));
+    out[(size_t)t * ldo + col0 + c] = D::from_float(act_f(proj[(size_t)t * ldp + up0 + c] + (bias ? bias[c] : 0.f), kind));
 }
 
 // ---- short causal depthwise convolution + SiLU over the first C columns of proj -------------------------------------------
@@ -1898,19 +1983,23 @@ __global__ void rms_cols_kernel(const float *in, int ldi, int n, const float *w,
 // absorption), the rotated part -> qbuf[t, h, rank ..] after its rotation.  With own_kv (the layer has its own latent projection, columns
 // kv0 .. of proj: rank latent columns, then rot columns of one rotated key part shared by all heads): the latent is RMS-normed with
 // its weight and appended to the sequence's page row [c (rank) | rotated key part (rot)] -- the whole K/V cache of the layer.
-// Rotation: pair (2i, 2i+1) by pos * freq[i], cos and sin times mult.  grid (rows, H + 1), one wave each.
+// Rotation of the first rot_dims of the rot dimensions by pos * freq[i], cos and sin times mult: pairs (i, i + rot_dims/2) with rot_half, (2i, 2i+1) without.
+// grid (rows, H + 1), one wave each.
 template <typename D>
 __global__ __launch_bounds__(64) void latent_prep_kernel(const float *q, int ldq, int H, int dim, int rot, int rank, const float *proj, int ldp, int kv0,
                                                          const float *c_norm, float eps, int own_kv, const int32_t *row_seq, const int32_t *row_pos,
                                                          const int32_t *seq_slot, const int32_t *block_table, int max_pages, int page_size,
-                                                         const float *freq, int rot_dims, float mult, typename D::storage *qn, float *qbuf,
+                                                         const float *freq, int rot_dims, int rot_half, float mult, typename D::storage *qn, float *qbuf,
                                                          typename D::storage *pool) {
     const int t = blockIdx.x, hh = blockIdx.y, lane = threadIdx.x;
     const int pos = row_pos[t];
-    auto turn = [&](const float *src, int p, float &u, float &v) {
-        const int c = 2 * p;
-        u = src[c], v = (c + 1 < rot) ? src[c + 1] : 0.f;
-        if (c + 1 < rot_dims) {
+    const int half = rot_dims / 2, units = rot_half ? rot - half : (rot + 1) / 2;
+    // unit p of a rotated part: rotation pair p below `half`, then (half-split: single, neighbours: paired) dimensions that pass; c0, c1 (-1: none): its places
+    auto turn = [&](const float *src, int p, int &c0, int &c1, float &u, float &v) {
+        if (rot_half) c0 = p < half ? p : p + half, c1 = p < half ? p + half : -1;
+        else c0 = 2 * p, c1 = 2 * p + 1 < rot ? 2 * p + 1 : -1;
+        u = src[c0], v = c1 >= 0 ? src[c1] : 0.f;
+        if (p < half) {
             float sn, cs;
             sincosf((float)pos * freq[p], &sn, &cs);
             sn *= mult, cs *= mult;
@@ -1922,11 +2011,12 @@ __global__ __launch_bounds__(64) void latent_prep_kernel(const float *q, int ldq
         const float *src = q + (size_t)t * ldq + (size_t)hh * (dim + rot);
         for (int c = lane; c < dim; c += 64) qn[((size_t)t * H + hh) * dim + c] = D::from_float(src[c]);
         float *dst = qbuf + ((size_t)t * H + hh) * (rank + rot) + rank;
-        for (int p = lane; 2 * p < rot; p += 64) {
+        for (int p = lane; p < units; p += 64) {
+            int c0, c1;
             float u, v;
-            turn(src + dim, p, u, v);
-            dst[2 * p] = u;
-            if (2 * p + 1 < rot) dst[2 * p + 1] = v;
+            turn(src + dim, p, c0, c1, u, v);
+            dst[c0] = u;
+            if (c1 >= 0) dst[c1] = v;
         }
         return;
     }
@@ -1940,11 +2030,12 @@ __global__ __launch_bounds__(64) void latent_prep_kernel(const float *q, int ldq
     ss = wave_sum(ss);
     const float inv = 1.f / sqrtf(ss / (float)rank + eps);
     for (int c = lane; c < rank; c += 64) dst[c] = D::from_float(src[c] * inv * c_norm[c]);
-    for (int p = lane; 2 * p < rot; p += 64) {
+    for (int p = lane; p < units; p += 64) {
+        int c0, c1;
         float u, v;
-        turn(src + rank, p, u, v);
-        dst[rank + 2 * p] = D::from_float(u);
-        if (2 * p + 1 < rot) dst[rank + 2 * p + 1] = D::from_float(v);
+        turn(src + rank, p, c0, c1, u, v);
+        dst[rank + c0] = D::from_float(u);
+        if (c1 >= 0) dst[rank + c1] = D::from_float(v);
     }
 }
 
@@ -1960,13 +2051,15 @@ __global__ void gate_mul_kernel(const float *in, int ldi, const float *g, int ld
     out[(size_t)t * ldo + c] = D::from_float(in[(size_t)t * ldi + c] * scale * (kind == 2 ? 1.f : (kind == 0 ? sigmoid_f(z) : silu_f(z))));
 }
 
-// ---- gated feed-forward activation: cat[t, col0 + c] = act(proj[t, g0 + c]) * proj[t, u0 + c] ------------------------------------
+// ---- gated feed-forward activation: cat[t, col0 + c] = act(proj[t, g0 + c] + bias[c]) * (proj[t, u0 + c] + bias[ff + c])  (bias NULL: none) ------------------------------------
 template <typename D>
-__global__ void ff_gated_act_kernel(const float *proj, int ldp, int g0, int u0, int ff, int kind, typename D::storage *out, int ldo, int col0, int rows) {
+__global__ void ff_gated_act_kernel(const float *proj, int ldp, int g0, int u0, int ff, int kind, typename D::storage *out, int ldo, int col0, int rows,
+                                    const float *bias) {
     const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
     if (i >= (size_t)rows * ff) return;
     const int t = (int)(i / ff), c = (int)(i % ff);
-    out[(size_t)t * ldo + col0 + c] = D::from_float(act_f(proj[(size_t)t * ldp + g0 + c], kind) * proj[(size_t)t * ldp + u0 + c]);
+    const float g = proj[(size_t)t * ldp + g0 + c] + (bias ? bias[c] : 0.f), u = proj[(size_t)t * ldp + u0 + c] + (bias ? bias[ff + c] : 0.f);
+    out[(size_t)t * ldo + col0 + c] = D::from_float(act_f(g, kind) * u);
 }
 
 // ---- linear recurrences with a decaying matrix state --------------------------------------------------------------------------------
@@ -2226,8 +2319,14 @@ __global__ void linrec_out_joint_kernel(const float *obuf, const float *w, float
 // the router of one row, by every thread of a 256-thread workgroup: scores s = softmax(z) or sigmoid(z) (router 0 / 1); choice = s + correction
 // (NULL: 0); groups, kept groups, the `top` largest choices (ties: the lower index).  Leaves sw[e] = s_e for the experts taken, 0 for the others.
 // bias (NULL: none) is added to the logits.  router 2: s = z, and the weights are the softmax over the chosen experts' logits only.
+// opt: a group scores the sum of its two largest choices (group_top2) instead of its largest; the weights of the experts taken are divided by their sum + 1e-20
+// (renorm) and multiplied by `scale`.
+struct RouteOpts {
+    int group_top2 = 0, renorm = 0;
+    float scale = 1.f;
+};
 __device__ __forceinline__ void moe_route_row(const float *row, int r0, int ET, int top, int groups, int keep, const float *correction, const float *bias, int router,
-                                              float *sw, float *sc, float *gm) {
+                                              const RouteOpts &opt, float *sw, float *sc, float *gm) {
     const int tid = threadIdx.x;
     if (tid < 64) {  // one wave scores (ET <= 256: four experts a lane at most)
         float z[4], mx = -INFINITY;
@@ -2265,9 +2364,12 @@ __device__ __forceinline__ void moe_route_row(const float *row, int r0, int ET, 
     if (tid == 0 && groups > 1) {  // groups, then the top choices: a few dozen comparisons
         const int per = ET / groups;
         for (int g = 0; g < groups; ++g) {
-            float m = -INFINITY;
-            for (int e = g * per; e < (g + 1) * per; ++e) m = fmaxf(m, sc[e]);
-            gm[g] = m;
+            float m = -INFINITY, second = -INFINITY;
+            for (int e = g * per; e < (g + 1) * per; ++e) {
+                second = fmaxf(second, fminf(m, sc[e]));
+                m = fmaxf(m, sc[e]);
+            }
+            gm[g] = opt.group_top2 && per > 1 ? m + second : m;
         }
         for (int g = 0; g < groups; ++g) {  // rank of the group: how many beat it (ties: the lower index first)
             int rank = 0;
@@ -2297,20 +2399,27 @@ __device__ __forceinline__ void moe_route_row(const float *row, int r0, int ET, 
             wgt = expf(wgt - mx) / sum;
         }
     }
-    if (tid < ET) sw[tid] = wgt;
+    if (opt.renorm) {
+        if (tid < ET) sc[tid] = wgt;
+        __syncthreads();
+        float sum = 1e-20f;
+        for (int o = 0; o < ET; ++o) sum += sc[o];
+        wgt /= sum;
+    }
+    if (tid < ET) sw[tid] = wgt * opt.scale;
     __syncthreads();
 }
 
 template <typename D>
 __global__ __launch_bounds__(256) void moe_route_act_kernel(const float *proj, int ldp, int r0, int sg0, int su0, int eu0, int experts, int identity, int top,
                                                             int groups, int keep, int ffe, int ffs, const float *correction, const float *bias,
-                                                            typename D::storage *out, int ldo, int col0, float *idw, int router) {
+                                                            typename D::storage *out, int ldo, int col0, float *idw, int router, RouteOpts opt) {
     __shared__ float sw[256], sc[256];
     __shared__ float gm[256];
     // blockIdx.y: a share of the row's columns (every share routes the row again: a few dozen comparisons against thousands of columns)
     const int t = blockIdx.x, tid = threadIdx.x, ET = experts + identity;
     const float *row = proj + (size_t)t * ldp;
-    moe_route_row(row, r0, ET, top, groups, keep, correction, bias, router, sw, sc, gm);
+    moe_route_row(row, r0, ET, top, groups, keep, correction, bias, router, opt, sw, sc, gm);
     if (tid == 0 && blockIdx.y == 0) {
         float a = 0.f;
         for (int e = experts; e < ET; ++e) a += sw[e];
@@ -2327,14 +2436,14 @@ __global__ __launch_bounds__(256) void moe_route_act_kernel(const float *proj, i
 // which experts the rows of a small step take: bit e of *mask is set when some row's router takes expert e (the products around the activation then leave the
 // others out, see SegSkip).  One workgroup; experts <= 64.
 __global__ __launch_bounds__(256) void moe_taken_mask_kernel(const float *proj, int ldp, int r0, int rows, int experts, int identity, int top, int groups, int keep,
-                                                             const float *correction, const float *bias, int router, unsigned long long *mask) {
+                                                             const float *correction, const float *bias, int router, RouteOpts opt, unsigned long long *mask) {
     __shared__ float sw[256], sc[256];
     __shared__ float gm[256];
     __shared__ unsigned long long taken;
     if (threadIdx.x == 0) taken = 0ull;
     __syncthreads();
     for (int t = 0; t < rows; ++t) {
-        moe_route_row(proj + (size_t)t * ldp, r0, experts + identity, top, groups, keep, correction, bias, router, sw, sc, gm);
+        moe_route_row(proj + (size_t)t * ldp, r0, experts + identity, top, groups, keep, correction, bias, router, opt, sw, sc, gm);
         if ((int)threadIdx.x < experts && sw[threadIdx.x] != 0.f) atomicOr(&taken, 1ull << threadIdx.x);
         __syncthreads();
     }
@@ -2347,12 +2456,12 @@ __global__ __launch_bounds__(256) void moe_taken_mask_kernel(const float *proj, 
 template <typename D>
 __global__ __launch_bounds__(256) void moe_gated_act_kernel(const float *proj, int ldp, int r0, int sg0, int g0, int u0, int experts, int identity, int top,
                                                             int groups, int keep, int ffe, int ffs, const float *correction, const float *bias,
-                                                            typename D::storage *out, int ldo, int col0, float *idw, int router, int scale_input, int act) {
+                                                            typename D::storage *out, int ldo, int col0, float *idw, int router, RouteOpts opt, int scale_input, int act) {
     __shared__ float sw[256], sc[256];
     __shared__ float gm[256];
     const int t = blockIdx.x, tid = threadIdx.x, ET = experts + identity;
     const float *row = proj + (size_t)t * ldp;
-    moe_route_row(row, r0, ET, top, groups, keep, correction, bias, router, sw, sc, gm);
+    moe_route_row(row, r0, ET, top, groups, keep, correction, bias, router, opt, sw, sc, gm);
     if (tid == 0 && blockIdx.y == 0) {
         float a = 0.f;
         for (int e = experts; e < ET; ++e) a += sw[e];
@@ -2385,6 +2494,11 @@ __global__ void identity_axpy_kernel(float *x, const typename D::storage *h, con
 __global__ void add_rowvec_kernel(float *x, const float *v, int width, int rows) {
     const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
     if (i < (size_t)rows * width) x[i] += v[i % width];
+}
+// entry of a loop pass: x += x0 (the embedding output; NULL: not added) + v[width]
+__global__ void pass_entry_kernel(float *x, const float *x0, const float *v, int width, int rows) {
+    const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
+    if (i < (size_t)rows * width) x[i] = (x0 ? x[i] + x0[i] : x[i]) + v[i % width];
 }
 __global__ void fill_kernel(float *p, size_t n, float v) {
     for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (size_t)gridDim.x * blockDim.x) p[i] = v;

@@ -56,7 +56,9 @@ class TlHybridLayer(ctypes.Structure):
                 ("side_gate_dev", _vp), ("side_proj_dev", _vp), ("side_norm_dev", _vp), ("side_col0", _i),
                 ("softcap", _f), ("bias_slope_dev", _vp), ("q_temp_coef", _f), ("q_temp_every", _f),
                 ("rec_silu", _i), ("rec_plain_k", _i), ("rec_joint_norm", _i), ("rec_sigmoid_gate", _i), ("router_bias_dev", _vp),
-                ("beside", _vp), ("mix_scale", _f)]
+                ("beside", _vp), ("mix_scale", _f),
+                ("keep_first", _i), ("moe_group_top2", _i), ("moe_renorm", _i), ("moe_scale", _f), ("ff_in_bias_dev", _vp), ("ff_out_bias_dev", _vp),
+                ("post_norm_bias_dev", _vp), ("post_norm2_bias_dev", _vp), ("post_norm_alpha", _f), ("post_norm2_alpha", _f)]
 
 
 class TlHybridConfig(ctypes.Structure):
@@ -68,7 +70,7 @@ class TlHybridConfig(ctypes.Structure):
                 ("page_size", _i), ("num_pages", _i), ("max_slots", _i), ("max_pages_per_seq", _i), ("max_rows", _i),
                 ("logit_scale", _f), ("embed_norm_dev", _vp), ("side_embed_dev", _vp), ("side_cols", _i), ("side_dim", _i),
                 ("pair_embed_dev", _vp), ("pair_buckets", ctypes.c_int64), ("pair_mul_prev", ctypes.c_int64), ("pair_mul_cur", ctypes.c_int64),
-                ("logit_softcap", _f)]
+                ("logit_softcap", _f), ("loop_add_embed", _i)]
 
 
 class TlHybridStats(ctypes.Structure):

@@ -52,7 +52,8 @@ class HybridEngine:
         self.page_size, self.max_batch, self.vocab_size = int(page_size), int(max_batch), cfg.vocab
         self.max_prefill_rows = max(int(max_prefill_rows), self.max_batch)
         self.num_hidden_layers = len(cfg.layers)
-        self.has_recurrent_state = cfg.pair_embed is not None or any(M.kind in ("delta", "linrec") for L in cfg.layers for M in (L, L.beside) if M is not None)
+        self.has_recurrent_state = cfg.pair_embed is not None or any(M.kind in ("delta", "linrec") or M.conv_taps > 1
+                                                                             for L in cfg.layers for M in (L, L.beside) if M is not None)
         for i, L in enumerate(cfg.layers):  # a size the configuration leaves to the tensors
             if L.a_rank < 0:
                 L.a_rank = int(model.tensors[cfg.prefix(i) + "mix.a1"].shape[0])
@@ -77,7 +78,11 @@ class HybridEngine:
             s.expert_ff, s.shared_ff, s.correction_dev, s.router_bias_dev = L.expert_ff, L.shared_ff, ptr("correction"), ptr("router_bias")
             s.moe_router, s.moe_gated, s.moe_scale_input = _ROUTER[L.router], int(L.moe_gated), int(L.moe_scale_input)
             s.moe_shared_sg = int(L.moe_gated and L.moe_shared_sg)
+            s.moe_group_top2, s.moe_renorm, s.moe_scale = int(L.moe_group_score == "top2"), int(L.moe_renorm), L.moe_scale
+            s.ff_in_bias_dev, s.ff_out_bias_dev = ptr("ff_in_bias"), ptr("ff_out_bias")
             s.post_norm_dev, s.post_norm2_dev = ptr("post_norm"), ptr("post_norm2")
+            s.post_norm_bias_dev, s.post_norm2_bias_dev = ptr("post_norm_bias"), ptr("post_norm2_bias")
+            s.post_norm_alpha, s.post_norm2_alpha = t.get("post_norm_alpha", 0.0), t.get("post_norm2_alpha", 0.0)
             s.side_gate_dev, s.side_proj_dev, s.side_norm_dev, s.side_col0 = ptr("side_gate"), ptr("side_proj"), ptr("side_norm"), i * cfg.side_dim
         c = ext.TlHybridConfig()
         c.dtype = ext.HY_BF16 if dtype == torch.bfloat16 else ext.HY_F32
@@ -88,6 +93,7 @@ class HybridEngine:
         if cfg.loop:
             c.loop_start, c.loop_stop, c.loop_times = cfg.loop
             c.loop_in_dev, c.loop_step_dev = (w["loop_in"].data_ptr() if "loop_in" in w else None), w["loop_step"].data_ptr()
+            c.loop_add_embed = int(cfg.loop_add_embed)
         c.embed_dev, c.final_norm_dev, c.final_norm_offset, c.head_dev = w["embed"].data_ptr(), w["final_norm"].data_ptr(), cfg.norm_offset, w["head"].data_ptr()
         c.embed_norm_dev = w["embed_norm"].data_ptr() if "embed_norm" in w else None
         c.logit_softcap = cfg.logit_softcap
@@ -127,6 +133,7 @@ class HybridEngine:
             if L.diff is not None:
                 s.diff_maps, s.diff_lambda, s.diff_init = 1, t["diff_lambda"], L.diff
             s.softcap, s.bias_slope_dev = L.softcap, ptr("bias_slope")
+            s.keep_first, s.conv_taps, s.conv_dev = L.keep_first, L.conv_taps, ptr("conv")
             if L.q_temp:
                 s.q_temp_coef, s.q_temp_every = L.q_temp
         elif L.kind == "linrec":
@@ -137,6 +144,7 @@ class HybridEngine:
         elif L.kind == "latent":
             s.q_rank, s.kv_rank, s.rot_dim, s.kv_from = L.q_rank, L.kv_rank, L.rot_dim, L.kv_from
             s.dq_norm_dev, s.dkv_norm_dev, s.uq_dev, s.uk_t_dev, s.uv_dev = ptr("dq_norm"), ptr("dkv_norm"), ptr("uq"), ptr("uk_t"), ptr("uv")
+            s.rot_half = int(L.rot_half)
 
     @classmethod
     def from_model(cls, model: Any, **kwargs) -> "HybridEngine":

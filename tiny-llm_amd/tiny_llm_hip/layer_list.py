@@ -83,6 +83,19 @@ sequential pre-norm blocks, norms with weights around zero, per-channel layer sc
     ff "dense": W_down relu(W_up h)^2.
     ff "moe": z = W_router h + b; the `top` largest z are taken, weights = softmax over those; expert = W_down (silu(W_gate h) * W_up h);
         plus a shared expert of the same form.
+
+Vabuzen -- x = embed[token]; Dynamic Tanh norms (as Zefapel's) on both sides of every sublayer, one residual factor m for the model:
+
+    x <- x + m * norm1b(mixer(norm1 x));   x <- x + m * norm2b(ff(norm2 x));   logits = cap tanh(head norm(x) / cap)
+
+    mixer "attention": q, k and v each pass a causal depthwise convolution of `conv` taps (no activation); the first rot.dims dimensions of q and k turn as
+        pairs (2i, 2i+1); query i sees key j <= i where i - j < mask.size or j < mask.keep_first; weights exp(s_j) / (1 + sum_j exp(s_j)); W_o.
+    mixer "latent_attention": q = W_q h directly ([plain | rotated] per head), latent as Zefapel's, rotation of pairs (i, i + rot_dim/2) with plain
+        frequencies; causal softmax; no gate.
+    ff "dense": W_down gelu_tanh(W_up h + b_up) + b_down.
+    ff "moe": s = sigmoid(W_router h); groups.count equal runs of neighbouring experts, a run scores the sum of its two largest s, the `top` largest s inside the
+        groups.keep best runs are taken; weights s / (sum of those + 1e-20) * router.scale; expert = W_down (silu(W_gate h) * W_up h); plus a shared expert.
+    loop {start, stop, times}: each pass but the first is entered by x <- x + x0 (x0 = the embedding output), every pass by x <- x + step[t].
 """
 
 from __future__ import annotations
@@ -92,7 +105,8 @@ from typing import Any, Callable
 
 import torch
 
-__all__ = ["LayerSpec", "LayerListConfig", "FAMILIES", "fonapel_config", "zefapel_config", "lovulix_config", "muduvik_config", "karorax_config", "pack_layer_list"]
+__all__ = ["LayerSpec", "LayerListConfig", "FAMILIES", "fonapel_config", "zefapel_config", "lovulix_config", "muduvik_config", "karorax_config",
+           "vabuzen_config", "pack_layer_list"]
 
 
 @dataclass
@@ -111,7 +125,7 @@ class LayerSpec:
     qk_unit_rms: bool = False
     sink: bool = False
     gated: bool = False
-    # delta
+    # delta; attention: > 0: q, k and v pass a short causal convolution without an activation (tensors mix.q.conv / mix.k.conv / mix.v.conv)
     conv_taps: int = 0
     unit_eps: float = 1e-6
     # feed-forward: "plain" W_down act(W_up h) | "gated" W_down (act(W_gate h) * W_up h) | "moe"
@@ -168,6 +182,13 @@ class LayerSpec:
     q_temp: tuple[float, float] | None = None  # (coef, every): q *= 1 + coef ln(floor((p + 1) / every) + 1)
     # mixture of experts, further options (2)
     moe_bias: bool = False          # the router's logits carry a bias (tensor mlp.router.b)
+    # attention, further options (4)
+    keep_first: int = 0             # with a window: keys j < keep_first stay visible
+    # feed-forward, further options
+    ff_bias: bool = False           # a dense feed-forward's projections carry biases (tensors mlp.up.b / mlp.down.b, mlp.gate.b)
+    moe_group_score: str = "max"    # "max": a group's largest choice | "top2": the sum of its two largest
+    moe_renorm: bool = False        # the weights of the experts taken are divided by their sum (+ 1e-20)
+    moe_scale: float = 1.0          # factor on the weights, behind that
     # two mixers side by side on one input
     beside: LayerSpec | None = None # the second mixer (its sizes and options only; the feed-forward is the layer's)
     mix_scale: float = 1.0          # factor on this mixer's result
@@ -187,11 +208,13 @@ class LayerListConfig:
     norm_kind: str = "rms"          # "rms" | "dyt" (tanh(alpha x) w + b: tensors <name>, <name>.alpha, <name>.b)
     block: str = "parallel"         # "parallel": x += m (mixer(h) + ff(h)), one norm | "sequential": two norms, two residual sums
                                     # | "postnorm": x += m norm1(mixer(x)); x += m norm2(ff(x))
-    layer_scale: bool = False       # sequential block: per-channel vectors ls1 / ls2 on the branches
+                                    # | "sandwich": x += m norm1b(mixer(norm1 x)); x += m norm2b(ff(norm2 x))
+    layer_scale: bool = False       # sequential and sandwich block: per-channel vectors ls1 / ls2 on the branches
     embed_scale: float = 1.0
     logit_scale: float = 1.0
     embed_norm: bool = False        # the embedding output passes the model's norm (tensor embed.norm)
     loop_projection: bool = True    # a loop pass is entered through loop.in [width, 2 width]; False: only loop.step is added
+    loop_add_embed: bool = False    # (without a projection) each pass but the first adds the embedding output
     side_dim: int = 0               # > 0: per-layer token input of this many columns a layer (tensors side.embed, <layer>.side.*)
     pair_embed: tuple[int, int, int] | None = None  # (buckets, factor of the previous token, factor of the token): a second embedding table
                                     # [buckets + 1, width] indexed by a hash of both is added (tensor bigram; the last row for a first token)
@@ -539,6 +562,83 @@ def _karorax_tensor_shapes(cfg: LayerListConfig) -> dict[str, tuple[int, ...]]:
     return want
 
 
+def vabuzen_config(config: dict) -> LayerListConfig:
+    """config.json of a Vabuzen checkpoint -> LayerListConfig.  Every size and every constant the file gives is read from it."""
+    for key in ("layers", "norm", "residual_mult", "vocab", "width"):
+        if key not in config:
+            raise ValueError(f"config.json lacks {key!r}")
+    layers = []
+    for i, entry in enumerate(config["layers"]):
+        kind, mc, mlp = entry.get("type"), entry.get("mixer") or {}, entry.get("mlp")
+        ff: dict[str, Any] = {}
+        if mlp is not None:
+            if mlp.get("kind") == "dense":
+                ff = dict(ff=int(mlp["ff"]), ff_kind="plain", ff_act="gelu_tanh", ff_bias=True)
+            elif mlp.get("kind") == "moe":
+                r, shared, groups = mlp["router"], mlp.get("shared"), mlp["router"].get("groups") or {"count": 1, "keep": 1}
+                experts, expert_ff, count, keep = int(r["experts"]), int(mlp["expert"]["ff"]), int(groups["count"]), int(groups["keep"])
+                shared_ff = int(shared["ff"]) if shared else 0
+                if count < 1 or experts % count:
+                    raise ValueError(f"layer {i}: {experts} experts do not form {count} equal groups")
+                if not (1 <= keep <= count and 1 <= int(r["top"]) <= keep * (experts // count)):
+                    raise ValueError(f"layer {i}: top={r['top']} of {keep} groups of {experts // count} experts")
+                ff = dict(ff=shared_ff + experts * expert_ff, ff_kind="moe", ff_act="silu", experts=experts, top=int(r["top"]), groups=count, keep=keep,
+                          expert_ff=expert_ff, shared_ff=shared_ff, router="sigmoid", moe_gated=True, moe_shared_sg=False, moe_correction=False,
+                          moe_group_score="top2", moe_renorm=True, moe_scale=float(r["scale"]))
+            else:
+                raise ValueError(f"layer {i}: unsupported mlp.kind={mlp.get('kind')!r}")
+        rot = mc.get("rot") or {}
+        common = dict(heads=int(mc["heads"]), dim=int(mc["dim"]), vdim=int(mc["vdim"]), rot_dims=int(rot.get("dims", 0)), rot_base=float(rot.get("base", 10000.0)),
+                      scale=float(mc["scale"]))
+        if kind == "attention":
+            mask, kv_heads = mc.get("mask") or {}, int(mc["kv_heads"])
+            if common["heads"] % kv_heads:
+                raise ValueError(f"layer {i}: {common['heads']} heads do not form {kv_heads} equal groups")
+            if int(mc["conv"]) < 1:
+                raise ValueError(f"layer {i}: conv={mc['conv']} (at least one tap)")
+            layers.append(LayerSpec(kind="attention", kv_heads=kv_heads, conv_taps=int(mc["conv"]), window=int(mask.get("size", 0)), keep_first=int(mask.get("keep_first", 0)),
+                                    sink=True, **common, **ff))
+        elif kind == "latent_attention":
+            layers.append(LayerSpec(kind="latent", kv_heads=1, kv_rank=int(mc["kv_rank"]), rot_dim=int(mc["rot_dim"]), rot_half=True, **common, **ff))
+        else:
+            raise ValueError(f"layer {i}: unknown mixer type {kind!r}")
+    loop, lp = None, config.get("loop")
+    if lp:
+        loop = (int(lp["start"]), int(lp["stop"]), int(lp["times"]))
+        if not (0 <= loop[0] < loop[1] <= len(layers)) or loop[2] < 1:
+            raise ValueError(f"loop {lp!r} does not fit {len(layers)} layers")
+    return LayerListConfig(family="Vabuzen", width=int(config["width"]), vocab=int(config["vocab"]), norm_eps=float(config["norm"]["eps"]),
+                           residual_mult=float(config["residual_mult"]), layers=layers, norm_offset=0.0, norm_kind="dyt", loop=loop, block="sandwich",
+                           loop_projection=False, loop_add_embed=True, logit_softcap=float(config.get("logit_softcap") or 0.0))
+
+
+def _vabuzen_tensor_shapes(cfg: LayerListConfig) -> dict[str, tuple[int, ...]]:
+    """Every tensor a Vabuzen checkpoint must hold, with its shape."""
+    W = cfg.width
+    want: dict[str, tuple[int, ...]] = {"embed": (cfg.vocab, W), "head": (cfg.vocab, W), **_norm_shapes(cfg, "final.norm")}
+    if cfg.loop:
+        want["loop.step"] = (cfg.loop[2], W)
+    for i, L in enumerate(cfg.layers):
+        p, m, f = cfg.prefix(i), cfg.prefix(i) + "mix.", cfg.prefix(i) + "mlp."
+        hv = L.heads * L.vdim
+        want.update({**_norm_shapes(cfg, p + "norm1"), **_norm_shapes(cfg, p + "norm1b"), m + "o": (W, hv)})
+        if L.kind == "attention":
+            for name, n in (("q", L.heads * L.dim), ("k", L.kv_heads * L.dim), ("v", L.kv_heads * L.vdim)):
+                want.update({m + name: (n, W), m + name + ".conv": (n, L.conv_taps)})
+        else:
+            want.update({m + "q": (L.heads * (L.dim + L.rot_dim), W), m + "dkv": (L.kv_rank + L.rot_dim, W), m + "dkv.norm": (L.kv_rank,),
+                         m + "uk": (L.heads * L.dim, L.kv_rank), m + "uv": (hv, L.kv_rank)})
+        if L.ff:
+            want.update({**_norm_shapes(cfg, p + "norm2"), **_norm_shapes(cfg, p + "norm2b")})
+            if L.ff_kind == "plain":
+                want.update({f + "up": (L.ff, W), f + "up.b": (L.ff,), f + "down": (W, L.ff), f + "down.b": (W,)})
+            else:
+                want[f + "router"] = (L.experts, W)
+                for name, n in [(f"e{e}.", L.expert_ff) for e in range(L.experts)] + ([("shared.", L.shared_ff)] if L.shared_ff else []):
+                    want.update({f + name + "gate": (n, W), f + name + "up": (n, W), f + name + "down": (W, n)})
+    return want
+
+
 def _norm_shapes(cfg: LayerListConfig, name: str) -> dict[str, tuple[int, ...]]:
     if cfg.norm_kind == "dyt":
         return {name: (cfg.width,), name + ".b": (cfg.width,), name + ".alpha": ()}
@@ -588,6 +688,7 @@ FAMILIES: dict[str, tuple[Callable[[dict], LayerListConfig], Callable[[LayerList
     "Lovulix": (lovulix_config, _lovulix_tensor_shapes),
     "Muduvik": (muduvik_config, _muduvik_tensor_shapes),
     "Karorax": (karorax_config, _karorax_tensor_shapes),
+    "Vabuzen": (vabuzen_config, _vabuzen_tensor_shapes),
 }
 
 
@@ -627,6 +728,8 @@ def _pack_mixer(entry: dict, L: LayerSpec, m: str, mat: Callable, vec: Callable,
             entry["sink"] = vec(m + "sink")
         if L.v_mix == "blend":
             entry["v_mix_lambda"] = float(tensors[m + "vmix"].float())
+        if L.conv_taps:
+            entry["conv"] = torch.cat([vec(m + "q.conv"), vec(m + "k.conv"), vec(m + "v.conv")], 0).contiguous()
         if L.distance_bias:
             entry["bias_slope"] = torch.tensor([2.0 ** (-8.0 * (h + 1) / L.heads) for h in range(L.heads)], dtype=torch.float32, device=device)
     if L.kind == "delta":
@@ -686,6 +789,9 @@ def pack_layer_list(cfg: LayerListConfig, tensors: dict[str, torch.Tensor], dtyp
             rows, out = rows + more_rows, out + more_out
         if L.ff:
             f = p + "mlp."
+            if L.ff_bias:
+                entry["ff_in_bias"] = torch.cat([vec(f + "gate.b"), vec(f + "up.b")] if L.ff_kind == "gated" else [vec(f + "up.b")]).contiguous()
+                entry["ff_out_bias"] = vec(f + "down.b")
             if L.ff_kind == "plain":
                 ff_rows, ff_out = [mat(f + "up")], [mat(f + "down")]
             elif L.ff_kind == "gated":
@@ -720,10 +826,10 @@ def pack_layer_list(cfg: LayerListConfig, tensors: dict[str, torch.Tensor], dtyp
             else:
                 norm(entry, "norm2", p + "norm2")
                 if cfg.block == "sandwich":
-                    entry["post_norm2"] = vec(p + "norm2b")
+                    norm(entry, "post_norm2", p + "norm2b")
                 entry["w_in2"], entry["w_out2"] = torch.cat(ff_rows, 0).contiguous(), torch.cat(ff_out, 1).contiguous()
         if cfg.block == "sandwich":
-            entry["post_norm"] = vec(p + "norm1b")
+            norm(entry, "post_norm", p + "norm1b")
         if cfg.side_dim:
             entry["side_gate"], entry["side_proj"], entry["side_norm"] = mat(p + "side.gate").contiguous(), mat(p + "side.proj").contiguous(), vec(p + "side.norm")
         if cfg.layer_scale:
