@@ -29,6 +29,11 @@ attention over the same 192 + 64-wide cache rows, a second layer on the first on
 W / 2 beside a shared one of W) and, for the capped attention, beside Fonapel's attention layers: 4 layers (parallel + squared-ReLU feed-forward of
 3 W, latent attention with a window of 1,024 + experts, latent attention on that cache + experts, parallel + experts); a parallel layer holds 16 heads of
 attention (a quarter of them K/V heads) AND 16 heads of lightning attention at width 2048.
+
+`--layer-list-family Vabuzen` measures the Vabuzen family beside Muduvik (the closest existing model: the same block with norms on both sides, windowed attention,
+latent attention without gates, dense feed-forwards) and, for its experts and its latent rows, beside Karorax, for its attention beside Fonapel's attention layers:
+4 layers (attention + feed-forward of 3 W, latent attention + experts, latent attention + feed-forward, attention + experts), convolutions of 4 taps, windows of
+1,024 positions and the 4 first tokens, latent rows of 192 + 64, 8 experts of W / 2 in 4 groups (2 kept, 2 experts taken) beside a shared one of W.
 """
 
 from __future__ import annotations
@@ -175,6 +180,53 @@ def karorax_costs(cfg: dict, ctx: int, dtype_bytes: int = 2) -> dict:
     return {"matrix_elems": fixed + sum(pe * top for pe, (top, _) in zip(per_expert, taken)), "head_elems": head, "attn_macs": attn_macs,
             "decode_bytes": lambda b: (fixed + head + sum(pe * min(n, b * top) for pe, (top, n) in zip(per_expert, taken))) * dtype_bytes
             + b * (sum(per * (min(ctx, win) if win else ctx) for per, win in terms) * dtype_bytes + 2 * state * 4)}
+
+
+def vabuzen_config(width: int, vocab: int = 32768, window: int = 1024) -> dict:
+    heads = max(1, width // 128)
+    dense = {"kind": "dense", "ff": 3 * width}
+    moe = {"kind": "moe", "expert": {"ff": width // 2}, "router": {"experts": 8, "groups": {"count": 4, "keep": 2}, "scale": 2.0, "top": 2}, "shared": {"ff": width}}
+    attn = {"conv": 4, "heads": heads, "kv_heads": max(1, heads // 4), "dim": 128, "vdim": 128, "mask": {"keep_first": 4, "size": window},
+            "rot": {"base": 1e6, "dims": 64}, "scale": 128 ** -0.5}
+    lat = {"heads": heads, "dim": 128, "vdim": 128, "rot_dim": 64, "kv_rank": 192, "rot": {"base": 1e6, "dims": 64}, "scale": 192 ** -0.5}
+    layers = [{"type": "attention", "mixer": attn, "mlp": dense}, {"type": "latent_attention", "mixer": lat, "mlp": moe},
+              {"type": "latent_attention", "mixer": lat, "mlp": dense}, {"type": "attention", "mixer": attn, "mlp": moe}]
+    return {"architecture": "Vabuzen", "layers": layers, "logit_softcap": 30.0, "norm": {"eps": 1e-6}, "residual_mult": 0.5, "vocab": vocab, "width": width}
+
+
+def vabuzen_costs(cfg: dict, ctx: int, dtype_bytes: int = 2) -> dict:
+    """What the design needs: matrix elements a token multiplies (the experts it takes), attention multiply-adds per (query, key) pair in the per-head form and the
+    pairs a window and the kept first tokens leave, the bytes a decode step of b sequences streams: every matrix once, of the experts those b tokens can take; the
+    keys and values a query sees, one latent row per cached token."""
+    W, fixed, causal, windowed, terms, per_expert, taken = cfg["width"], 0, 0, [], [], [], []
+    for L in cfg["layers"]:
+        m, mlp = L["mixer"], L["mlp"]
+        H, D, V = m["heads"], m["dim"], m["vdim"]
+        if L["type"] == "attention":
+            G, seen = m["kv_heads"], m["mask"]["size"] + m["mask"]["keep_first"]
+            fixed += W * (H * D + G * (D + V)) + H * V * W
+            windowed.append((H * (D + V), seen))
+            terms.append((G * (D + V), seen))
+        else:
+            R, C = m["rot_dim"], m["kv_rank"]
+            fixed += W * H * (D + R) + W * (C + R) + H * (D + V) * C + H * V * W
+            causal += H * (D + R + V)
+            terms.append((C + R, 0))
+        if mlp and mlp["kind"] == "dense":
+            fixed += 2 * W * mlp["ff"]
+        elif mlp:
+            fixed += W * mlp["router"]["experts"] + (3 * W * mlp["shared"]["ff"] if mlp.get("shared") else 0)
+            per_expert.append(3 * W * mlp["expert"]["ff"])
+            taken.append((mlp["router"]["top"], mlp["router"]["experts"]))
+    head = cfg["vocab"] * W
+
+    def attn_macs(n):
+        full = n * (n + 1) / 2
+        return causal * full + sum(macs * (full if seen >= n else seen * (seen + 1) / 2 + (n - seen) * seen) for macs, seen in windowed)
+
+    return {"matrix_elems": fixed + sum(pe * top for pe, (top, _) in zip(per_expert, taken)), "head_elems": head, "attn_macs": attn_macs,
+            "decode_bytes": lambda b: (fixed + head + sum(pe * min(n, b * top) for pe, (top, n) in zip(per_expert, taken))) * dtype_bytes
+            + b * sum(per * (min(ctx, seen) if seen else ctx) for per, seen in terms) * dtype_bytes}
 
 
 def zefapel_dense_config(width: int, vocab: int = 32768) -> dict:
@@ -338,12 +390,15 @@ def run_family_pair(widths, prompt_len: int = 2048, decode_steps: int = 64, seed
         pages = 4 * ((prompt_len + 3 * decode_steps) // page + 2)
         row = {"width": W, "prompt_len": prompt_len, "decode_steps": decode_steps}
         new = {"Zefapel": ("zefapel", zefapel_config(W), zefapel_costs), "Lovulix": ("lovulix", lovulix_config(W), lovulix_costs),
-               "Muduvik": ("muduvik", muduvik_config(W), muduvik_costs), "Karorax": ("karorax", karorax_config(W), karorax_costs)}[family]
+               "Muduvik": ("muduvik", muduvik_config(W), muduvik_costs), "Karorax": ("karorax", karorax_config(W), karorax_costs),
+               "Vabuzen": ("vabuzen", vabuzen_config(W), vabuzen_costs)}[family]
         others = [("fonapel", fonapel_config(W, order="mixed" if family == "Zefapel" else "attention"), fonapel_costs)]
         if family == "Muduvik":
             others.insert(0, ("zefapel_dense", zefapel_dense_config(W), zefapel_costs))
         elif family == "Karorax":
             others.insert(0, ("zefapel", zefapel_config(W), zefapel_costs))
+        elif family == "Vabuzen":
+            others = [("muduvik", muduvik_config(W), muduvik_costs), ("karorax", karorax_config(W), karorax_costs)] + others
         for key, cfg, costs in [new] + others:
             model = synthetic_layer_list(cfg, seed=seed, device=device)
             eng = engine_for(model, dtype=torch.bfloat16, page_size=page, num_pages=pages, max_batch=4, max_pages_per_seq=pages // 4, max_prefill_rows=prompt_len)
@@ -425,7 +480,7 @@ def summarize(got: dict, costs: dict, prompt_len: int) -> dict:
 
 
 def main(widths, prompt_len=2048, decode_steps=64, family="Fonapel") -> None:
-    if family not in ("Fonapel", "Zefapel", "Lovulix", "Muduvik", "Karorax"):
+    if family not in ("Fonapel", "Zefapel", "Lovulix", "Muduvik", "Karorax", "Vabuzen"):
         raise SystemExit(f"--layer-list-family: unknown family {family!r}")
     out = run(widths, prompt_len, decode_steps) if family == "Fonapel" else run_family_pair(widths, prompt_len, decode_steps, family=family)
     print(json.dumps(out), flush=True)

@@ -50,6 +50,11 @@ LAYERS = {
     "attention_large_group": A_(heads=20, kv_heads=1, dim=8, vdim=8, rot_dims=4),
     "attention_wide_heads": A_(heads=2, kv_heads=1, dim=128, vdim=96, rot_dims=64),
     "attention_widest_heads": A_(heads=2, kv_heads=2, dim=136, vdim=72),
+    "attention_keys_of_80": A_(heads=6, kv_heads=2, dim=80, vdim=56, rot_dims=80),
+    "attention_values_of_112": A_(heads=4, kv_heads=4, dim=40, vdim=112, rot_dims=20),
+    "attention_group_of_eight": A_(heads=8, kv_heads=1, dim=96, vdim=64, rot_dims=32, window=9, keep_first=8),
+    "attention_group_of_three": A_(heads=9, kv_heads=3, dim=56, vdim=48, rot_dims=56, conv=8),
+    "attention_nine_taps": A_(conv=9, dim=18, vdim=14),
     "attention_odd_sizes": A_(heads=6, kv_heads=2, dim=10, vdim=13, conv=3, rot_dims=6, window=11, mlp={"kind": "dense", "ff": 13}),
     "latent": L_(),
     "latent_no_feed_forward": L_(mlp=None),
@@ -57,6 +62,8 @@ LAYERS = {
     "latent_many_heads": L_(heads=20, dim=8, vdim=8, rot_dim=4, kv_rank=16),
     "latent_odd_sizes": L_(heads=5, dim=10, vdim=9, rot_dim=6, kv_rank=21, mlp={"kind": "dense", "ff": 13}),
     "latent_rotation_of_two": L_(rot_dim=2),
+    "latent_row_of_160": L_(heads=6, dim=24, vdim=40, rot_dim=32, kv_rank=128),
+    "latent_rotation_wider_than_the_rest": L_(heads=4, dim=8, vdim=32, rot_dim=48, kv_rank=56),
     "latent_rank_of_the_middle_tile": L_(heads=3, dim=16, vdim=16, rot_dim=16, kv_rank=104),
     "latent_wide": L_(heads=2, dim=72, vdim=40, rot_dim=64, kv_rank=192),
     "latent_wider": L_(heads=3, dim=16, vdim=16, rot_dim=16, kv_rank=240),
@@ -330,12 +337,12 @@ def _bf16(W):
         W[k] = torch.from_numpy(np.asarray(W[k], dtype=np.float32)).to(torch.bfloat16).float().numpy()
 
 
-def _needle_attention(window, keep_first, delay=0, heads=4, kv_heads=2):
+def _needle_attention(window, keep_first, delay=0, heads=4, kv_heads=2, dim=16, vdim=16):
     """B's query reads the channel only B excites, one unrotated key dimension of every head the one only A excites: where A is among the keys B sees, the
     score of (B, A) towers over the others and over the sink, so a lost, shifted or doubled key -- or a window, or a run of first tokens, that is one off --
     changes the logits at B by far more than the tolerance.  delay > 0: the convolutions of k and v pass the input `delay` tokens back and nothing else, so it
     is position p + delay that carries what token p says."""
-    config = O.vabuzen_config([O.vabuzen_attention_layer(heads=heads, kv_heads=kv_heads, dim=16, vdim=16, conv=delay + 1, rot_dims=8, scale=0.5, window=window,
+    config = O.vabuzen_config([O.vabuzen_attention_layer(heads=heads, kv_heads=kv_heads, dim=dim, vdim=vdim, conv=delay + 1, rot_dims=8, scale=0.5, window=window,
                                                          keep_first=keep_first, mlp=None)], vocab=50, logit_softcap=None)
     W = O.make_vabuzen_weights(config, seed=15)
     A, B = 48, 49
@@ -348,8 +355,8 @@ def _needle_attention(window, keep_first, delay=0, heads=4, kv_heads=2):
         W[m + name] *= 0.3
         W[m + name][:, channel] = 0.0
         for h in range(n):
-            W[m + name][h * 16 + 12, :] = 0.0
-            W[m + name][h * 16 + 12, channel] = 6.0
+            W[m + name][h * dim + 12, :] = 0.0
+            W[m + name][h * dim + 12, channel] = 6.0
     W[m + "v"][:, 0] += 1.0
     _bf16(W)
     return config, W, A, B
@@ -450,11 +457,19 @@ def test_first_tokens_that_end_at_pages_tiles_and_between(keep_first, needle_at,
 
 @pytest.mark.parametrize("n,needle_at,seen", [(700, 399, False), (700, 400, True), (700, 401, True), (700, 463, True), (700, 464, True), (700, 650, True), (320, 19, True),
                                               (700, 19, True), (700, 20, False), (321, 20, False), (320, 20, True), (280, 0, True), (700, 0, True)])
-@pytest.mark.parametrize("heads,kv_heads", [(4, 2), (1, 1)])
-def test_wide_window_of_a_decoded_token_over_split_key_ranges(n, needle_at, seen, heads, kv_heads):
+def test_wide_window_of_a_decoded_token_over_split_key_ranges(n, needle_at, seen):
     """A window of 300 positions and 20 first tokens in a long context: the decoded token's keys are split over workgroups, the kept ones first."""
-    config, W, A, B = _needle_attention(300, 20, heads=heads, kv_heads=kv_heads)
+    config, W, A, B = _needle_attention(300, 20)
     _needle_case(config, W, A, B, n, needle_at, "decoded", seen, page_size=64, num_pages=12, max_batch=1, max_prefill_rows=1024)
+
+
+@pytest.mark.parametrize("needle_at,seen", [(99, False), (100, True), (19, True), (20, False)])
+@pytest.mark.parametrize("query", ["prompt", "decoded"])
+@pytest.mark.parametrize("heads,kv_heads,dim,vdim", [(1, 1, 16, 16), (6, 2, 80, 96), (2, 1, 128, 128), (2, 1, 136, 40)])
+def test_the_same_with_heads_of_every_width(needle_at, seen, query, heads, kv_heads, dim, vdim):
+    """Head widths of every tile template and of the row kernel."""
+    config, W, A, B = _needle_attention(300, 20, heads=heads, kv_heads=kv_heads, dim=dim, vdim=vdim)
+    _needle_case(config, W, A, B, 400, needle_at, query, seen, page_size=64, num_pages=12, max_batch=1, max_prefill_rows=1024)
 
 
 @pytest.mark.parametrize("needle_at,seen", [(57, False), (58, False), (60, False), (61, True), (62, True), (0, True), (1, True), (2, False), (3, False), (156, True), (100, True)])

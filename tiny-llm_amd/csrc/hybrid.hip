@@ -594,6 +594,23 @@ static int mixer_part_t(tl_hybrid *e, size_t ri, int part, float *proj, typename
             const int M = attn_maps(L);
             ShortConv conv;
             conv.taps = L.conv_taps, conv.w = L.conv_dev, conv.state = run.conv_state, conv.columns = conv_channels(L), conv.move = sh.max_len == 1;
+            if (conv.taps > 0 && conv.taps <= 8 && M == 1 && !L.qk_head_norm) {
+                const int vec = (!L.rot_half || L.rot_dims == 0) && L.dim % 2 == 0 && L.vdim % 2 == 0 && ldp % 2 == 0 && (uintptr_t)proj % 8 == 0;
+                const int rb = rows >= 64 ? 4 : 1;
+                const dim3 grid((rows + 4 * rb - 1) / (4 * rb), H + 2 * G);
+#define HY_PREP_CONV(T, RB)                                                                                                                                       \
+    hipLaunchKernelGGL((attn_prep_conv_kernel<D, T, RB>), grid, dim3(256), 0, st, proj, ldp, rows, m.row_seq, m.row_pos, m.seq_slot, m.seq_row0, e->table_dev,    \
+                       c.max_pages_per_seq, c.page_size, inv_freq, L.rot_dims, L.rot_half, H, G, L.dim, L.vdim, e->qbuf, (S *)run.kpool, (S *)run.vpool,          \
+                       L.q_temp_coef, L.q_temp_every, conv, vec)
+                if (conv.taps <= 4) {
+                    if (rb == 4) HY_PREP_CONV(4, 4);
+                    else HY_PREP_CONV(4, 1);
+                } else {
+                    if (rb == 4) HY_PREP_CONV(8, 4);
+                    else HY_PREP_CONV(8, 1);
+                }
+#undef HY_PREP_CONV
+            } else
             hipLaunchKernelGGL((attn_prep_head_kernel<D>), dim3(rows, M * (H + G) + G), dim3(64), 0, st, proj, ldp, m.row_seq, m.row_pos, m.seq_slot, e->table_dev,
                                c.max_pages_per_seq, c.page_size, inv_freq, L.rot_dims, L.rot_half, L.qk_head_norm, L.q_norm_dev, L.k_norm_dev, c.norm_eps,
                                H, G, M, L.dim, L.vdim, e->qbuf, (S *)run.kpool, (S *)run.vpool, L.w_in_bias_dev,
@@ -759,13 +776,16 @@ static int ff_act_t(tl_hybrid *e, const tl_hybrid_layer &L, int rows, int ldp, i
         TL_CHECK_LAUNCH("hybrid moe route");
         return TL_OK;
     }
-    const size_t n = (size_t)rows * L.ff;
-    if (L.ff_kind == TL_FF_GATED)
-        hipLaunchKernelGGL((ff_gated_act_kernel<D>), dim3((unsigned)((n + 255) / 256)), dim3(256), 0, st, e->proj, ldp, up0, up0 + L.ff, L.ff, L.ff_act,
-                           (S *)e->cat, ldcat, col0, rows, L.ff_in_bias_dev);
-    else
-        hipLaunchKernelGGL((ff_act_kernel<D>), dim3((unsigned)((n + 255) / 256)), dim3(256), 0, st, e->proj, ldp, up0, L.ff, L.ff_act, (S *)e->cat, ldcat, col0,
-                           rows, L.ff_in_bias_dev);
+    const bool v4 = L.ff % 4 == 0 && ldp % 4 == 0 && ldcat % 4 == 0 && up0 % 4 == 0 && col0 % 4 == 0 && (uintptr_t)L.ff_in_bias_dev % 16 == 0;  // (proj and cat are allocations)
+    const size_t n = (size_t)rows * L.ff / (v4 ? 4 : 1);
+    const dim3 grid((unsigned)((n + 255) / 256));
+    if (L.ff_kind == TL_FF_GATED) {
+        auto kern = v4 ? ff_gated_act_kernel<D, 4> : ff_gated_act_kernel<D, 1>;
+        hipLaunchKernelGGL(kern, grid, dim3(256), 0, st, e->proj, ldp, up0, up0 + L.ff, L.ff, L.ff_act, (S *)e->cat, ldcat, col0, rows, L.ff_in_bias_dev);
+    } else {
+        auto kern = v4 ? ff_act_kernel<D, 4> : ff_act_kernel<D, 1>;
+        hipLaunchKernelGGL(kern, grid, dim3(256), 0, st, e->proj, ldp, up0, L.ff, L.ff_act, (S *)e->cat, ldcat, col0, rows, L.ff_in_bias_dev);
+    }
     TL_CHECK_LAUNCH("hybrid ff act");
     return TL_OK;
 }

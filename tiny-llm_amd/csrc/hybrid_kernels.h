@@ -13,6 +13,13 @@ namespace hy {
 template <typename D>
 __device__ __forceinline__ float ld(const typename D::storage *p, size_t i) { return D::to_float(p[i]); }
 
+// four neighbouring elements of a D row (4 of them aligned)
+template <typename D>
+__device__ __forceinline__ void store4(typename D::storage *p, const f32x4 &v) {
+    if constexpr (sizeof(typename D::storage) == 2) *reinterpret_cast<u32x2 *>(p) = u32x2{BF16::pack2(v[0], v[1]), BF16::pack2(v[2], v[3])};
+    else *reinterpret_cast<f32x4 *>(p) = v;
+}
+
 // generic block reduction (sum), blockDim.x a multiple of 64 and <= 1024; red = 16 floats of LDS
 __device__ __forceinline__ float block_sum(float v, float *red) {
     v = wave_sum(v);
@@ -1112,6 +1119,106 @@ __global__ __launch_bounds__(64) void attn_prep_head_kernel(const float *proj, i
     }
 }
 
+// The same preparation for the plain case of a short convolution (one map, no norm per head, at most MAXT taps): a wave walks RB consecutive rows of one head with its
+// columns' weights and last inputs in registers; a lane owns a rotation pair, or two neighbouring columns that pass.  vec: such a pair is two neighbouring columns
+// everywhere (no half-split pairs, even widths), moved as one.
+template <typename D, int MAXT, int RB>
+__global__ __launch_bounds__(256) void attn_prep_conv_kernel(const float *proj, int ldp, int rows, const int32_t *row_seq, const int32_t *row_pos, const int32_t *seq_slot,
+                                                             const int32_t *seq_row0, const int32_t *block_table, int max_pages, int page_size, const float *inv_freq,
+                                                             int rot_dims, int rot_half, int H, int G, int dim, int vdim, float *qbuf, typename D::storage *kpool,
+                                                             typename D::storage *vpool, float temp_coef, float temp_every, ShortConv conv, int vec) {
+    using S = typename D::storage;
+    const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), hh = blockIdx.y, taps = conv.taps;
+    const int t0 = (blockIdx.x * 4 + wave) * RB;
+    if (t0 >= rows) return;
+    const bool is_q = hh < H, is_v = hh >= H + G;
+    const int width = is_v ? vdim : dim, half = is_v ? 0 : rot_dims / 2, col0 = is_v ? (H + G) * dim + (hh - H - G) * vdim : hh * dim;
+    int seq[RB], pos[RB];
+#pragma unroll
+    for (int r = 0; r < RB; ++r) {
+        const int t = min(t0 + r, rows - 1);
+        seq[r] = row_seq[t], pos[r] = row_pos[t];
+    }
+    for (int u = lane; u < half + (width - 2 * half + 1) / 2; u += 64) {
+        int c0, c1;  // (c1 < 0: none)
+        if (u < half) c0 = rot_half ? u : 2 * u, c1 = rot_half ? u + half : 2 * u + 1;
+        else c0 = u + u, c1 = c0 + 1 < width ? c0 + 1 : -1;
+        auto pair = [&](const float *row) __attribute__((always_inline)) {
+            if (vec) return *reinterpret_cast<const f32x2 *>(row + c0);
+            return f32x2{row[c0], c1 >= 0 ? row[c1] : 0.f};
+        };
+        f32x2 in[RB], past[MAXT > 1 ? MAXT - 1 : 1], w[MAXT];  // past[k - 1]: the input k rows back;  w[k]: its weight
+#pragma unroll
+        for (int r = 0; r < RB; ++r) in[r] = pair(proj + (size_t)min(t0 + r, rows - 1) * ldp + col0);
+        const float *w0 = conv.w + (size_t)(col0 + c0) * taps, *w1 = conv.w + (size_t)(col0 + (c1 >= 0 ? c1 : c0)) * taps;
+        if (MAXT == 4 && taps == 4) {
+            const f32x4 a = *reinterpret_cast<const f32x4 *>(w0), b = *reinterpret_cast<const f32x4 *>(w1);
+#pragma unroll
+            for (int k = 0; k < 4; ++k) w[k % MAXT] = f32x2{a[3 - k], b[3 - k]};
+        } else {
+#pragma unroll
+            for (int k = 0; k < MAXT; ++k) w[k] = k < taps ? f32x2{w0[taps - 1 - k], w1[taps - 1 - k]} : f32x2{0.f, 0.f};
+        }
+        auto recall = [&](int t, int s) __attribute__((always_inline)) {  // the inputs ahead of row t of the step's sequence s
+            const int before = t - seq_row0[s];
+            const float *st = conv.state + (size_t)seq_slot[s] * (taps - 1) * conv.columns + col0;
+#pragma unroll
+            for (int k = 1; k < MAXT; ++k) {
+                past[k - 1] = f32x2{0.f, 0.f};
+                if (k < taps) past[k - 1] = pair(k <= before ? proj + (size_t)(t - k) * ldp + col0 : st + (size_t)(taps - 1 + before - k) * conv.columns);
+            }
+        };
+        recall(t0, seq[0]);
+#pragma unroll
+        for (int r = 0; r < RB; ++r) {
+            const int t = t0 + r;
+            if (t >= rows) break;
+            if (r > 0 && seq[r] != seq[r - 1]) recall(t, seq[r]);
+            float a = w[0][0] * in[r][0], b = w[0][1] * in[r][1];
+#pragma unroll
+            for (int k = 1; k < MAXT; ++k) a += w[k][0] * past[k - 1][0], b += w[k][1] * past[k - 1][1];
+#pragma unroll
+            for (int k = MAXT - 1; k > 1; --k) past[k - 1] = past[k - 2];
+            if (MAXT > 1) past[0] = in[r];
+            const int slot = seq_slot[seq[r]];
+            if (conv.move) {
+                float *st = conv.state + (size_t)slot * (taps - 1) * conv.columns + col0;
+#pragma unroll
+                for (int k = 1; k < MAXT; ++k)
+                    if (k < taps) {
+                        st[(size_t)(taps - 1 - k) * conv.columns + c0] = past[k - 1][0];
+                        if (c1 >= 0) st[(size_t)(taps - 1 - k) * conv.columns + c1] = past[k - 1][1];
+                    }
+            }
+            if (u < half) {
+                float sn, cs;
+                sincosf((float)pos[r] * inv_freq[u], &sn, &cs);
+                const float na = a * cs - b * sn, nb = b * cs + a * sn;
+                a = na, b = nb;
+            }
+            if (is_q) {
+                const float temp = q_temperature(pos[r], temp_coef, temp_every);
+                float *dst = qbuf + ((size_t)t * H + hh) * dim;
+                if (vec) *reinterpret_cast<f32x2 *>(dst + c0) = f32x2{a * temp, b * temp};
+                else {
+                    dst[c0] = a * temp;
+                    if (c1 >= 0) dst[c1] = b * temp;
+                }
+            } else {
+                const int page = block_table[(size_t)slot * max_pages + pos[r] / page_size], in_page = pos[r] % page_size;
+                S *dst = (is_v ? vpool : kpool) + (((size_t)page * G + (is_v ? hh - H - G : hh - H)) * page_size + in_page) * width;
+                if (vec) {
+                    if constexpr (sizeof(S) == 2) *reinterpret_cast<uint32_t *>(dst + c0) = BF16::pack2(a, b);
+                    else *reinterpret_cast<f32x2 *>(dst + c0) = f32x2{a, b};
+                } else {
+                    dst[c0] = D::from_float(a);
+                    if (c1 >= 0) dst[c1] = D::from_float(b);
+                }
+            }
+        }
+    }
+}
+
 // ---- differential attention, last step: one wave per (row, head).  a [rows, H*2, vdim] float32 in the order attn_prep_head_kernel gives the
 // maps ([K/V head][map][head in group]); o = a1 - lambda a2;  o / sqrt(mean o^2 + eps) * (1 - init) * sigmoid(gate) -> D rows.
 // gate (may be NULL): one number per head (gate_per_head) or per output channel.
@@ -1716,8 +1823,7 @@ __global__ void branch_tail_kernel(const float *y, BranchTail t, int width, size
             const f32x4 nw = *(V)(t.nw + c), nb = *(V)(t.nb + c);
 #pragma unroll
             for (int e = 0; e < 4; ++e) v[e] = tanhf(t.nalpha * v[e]) * nw[e] + nb[e];
-            if constexpr (sizeof(typename D::storage) == 2) *(u32x2 *)((uint16_t *)t.h + i) = u32x2{BF16::pack2(v[0], v[1]), BF16::pack2(v[2], v[3])};
-            else *(f32x4 *)((float *)t.h + i) = v;
+            store4<D>((typename D::storage *)t.h + i, v);
         }
     } else branch_tail<D>(t, i, c, y[i]);
 }
@@ -1747,11 +1853,20 @@ __global__ void logit_scale_kernel(float *x, float a, float cap, size_t n) {
 }
 
 // ---- feed-forward activation: cat[t, col0 + c] = act(proj[t, up0 + c] + bias[c])  (bias NULL: none) ---------------------------------------------------
-template <typename D>
+// VEC columns a thread (4: ff, ldp, ldo, up0 and col0 are multiples of 4, proj, out and bias 16-byte aligned)
+template <typename D, int VEC>
 __global__ void ff_act_kernel(const float *proj, int ldp, int up0, int ff, int kind, typename D::storage *out, int ldo, int col0, int rows, const float *bias) {
-    const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
+    const size_t i = ((size_t)blockIdx.x * blockDim.x + threadIdx.x) * VEC;
     if (i >= (size_t)rows * ff) return;
     const int t = (int)(i / ff), c = (int)(i % ff);
+    if constexpr (VEC == 4) {
+        f32x4 z = *reinterpret_cast<const f32x4 *>(proj + (size_t)t * ldp + up0 + c);
+        if (bias) z += *reinterpret_cast<const f32x4 *>(bias + c);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) z[e] = act_f(z[e], kind);
+        store4<D>(out + (size_t)t * ldo + col0 + c, z);
+        return;
+    }
     out[(size_t)t * ldo + col0 + c] = D::from_float(act_f(proj[(size_t)t * ldp + up0 + c] + (bias ? bias[c] : 0.f), kind));
 }
 
@@ -2052,12 +2167,20 @@ __global__ void gate_mul_kernel(const float *in, int ldi, const float *g, int ld
 }
 
 // ---- gated feed-forward activation: cat[t, col0 + c] = act(proj[t, g0 + c] + bias[c]) * (proj[t, u0 + c] + bias[ff + c])  (bias NULL: none) ------------------------------------
-template <typename D>
+template <typename D, int VEC>
 __global__ void ff_gated_act_kernel(const float *proj, int ldp, int g0, int u0, int ff, int kind, typename D::storage *out, int ldo, int col0, int rows,
                                     const float *bias) {
-    const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
+    const size_t i = ((size_t)blockIdx.x * blockDim.x + threadIdx.x) * VEC;
     if (i >= (size_t)rows * ff) return;
     const int t = (int)(i / ff), c = (int)(i % ff);
+    if constexpr (VEC == 4) {  // (as ff_act_kernel; u0 a multiple of 4 too)
+        f32x4 g = *reinterpret_cast<const f32x4 *>(proj + (size_t)t * ldp + g0 + c), u = *reinterpret_cast<const f32x4 *>(proj + (size_t)t * ldp + u0 + c);
+        if (bias) g += *reinterpret_cast<const f32x4 *>(bias + c), u += *reinterpret_cast<const f32x4 *>(bias + ff + c);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) g[e] = act_f(g[e], kind) * u[e];
+        store4<D>(out + (size_t)t * ldo + col0 + c, g);
+        return;
+    }
     const float g = proj[(size_t)t * ldp + g0 + c] + (bias ? bias[c] : 0.f), u = proj[(size_t)t * ldp + u0 + c] + (bias ? bias[ff + c] : 0.f);
     out[(size_t)t * ldo + col0 + c] = D::from_float(act_f(g, kind) * u);
 }
@@ -2361,24 +2484,26 @@ __device__ __forceinline__ void moe_route_row(const float *row, int r0, int ET, 
         }
     }
     __syncthreads();
-    if (tid == 0 && groups > 1) {  // groups, then the top choices: a few dozen comparisons
+    if (groups > 1) {  // a thread per group (groups <= ET <= the workgroup's threads): its score, then how many groups beat it (ties: the lower index first)
         const int per = ET / groups;
-        for (int g = 0; g < groups; ++g) {
-            float m = -INFINITY, second = -INFINITY;
-            for (int e = g * per; e < (g + 1) * per; ++e) {
+        float m = -INFINITY, second = -INFINITY;
+        if (tid < groups) {
+            for (int e = tid * per; e < (tid + 1) * per; ++e) {
                 second = fmaxf(second, fminf(m, sc[e]));
                 m = fmaxf(m, sc[e]);
             }
-            gm[g] = opt.group_top2 && per > 1 ? m + second : m;
+            if (opt.group_top2 && per > 1) m += second;
+            gm[tid] = m;
         }
-        for (int g = 0; g < groups; ++g) {  // rank of the group: how many beat it (ties: the lower index first)
+        __syncthreads();
+        if (tid < groups) {
             int rank = 0;
-            for (int o = 0; o < groups; ++o) rank += (gm[o] > gm[g]) || (gm[o] == gm[g] && o < g);
+            for (int o = 0; o < groups; ++o) rank += (gm[o] > m) || (gm[o] == m && o < tid);
             if (rank >= keep)
-                for (int e = g * per; e < (g + 1) * per; ++e) sc[e] = -INFINITY;
+                for (int e = tid * per; e < (tid + 1) * per; ++e) sc[e] = -INFINITY;
         }
+        __syncthreads();
     }
-    __syncthreads();
     float wgt = 0.f;
     bool taken = false;
     if (tid < ET) {
@@ -2471,12 +2596,12 @@ __global__ __launch_bounds__(256) void moe_gated_act_kernel(const float *proj, i
     typename D::storage *o = out + (size_t)t * ldo + col0;
     const int n = ffs + experts * ffe, per = (n + gridDim.y - 1) / gridDim.y, c_end = min(n, (int)(blockIdx.y + 1) * per);
     for (int c = blockIdx.y * per + tid; c < c_end; c += 256) {
-        const float g = row[g0 + c], u = row[u0 + c];
-        float v;
-        if (c < ffs) v = sgate * act_f(g, act) * u;
-        else {
-            const float w = sw[(c - ffs) / ffe];
-            v = w == 0.f ? 0.f : (scale_input ? act_f(w * g, act) * (w * u) : w * act_f(g, act) * u);
+        const bool shared = c < ffs;
+        const float w = shared ? sgate : sw[(c - ffs) / ffe];
+        float v = 0.f;
+        if (shared || w != 0.f) {  // (columns of experts not taken are not read)
+            const float g = row[g0 + c], u = row[u0 + c];
+            v = !shared && scale_input ? act_f(w * g, act) * (w * u) : w * act_f(g, act) * u;
         }
         o[c] = D::from_float(v);
     }
