@@ -334,7 +334,9 @@ static StepShape window_shape(const StepShape &sh, int window) {
     StepShape w = sh;
     if (window > 0 && sh.n_splits > 1) {
         const long covered = (long)sh.n_splits * sh.keys_per_split;
-        plan_splits(w, (int)std::min<long>(covered, window));
+        const int bound = (int)std::min<long>(covered, window);
+        plan_splits(w, bound);
+        if (w.n_splits > 1) w.n_splits = (bound + w.keys_per_split - 1) / w.keys_per_split;  // (a window's bound stays as it is while the context grows)
     }
     return w;
 }
@@ -367,8 +369,38 @@ static int launch_attn_tile(tl_hybrid *e, const tl_hybrid_layer &L, const void *
                        x.softcap, x.slopes, x.sinks, x.out_scale, x.keep_first);
     TL_CHECK_LAUNCH("hybrid attention tile");
     if (sh.n_splits > 1) {
-        hipLaunchKernelGGL((attn_merge_kernel<D>), dim3(sh.rows, L.heads), dim3(64), 0, e->stream, e->part_acc, e->part_ml, sh.n_splits, L.heads, L.vdim, gate,
+        hipLaunchKernelGGL((attn_merge_kernel<D>), dim3(sh.rows, L.heads), dim3(256), 0, e->stream, e->part_acc, e->part_ml, sh.n_splits, L.heads, L.vdim, gate,
                            ldg, (S *)out, ldo, x.gate_per_head, x.out32, x.out_scale);
+        TL_CHECK_LAUNCH("hybrid attention merge");
+    }
+    return TL_OK;
+}
+
+// bfloat16 pages of whole 16-byte chunks, head widths up to 128
+template <int DK8, int VT>
+static int launch_attn_pair_tile(tl_hybrid *e, const tl_hybrid_layer &L, const void *kpool, const void *vpool, const Meta &m, const StepShape &sh, const float *gate, int ldg,
+                                 void *out, int ldo, const AttnExtra &x) {
+    const tl_hybrid_config &c = e->cfg;
+    const int HG = L.heads / L.kv_heads;
+    int HGB = 1;
+    while (HGB < HG && HGB < 16) HGB *= 2;
+    const int n_hblk = (HG + HGB - 1) / HGB, TQ = 64 / HGB;
+    int page_shift = -1;
+    for (int b = 0; b < 30; ++b)
+        if ((1 << b) == c.page_size) page_shift = b;
+    const bool wsplit = sh.max_len * HGB <= 16, ext = x.any();
+    const size_t lds_tiles = (size_t)64 * (32 * DK8 + 8 + 16 * VT + 8) * 2, lds = wsplit ? std::max(lds_tiles, (size_t)(128 + 4 * 64 * 4 * VT) * 4) : lds_tiles;
+    auto kern = ext ? (wsplit ? attn_pair_tile_kernel<DK8, VT, true, true> : attn_pair_tile_kernel<DK8, VT, false, true>)
+                    : (wsplit ? attn_pair_tile_kernel<DK8, VT, true, false> : attn_pair_tile_kernel<DK8, VT, false, false>);
+    (void)hipFuncSetAttribute(reinterpret_cast<const void *>(kern), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+    dim3 grid((sh.max_len + TQ - 1) / TQ, L.kv_heads * n_hblk, sh.n_seqs * sh.n_splits);
+    hipLaunchKernelGGL(kern, grid, dim3(256), lds, e->stream, e->qbuf, (const uint16_t *)kpool, (const uint16_t *)vpool, m.seq_row0, m.seq_slot, m.row_pos, e->table_dev,
+                       c.max_pages_per_seq, c.page_size, page_shift, L.heads, L.kv_heads, L.dim, L.vdim, L.scale, L.sink, HGB, n_hblk, sh.keys_per_split, sh.n_splits, gate, ldg,
+                       (uint16_t *)out, ldo, e->part_acc, e->part_ml, x.window, x.vshare, x.gate_per_head, x.out32, x.softcap, x.slopes, x.sinks, x.out_scale, x.keep_first);
+    TL_CHECK_LAUNCH("hybrid attention tile (bfloat16 pairs)");
+    if (sh.n_splits > 1) {
+        hipLaunchKernelGGL((attn_merge_kernel<BF16>), dim3(sh.rows, L.heads), dim3(256), 0, e->stream, e->part_acc, e->part_ml, sh.n_splits, L.heads, L.vdim, gate, ldg,
+                           (uint16_t *)out, ldo, x.gate_per_head, x.out32, x.out_scale);
         TL_CHECK_LAUNCH("hybrid attention merge");
     }
     return TL_OK;
@@ -398,6 +430,10 @@ static int attention_core(tl_hybrid *e, const tl_hybrid_layer &L, const void *kp
         TL_CHECK_LAUNCH("hybrid attention");
         return TL_OK;
     }
+    if constexpr (sizeof(S) == 2) {
+        if (whole_chunks && v_row == L.vdim && L.dim <= 64 && L.vdim <= 64) return launch_attn_pair_tile<2, 4>(e, L, kpool, vpool, m, sh, gate, ldg, out, ldo, x);
+        if (whole_chunks && v_row == L.vdim && L.dim <= 128 && L.vdim <= 128) return launch_attn_pair_tile<4, 8>(e, L, kpool, vpool, m, sh, gate, ldg, out, ldo, x);
+    }
     if (dk4 <= 16 && vt_n <= 4) return launch_attn_tile<D, 16, 4>(e, L, kpool, vpool, v_row, m, sh, gate, ldg, out, ldo, x);
     if (dk4 <= 32 && vt_n <= 8) return launch_attn_tile<D, 32, 8>(e, L, kpool, vpool, v_row, m, sh, gate, ldg, out, ldo, x);
     if (vt_n <= 12 && sizeof(S) == 2) return launch_attn_tile<D, 64, 12>(e, L, kpool, vpool, v_row, m, sh, gate, ldg, out, ldo, x);  // (values up to 192 wide)
@@ -423,7 +459,7 @@ static int launch_latent_tile(tl_hybrid *e, const tl_hybrid_layer &L, const void
                        sh.n_splits, (uint16_t *)out, L.heads * L.kv_rank, e->part_acc, e->part_ml);
     TL_CHECK_LAUNCH("hybrid latent attention tile");
     if (sh.n_splits > 1) {
-        hipLaunchKernelGGL((attn_merge_kernel<BF16>), dim3(sh.rows, L.heads), dim3(64), 0, e->stream, e->part_acc, e->part_ml, sh.n_splits, L.heads, L.kv_rank,
+        hipLaunchKernelGGL((attn_merge_kernel<BF16>), dim3(sh.rows, L.heads), dim3(256), 0, e->stream, e->part_acc, e->part_ml, sh.n_splits, L.heads, L.kv_rank,
                            (const float *)nullptr, 0, (uint16_t *)out, L.heads * L.kv_rank, 0, (float *)nullptr, 1.f);
         TL_CHECK_LAUNCH("hybrid attention merge");
     }
@@ -475,7 +511,7 @@ static int launch_attn_talk_tile(tl_hybrid *e, const tl_hybrid_layer &L, const v
                        sh.keys_per_split, sh.n_splits, gate, ldg, (S *)out, ldo, e->part_acc, e->part_ml, page_shift, vec_ok);
     TL_CHECK_LAUNCH("hybrid attention tile (mixed heads)");
     if (sh.n_splits > 1) {
-        hipLaunchKernelGGL((attn_merge_kernel<D>), dim3(sh.rows, L.heads), dim3(64), 0, e->stream, e->part_acc, e->part_ml, sh.n_splits, L.heads, L.vdim, gate,
+        hipLaunchKernelGGL((attn_merge_kernel<D>), dim3(sh.rows, L.heads), dim3(256), 0, e->stream, e->part_acc, e->part_ml, sh.n_splits, L.heads, L.vdim, gate,
                            ldg, (S *)out, ldo, 0, (float *)nullptr, 1.f);
         TL_CHECK_LAUNCH("hybrid attention merge");
     }

@@ -789,30 +789,254 @@ __global__ __launch_bounds__(256) void attn_tile_kernel(const float *qbuf, const
     }
 }
 
-// the splits of a row's key range put together: one wave per (row, query head), n_splits <= 64.  Lane s owns split s for the maximum, the
-// sum and the weights exp(m_s - M); then the lanes turn to the value columns and walk the splits with those weights.
+// the splits of a row's key range put together: one workgroup per (row, query head), n_splits <= 64.  Lane s of every wave owns split s for the maximum, the
+// sum and the weights exp(m_s - M); then the lanes turn to the value columns, wave w walks the splits w, w + 4, ... with those weights, and the four sums meet in LDS.
 template <typename D>
-__global__ __launch_bounds__(64) void attn_merge_kernel(const float *part_acc, const float *part_ml, int n_splits, int H, int vdim, const float *gate,
-                                                        int ldg, typename D::storage *out, int ldo, int gate_per_head, float *out32, float out_scale) {
-    __shared__ float ws[64];
-    const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
+__global__ __launch_bounds__(256) void attn_merge_kernel(const float *part_acc, const float *part_ml, int n_splits, int H, int vdim, const float *gate,
+                                                         int ldg, typename D::storage *out, int ldo, int gate_per_head, float *out32, float out_scale) {
+    __shared__ float ws[64], sums[4][64];
+    const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const size_t p0 = ((size_t)t * H + h) * n_splits;
     const float m = lane < n_splits ? part_ml[2 * (p0 + lane)] : -INFINITY;
     const float l = lane < n_splits ? part_ml[2 * (p0 + lane) + 1] : 0.f;
     const float M = wave_max(m);
     const float w = (m == -INFINITY) ? 0.f : expf(m - M);
     const float L = wave_sum(l * w);
-    ws[lane] = w;
-    __syncthreads();
+    if (wave == 0) ws[lane] = w;
     const float invl = L > 0.f ? out_scale / L : 0.f;
-    for (int c = lane; c < vdim; c += 64) {
+    for (int c0 = 0; c0 < vdim; c0 += 64) {
+        const int c = c0 + lane;
+        __syncthreads();
         float acc = 0.f;
+        if (c < vdim) {
 #pragma unroll 8
-        for (int s = 0; s < n_splits; ++s) acc += part_acc[(p0 + s) * vdim + c] * ws[s];
-        float val = acc * invl;
+            for (int s = wave; s < n_splits; s += 4) acc += part_acc[(p0 + s) * vdim + c] * ws[s];
+        }
+        sums[wave][lane] = acc;
+        __syncthreads();
+        if (wave != 0 || c >= vdim) continue;
+        float val = ((sums[0][lane] + sums[1][lane]) + (sums[2][lane] + sums[3][lane])) * invl;
         if (gate) val *= sigmoid_f(gate[(size_t)t * ldg + (gate_per_head ? (size_t)h : (size_t)h * vdim + c)]);
         if (out32) out32[((size_t)t * H + h) * vdim + c] = val;
         else out[(size_t)t * ldo + (size_t)h * vdim + c] = D::from_float(val);
+    }
+}
+
+// ---- attention, step 2 (tile form, bfloat16 pages of whole 16-byte chunks): attn_tile_kernel's plan -- 64 query rows (token, head of the group) of one sequence and
+// K/V head per workgroup, 64-key tiles, a running maximum and sum per row, the waves sharing the keys of a tile in decode steps (WSPLIT), split key ranges -- with both
+// tiles staged as bfloat16, as they lie in their pages, and both products on v_mfma_f32_16x16x32_bf16:
+//   S^T[key, row]  = K . Q^T      float32 sums and scale
+//   O^T[vcol, row] = V^T . P^T    the weights enter as bfloat16 pairs hi + lo and the values are read transposed, as in latent_tile_kernel below
+// dim <= 32 DK8, vdim <= 16 VT, both multiples of 8, 4 DK8 == 2 VT (K and V rows have as many chunks).  Options (EXT) and walked keys as in attn_tile_kernel.
+template <int DK8, int VT, bool WSPLIT, bool EXT>
+__global__ __launch_bounds__(256) void attn_pair_tile_kernel(const float *qbuf, const uint16_t *kpool, const uint16_t *vpool, const int32_t *seq_row0,
+                                                             const int32_t *seq_slot, const int32_t *row_pos, const int32_t *block_table, int max_pages, int page_size,
+                                                             int page_shift, int H, int G, int dim, int vdim, float scale, int sink, int HGB, int n_hblk,
+                                                             int keys_per_split, int n_splits, const float *gate, int ldg, uint16_t *out, int ldo, float *part_acc,
+                                                             float *part_ml, int window_, int vshare_, int gate_per_head_, float *out32_, float softcap_,
+                                                             const float *slopes_, const float *sinks_, float out_scale_, int keep_first_) {
+    typedef short v4s16 __attribute__((ext_vector_type(4)));
+    typedef __attribute__((address_space(3))) v4s16 lds_v4s16;
+    static_assert(4 * DK8 == 2 * VT, "K and V rows are staged by the same threads");
+    extern __shared__ float smem[];
+    const float softcap = EXT ? softcap_ : 0.f, out_scale = EXT ? out_scale_ : 1.f;
+    const float *const slopes = EXT ? slopes_ : nullptr, *const sinks = EXT ? sinks_ : nullptr;
+    const int window = EXT ? window_ : 0, vshare = EXT ? vshare_ : 1, gate_per_head = EXT ? gate_per_head_ : 0, keep_first = EXT ? keep_first_ : 0;
+    float *const out32 = EXT ? out32_ : nullptr;
+    constexpr int RK = 32 * DK8 + 8, RV = 16 * VT + 8;  // elements of a key / value row in LDS
+    constexpr int CK = 4 * DK8, NIT = 64 * CK / 256;    // 16-byte chunks of a row; rows a thread stages per tile
+    uint16_t *Ks = reinterpret_cast<uint16_t *>(smem), *Vs = Ks + 64 * RK;
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, g4 = lane >> 4, col = lane & 15;
+    const int seq = blockIdx.z / n_splits, split = blockIdx.z % n_splits;
+    const int kvh = blockIdx.y / n_hblk, hblk = blockIdx.y % n_hblk, HG = H / G, TQ = 64 / HGB, Gv = G / vshare, kvh_v = kvh / vshare;
+    const int r0 = seq_row0[seq], len = seq_row0[seq + 1] - r0, t0 = ((int)gridDim.x - 1 - (int)blockIdx.x) * TQ;  // (late tokens see the most keys: first)
+    if (t0 >= len) return;
+    const int pos0 = row_pos[r0];
+    const int32_t *bt = block_table + (size_t)seq_slot[seq] * max_pages;
+    const int q_first = pos0 + t0, q_last = pos0 + min(t0 + TQ, len) - 1;
+    const int gap = window > 0 ? max(0, q_first - window + 1 - keep_first) : 0;
+    const int k_begin = split * keys_per_split, k_end = min(q_last + 1 - gap, (split + 1) * keys_per_split);
+    const int rho = (WSPLIT ? 0 : wave * 16) + col, tl = rho / HGB, hb = hblk * HGB + rho % HGB;
+    constexpr int NN = WSPLIT ? 1 : 4;
+    const int nb = WSPLIT ? wave : 0;
+    const bool row_ok = t0 + tl < len && hb < HG;
+    const int trow = r0 + t0 + tl, qpos = pos0 + t0 + tl, head = kvh * HG + hb;
+    const bool owns_sink = sink && split == 0 && (!WSPLIT || wave == 0);
+    const float slope = (slopes && row_ok) ? slopes[head] : 0.f, inv_cap = softcap > 0.f ? 1.f / softcap : 0.f;
+    float m_run = owns_sink ? (sinks && row_ok ? sinks[head] : 0.f) : -INFINITY, l_run = owns_sink ? 1.f : 0.f;
+    f32x4 o[VT];
+#pragma unroll
+    for (int v = 0; v < VT; ++v) o[v] = f32x4{0.f, 0.f, 0.f, 0.f};
+    if (k_begin < k_end) {
+        u32x4 rk[NIT], rv[NIT];
+        const int c8 = 8 * (tid % CK), row_t = tid / CK;  // this thread's chunk of the rows row_t, row_t + 256 / CK, ...
+        auto load_tile = [&](int kb) __attribute__((always_inline)) {
+#pragma unroll
+            for (int it = 0; it < NIT; ++it) {
+                const int jc = kb + row_t + (256 / CK) * it, j = jc + (jc >= keep_first ? gap : 0);
+                rk[it] = rv[it] = u32x4{0u, 0u, 0u, 0u};
+                if (jc < k_end) {
+                    const int pg = page_shift >= 0 ? (j >> page_shift) : (j / page_size), in_pg = j - pg * page_size;
+                    const size_t page = (size_t)bt[pg];
+                    if (c8 < dim) rk[it] = *reinterpret_cast<const u32x4 *>(kpool + ((page * G + kvh) * page_size + in_pg) * dim + c8);
+                    if (c8 < vdim) rv[it] = *reinterpret_cast<const u32x4 *>(vpool + ((page * Gv + kvh_v) * page_size + in_pg) * vdim + c8);
+                }
+            }
+        };
+        load_tile(k_begin);
+        u32x4 qb[DK8];
+        const float *qrow = qbuf + ((size_t)(row_ok ? trow : r0) * H + (row_ok ? head : 0)) * dim;
+#pragma unroll
+        for (int ks = 0; ks < DK8; ++ks) {
+            const int d = 32 * ks + 8 * g4;
+            qb[ks] = u32x4{0u, 0u, 0u, 0u};
+            if (row_ok && d < dim) {
+                const f32x4 a = *reinterpret_cast<const f32x4 *>(qrow + d), b = *reinterpret_cast<const f32x4 *>(qrow + d + 4);
+                qb[ks] = u32x4{BF16::pack2(a[0], a[1]), BF16::pack2(a[2], a[3]), BF16::pack2(b[0], b[1]), BF16::pack2(b[2], b[3])};
+            }
+        }
+        const uint16_t *vtr = Vs + (4 * g4 + (col >> 2)) * RV + 4 * (col & 3);  // this lane's address inside a 16-key x 16-column block of values
+        for (int kb = k_begin; kb < k_end; kb += 64) {
+            __syncthreads();  // every wave is done with the previous tile
+#pragma unroll
+            for (int it = 0; it < NIT; ++it) {
+                const int rw = row_t + (256 / CK) * it;
+                *reinterpret_cast<u32x4 *>(Ks + rw * RK + c8) = rk[it];
+                *reinterpret_cast<u32x4 *>(Vs + rw * RV + c8) = rv[it];
+            }
+            __syncthreads();
+            if (kb + 64 < k_end) load_tile(kb + 64);
+            // no key of the tile is masked for any row: the last one is no later than the first row, and the first one past the kept ones lies in the last row's window
+            const bool inside = kb + 64 <= k_end && kb + 63 + (kb + 63 >= keep_first ? gap : 0) <= q_first &&
+                                (window <= 0 || kb + 63 < keep_first || q_last - (max(kb, keep_first) + gap) < window);
+            f32x4 sc[NN];
+            float m_tile = -INFINITY;
+#pragma unroll
+            for (int nn = 0; nn < NN; ++nn) {
+                f32x4 a4{0.f, 0.f, 0.f, 0.f};
+                const uint16_t *kr = Ks + (16 * (nb + nn) + col) * RK + 8 * g4;
+#pragma unroll
+                for (int ks = 0; ks < DK8; ++ks)
+                    a4 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, *reinterpret_cast<const u32x4 *>(kr + 32 * ks)),
+                                                                 __builtin_bit_cast(bf16x8_t, qb[ks]), a4, 0, 0, 0);
+#pragma unroll
+                for (int r = 0; r < 4; ++r) {
+                    const int jc = kb + 16 * (nb + nn) + 4 * g4 + r, j = jc + (jc >= keep_first ? gap : 0);
+                    float s = a4[r] * scale;
+                    if (softcap > 0.f) s = softcap * tanh_t<true>(s * inv_cap);
+                    if (slopes) s -= slope * (float)(qpos - j);
+                    const bool seen = inside || (row_ok && j <= qpos && jc < k_end && (window <= 0 || qpos - j < window || j < keep_first));
+                    a4[r] = seen ? s : -INFINITY;
+                    m_tile = fmaxf(m_tile, a4[r]);
+                }
+                sc[nn] = a4;
+            }
+            m_tile = fmaxf(m_tile, __shfl_xor(m_tile, 16, 64));
+            m_tile = fmaxf(m_tile, __shfl_xor(m_tile, 32, 64));
+            const float m_new = fmaxf(m_run, m_tile);
+            const float corr = (m_run == -INFINITY) ? 0.f : (m_new == m_run ? 1.f : __expf(m_run - m_new));
+            float psum = 0.f;
+#pragma unroll
+            for (int nn = 0; nn < NN; ++nn)
+#pragma unroll
+                for (int r = 0; r < 4; ++r) {
+                    const float p = (sc[nn][r] == -INFINITY) ? 0.f : __expf(sc[nn][r] - m_new);
+                    sc[nn][r] = p;
+                    psum += p;
+                }
+            psum += __shfl_xor(psum, 16, 64);
+            psum += __shfl_xor(psum, 32, 64);
+            if (__any(corr != 1.f && l_run != 0.f)) {  // (most tiles move no row's maximum: the sums keep their scale)
+#pragma unroll
+                for (int v = 0; v < VT; ++v)
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) o[v][r] *= corr;
+            }
+            l_run = l_run * corr + psum;
+            m_run = m_new;
+#pragma unroll
+            for (int nn = 0; nn < NN; ++nn) {
+                const uint32_t h0 = BF16::pack2(sc[nn][0], sc[nn][1]), h1 = BF16::pack2(sc[nn][2], sc[nn][3]);
+                const uint32_t l0 = BF16::pack2(sc[nn][0] - __uint_as_float(h0 << 16), sc[nn][1] - __uint_as_float(h0 & 0xffff0000u));
+                const uint32_t l1 = BF16::pack2(sc[nn][2] - __uint_as_float(h1 << 16), sc[nn][3] - __uint_as_float(h1 & 0xffff0000u));
+                const u32x4 pf{h0, h1, l0, l1};
+                const uint16_t *vr = vtr + 16 * (nb + nn) * RV;
+#pragma unroll
+                for (int v = 0; v < VT; ++v) {
+                    const u32x2 x = __builtin_bit_cast(u32x2, __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_v4s16 *)(vr + 16 * v)));
+                    o[v] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, u32x4{x[0], x[1], x[0], x[1]}), __builtin_bit_cast(bf16x8_t, pf), o[v], 0, 0, 0);
+                }
+            }
+        }
+    }
+    // four consecutive columns c .. c + 3 of this lane's row leave: times `mul`, the gate, as float32 or bfloat16 (n_splits 1), or as they are to the partial sums
+    const bool whole = (ldo & 3) == 0 && ((uintptr_t)out & 7) == 0;
+    const size_t pi = ((size_t)trow * H + head) * n_splits + split;
+    auto leave = [&](int c, f32x4 val, float mul) __attribute__((always_inline)) {
+        if (c >= vdim) return;
+        if (n_splits > 1) {
+            *reinterpret_cast<f32x4 *>(part_acc + pi * vdim + c) = val;
+            return;
+        }
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            val[r] *= mul;
+            if (gate) val[r] *= sigmoid_f(gate[(size_t)trow * ldg + (gate_per_head ? (size_t)head : (size_t)head * vdim + c + r)]);
+        }
+        if (out32) *reinterpret_cast<f32x4 *>(out32 + ((size_t)trow * H + head) * vdim + c) = val;
+        else {
+            uint16_t *dst = out + (size_t)trow * ldo + (size_t)head * vdim + c;
+            if (whole) store4<BF16>(dst, val);
+            else {
+#pragma unroll
+                for (int r = 0; r < 4; ++r) dst[r] = BF16::from_float(val[r]);
+            }
+        }
+    };
+    if constexpr (WSPLIT) {  // four waves, four partial sets of the same 16 rows: through LDS (the tiles are no longer needed); wave w finishes the value tiles w, w + 4, ...
+        float *xm = smem, *xl = smem + 64, *xo = smem + 128;  // [4][16], [4][16], [4][VT][64][4]
+        __syncthreads();
+        if (g4 == 0) {
+            xm[wave * 16 + col] = m_run;
+            xl[wave * 16 + col] = l_run;
+        }
+#pragma unroll
+        for (int v = 0; v < VT; ++v) *reinterpret_cast<f32x4 *>(xo + ((size_t)(wave * VT + v) * 64 + lane) * 4) = o[v];
+        __syncthreads();
+        float M = -INFINITY, L = 0.f, f[4];
+#pragma unroll
+        for (int w = 0; w < 4; ++w) M = fmaxf(M, xm[w * 16 + col]);
+#pragma unroll
+        for (int w = 0; w < 4; ++w) {
+            const float mw = xm[w * 16 + col];
+            f[w] = (mw == -INFINITY) ? 0.f : __expf(mw - M);
+            L += xl[w * 16 + col] * f[w];
+        }
+        if (!row_ok) return;
+        const float invl = L > 0.f ? out_scale / L : 0.f;
+        for (int v = wave; v < VT; v += 4) {
+            f32x4 s{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int w = 0; w < 4; ++w) {
+                const f32x4 ow = *reinterpret_cast<const f32x4 *>(xo + ((size_t)(w * VT + v) * 64 + lane) * 4);
+#pragma unroll
+                for (int r = 0; r < 4; ++r) s[r] += ow[r] * f[w];
+            }
+            leave(16 * v + 4 * g4, s, invl);
+        }
+        if (n_splits > 1 && wave == 0 && g4 == 0) {
+            part_ml[2 * pi] = M;
+            part_ml[2 * pi + 1] = L;
+        }
+        return;
+    }
+    if (!row_ok) return;
+    const float invl = l_run > 0.f ? out_scale / l_run : 0.f;
+#pragma unroll
+    for (int v = 0; v < VT; ++v) leave(16 * v + 4 * g4, o[v], invl);
+    if (n_splits > 1 && g4 == 0) {
+        part_ml[2 * pi] = m_run;
+        part_ml[2 * pi + 1] = l_run;
     }
 }
 
